@@ -5,8 +5,9 @@ experts), on a float32 residual stream.
 The stream's rule is a parameter of the configuration: the norm on the sublayer's OUTPUT (``out_norm``:
 x <- x + layer_norm(sublayer(x))), AFTER the sum (``post_norm``: x <- rms_norm(alpha x + sublayer(x))), on the
 sublayer's INPUT (``pre_norm``: x <- x + sublayer(rms_norm(x))) or on both sides (``sandwich``:
-x <- x + norm_b(sublayer(norm_a(x))), RMS norms over ``norm_groups`` equal parts of the row).  A range of layers may
-repeat, back to back, on shared weights (``loop``), or single layers may name another layer whose weights they use
+x <- x + norm_b(sublayer(norm_a(x))), RMS norms over ``norm_groups`` equal parts of the row).  A pre-norm stream may
+use Dynamic Tanh in place of the RMS norm, scale what it adds, gate every sublayer's result by a projection of what
+the sublayer read, and hand on weighted sums of all earlier layers' results.  A range of layers may repeat, back to back, on shared weights (``loop``), or single layers may name another layer whose weights they use
 (``share``); every run has its own pages and state.
 
 This module is the design-independent part: the mixer and feed-forward kinds with their sizes and constants as
@@ -47,7 +48,10 @@ class MLSTMSpec:
 @dataclass
 class LatentAttentionSpec:
     """Attention whose keys and values are up-projections of one cached low-rank latent per token, plus a rotated key
-    part shared by all heads; sigmoid output gate per head."""
+    part shared by all heads; through a sliding window or over the whole prefix; a sigmoid output gate (one number per
+    head, or with ``gate_wide`` one per output column).  ``rope_interleaved``: neighbouring columns form the rotated
+    pairs (else column i pairs with i + rope_dims / 2).  ``two_term``: on the matrix cores the softmax weights enter
+    the weighted sum as two bfloat16 terms each."""
     heads: int
     dim: int        # unrotated query / key columns per head
     rot_dim: int    # rotated columns per head (the shared rotated key has as many)
@@ -56,6 +60,10 @@ class LatentAttentionSpec:
     scale: float
     rope_base: float
     rope_dims: int  # leading columns of the rotated part that are actually rotated
+    window: int = 0            # > 0: only the last ``window`` positions (the query's own included) are visible
+    rope_interleaved: bool = False
+    gate_wide: bool = False
+    two_term: bool = False
     kind: str = "latent_attention"
 
 
@@ -64,6 +72,14 @@ class DenseFFSpec:
     ff: int
     act: int = hops.ACT_RELU2
     kind: str = "dense"
+
+
+@dataclass
+class PolyFFSpec:
+    """Dense feed-forward with the PolyNorm activation a N(z) + b N(z^2) + c N(z^3) + e, N = division by the row's root
+    mean square over the ``ff`` values."""
+    ff: int
+    kind: str = "poly"
 
 
 @dataclass
@@ -110,12 +126,15 @@ class WindowAttentionSpec:
     v_from_k: bool = False   # values = the keys as projected
     v_rot: bool = False      # values rotated by their position, outputs turned back
     gate_wide: bool = False  # the sigmoid output gate has heads * vdim rows instead of heads
+    sink_fixed: Optional[float] = None  # with ``sink``: every head's sink score is this constant (no weights)
+    bias_o: bool = False     # the output projection adds a bias
     kind: str = "window_attention"
 
     def params(self, d: int) -> int:
         qkv = self.heads * self.dim + self.kv_heads * (self.dim + (0 if self.v_from_k else self.vdim))
         gate = self.heads * (self.vdim if self.gate_wide else 1) * self.gate
-        return d * (qkv + gate) + 2 * self.dim * self.qk_norm + self.heads * self.sink + \
+        return d * (qkv + gate) + 2 * self.dim * self.qk_norm + \
+            (self.heads if self.sink and self.sink_fixed is None else 0) + self.bias_o * d + \
             (1 if self.v_mix and not self.v_mix_first else 0) + \
             self.heads * self.vdim * d + qkv * self.bias
 
@@ -292,6 +311,11 @@ class HybridConfig:
     residual_alpha: float = 1.0
     tied_head: bool = False        # the logits come from the embedding table
     loop: Optional[tuple] = None   # (start, stop, times): layers [start, stop) run ``times`` times, back to back
+    norm: str = "rms"              # pre_norm: the stream's norms, "rms" or "tanh" (Dynamic Tanh: tanh(alpha x) w + b)
+    residual_mult: float = 1.0     # pre_norm: x <- x + residual_mult * sublayer(norm(x))
+    residual_gate: bool = False    # pre_norm: a sublayer's result times sigmoid(W h + b), h what the sublayer read
+    depth_average: bool = False    # pre_norm: after layer i the stream is sum_j dwa_i[j] X_j over the embedding output
+    #                                X_0 and the layers' own results X_1 .. X_(i+1)
     token_side: int = 0            # > 0: after every layer's feed-forward a gated, RMS-normed projection of this many
     #                                columns of a second embedding table (layer i owns columns [i dim, (i+1) dim))
 
@@ -312,7 +336,7 @@ class HybridConfig:
 
     def param_count(self) -> int:
         d = self.hidden_size
-        n = (1 if self.tied_head else 2) * self.vocab_size * d + d
+        n = (1 if self.tied_head else 2) * self.vocab_size * d + d + (d + 1 if self.norm == "tanh" else 0)
         own = set(self.runs)
         for i, l in enumerate(self.layers):
             if i not in own:
@@ -323,13 +347,19 @@ class HybridConfig:
             elif m.kind == "mlstm":
                 n += d * (2 * m.heads * m.dim + 2 * m.heads * m.vdim) + 2 * m.heads * (d + 1) + m.heads * m.vdim * (d + 1)
             else:
-                n += d * (m.heads * (m.dim + m.rot_dim) + m.kv_rank + m.rot_dim + m.heads) + m.kv_rank
+                gates = m.heads * (m.vdim if m.gate_wide else 1)
+                n += d * (m.heads * (m.dim + m.rot_dim) + m.kv_rank + m.rot_dim + gates) + m.kv_rank
                 n += m.kv_rank * m.heads * (m.dim + m.vdim) + m.heads * m.vdim * d
-            n += d * (2 if self.residual == "sandwich" else 1)
+            sub = d * (2 if self.residual == "sandwich" else 1)    # what every sublayer carries beside its own weights
+            if self.norm == "tanh":
+                sub += d + 1
+            if self.residual_gate:
+                sub += d * (d + 1)
+            n += sub + (i + 2 if self.depth_average else 0)
             if l.ff is not None:
                 f = l.ff
-                n += d * (2 if self.residual == "sandwich" else 1)
-                n += {"dense": lambda: 2 * d * f.ff, "glu": lambda: 3 * d * f.ff,
+                n += sub
+                n += {"dense": lambda: 2 * d * f.ff, "poly": lambda: 2 * d * f.ff + 4, "glu": lambda: 3 * d * f.ff,
                       "moe": lambda: (f.experts * f.ff + f.shared_ff) * 2 * d + (f.experts + f.identity) * (d + f.correction),
                       "moe_glu": lambda: f.experts * (3 * d * f.ff + d + 1),
                       "moe_group_glu": lambda: f.experts * (3 * d * f.ff + d) + (
@@ -442,6 +472,9 @@ class HybridLayerWeights:
     side: dict = field(default_factory=dict)   # the per-layer token input: w_gate, w_proj, norm, col0
     norm1b: Optional[torch.Tensor] = None      # sandwich stream: the norms on the sublayers' outputs
     norm2b: Optional[torch.Tensor] = None
+    gate1: dict = field(default_factory=dict)  # residual gates: b (float32 bias) and, when the sublayer's own first
+    gate2: dict = field(default_factory=dict)  # projection does not carry the gate's rows, w
+    dwa: Optional[torch.Tensor] = None         # depth average: float32 [layer + 2]
 
 
 @dataclass
@@ -458,12 +491,22 @@ class HybridWeights:
             if t is not None:
                 n += t.numel() * t.element_size()
         for l in {id(l): l for l in self.layers}.values():   # a layer that runs on another's weights counts once
-            for t in (l.norm1, l.norm2, l.norm1b, l.norm2b, *l.mix.values(), *l.ff.values(), *l.side.values()):
+            for t in (l.norm1, l.norm2, l.norm1b, l.norm2b, l.dwa, *l.mix.values(), *l.ff.values(), *l.side.values(),
+                      *l.gate1.values(), *l.gate2.values()):
                 if isinstance(t, torch.Tensor):
                     n += t.numel() * t.element_size()
                 elif isinstance(t, dict):
                     n += sum(v.numel() * v.element_size() for v in t.values() if isinstance(v, torch.Tensor))
         return n
+
+
+def _in_proj(rows: list, t: dict, out: dict, key: str, cast) -> None:
+    """out[key] = the sublayer's first projection: ``rows`` stacked and, when t holds "rg" (a residual gate's rows, which
+    read the same input), those last, from column out["rg_off"] on."""
+    if "rg" in t:
+        out["rg_off"] = sum(r.shape[0] for r in rows)
+        rows = rows + [t["rg"]]
+    out[key] = cast(rows[0] if len(rows) == 1 else torch.cat(rows, 0))
 
 
 def pack_mlstm(spec: MLSTMSpec, t: dict, device, act_dtype) -> dict:
@@ -476,19 +519,32 @@ def pack_mlstm(spec: MLSTMSpec, t: dict, device, act_dtype) -> dict:
 
 
 def pack_latent(spec: LatentAttentionSpec, t: dict, device, act_dtype) -> dict:
-    """t: q, dkv, dkv.norm, uk, uv, g, o.  The per-head up-projections are kept as [H, D, rank] and [H, Dv, rank]:
-    keys are never materialised (the query is carried into the latent space instead) and the value up-projection
-    is applied to the attention's latent-space output."""
+    """t: q, dkv, dkv.norm, uk, uv, g, o.  q | dkv (| g with a gate per output column) are one projection; per-head
+    gate rows are a few-row float32-output projection.  The per-head up-projections are kept as [H, rank, D] and
+    [H, Dv, rank]: keys are never materialised (the query is carried into the latent space instead) and the value
+    up-projection is applied to the attention's latent-space output."""
     a = lambda x: x.to(device=device, dtype=act_dtype).contiguous()  # noqa: E731
     f = lambda x: x.to(device=device, dtype=torch.float32).contiguous()  # noqa: E731
-    return dict(w_q=a(t["q"]), w_dkv=a(t["dkv"]), dkv_norm=f(t["dkv.norm"]), w_g=a(t["g"]), w_o=a(t["o"]),
-                w_uk=a(t["uk"].view(spec.heads, spec.dim, spec.kv_rank)),
-                w_uv=a(t["uv"].view(spec.heads, spec.vdim, spec.kv_rank)))
+    out = dict(dkv_norm=f(t["dkv.norm"]), w_o=a(t["o"]),
+               w_uk=a(t["uk"].view(spec.heads, spec.dim, spec.kv_rank).transpose(1, 2)),
+               w_uv=a(t["uv"].view(spec.heads, spec.vdim, spec.kv_rank)))
+    _in_proj([t["q"], t["dkv"]] + ([t["g"]] if spec.gate_wide else []), t, out, "w_in", a)
+    if not spec.gate_wide:
+        out["w_g"] = a(t["g"])
+    return out
 
 
 def pack_dense(spec: DenseFFSpec, t: dict, device, act_dtype) -> dict:
     a = lambda x: x.to(device=device, dtype=act_dtype).contiguous()  # noqa: E731
     return dict(w_up=a(t["up"]), w_down=a(t["down"]))
+
+
+def pack_poly(spec: PolyFFSpec, t: dict, device, act_dtype) -> dict:
+    """t: up, down, act (a, b, c, e)."""
+    a = lambda x: x.to(device=device, dtype=act_dtype).contiguous()  # noqa: E731
+    out = dict(w_down=a(t["down"]), act=t["act"].to(device=device, dtype=torch.float32).contiguous())
+    _in_proj([t["up"]], t, out, "w_up", a)
+    return out
 
 
 def pack_moe(spec: MoEFFSpec, t: dict, device, act_dtype) -> dict:
@@ -511,15 +567,19 @@ def pack_window_attention(spec: WindowAttentionSpec, t: dict, device, act_dtype)
     a = lambda x: x.to(device=device, dtype=act_dtype).contiguous()  # noqa: E731
     f = lambda x: x.to(device=device, dtype=torch.float32).contiguous()  # noqa: E731
     rows = [t["q"], t["k"]] + ([] if spec.v_from_k else [t["v"]]) + ([t["g"]] if spec.gate and spec.gate_wide else [])
-    out = dict(w_qkv=a(torch.cat(rows, 0)), w_o=a(t["o"]))
+    out = dict(w_o=a(t["o"]))
+    _in_proj(rows, t, out, "w_qkv", a)
     if spec.qk_norm:
         out.update(q_norm=f(t["q.norm"]), k_norm=f(t["k.norm"]))
     if spec.sink:
-        out["sink"] = f(t["sink"])
+        out["sink"] = f(t["sink"] if spec.sink_fixed is None else torch.full((spec.heads,), float(spec.sink_fixed)))
     if spec.gate and not spec.gate_wide:
         out["w_g"] = a(t["g"])
     if spec.bias:
-        out["b_qkv"] = a(torch.cat([t["q.b"], t["k.b"], t["v.b"]], 0))
+        rest = out["w_qkv"].shape[0] - spec.heads * spec.dim - spec.kv_heads * (spec.dim + spec.vdim)  # gate rows: none
+        out["b_qkv"] = a(torch.cat([t["q.b"], t["k.b"], t["v.b"], torch.zeros(rest, dtype=t["q.b"].dtype)], 0))
+    if spec.bias_o:
+        out["b_o"] = a(t["o.b"])
     if spec.v_mix and not spec.v_mix_first:
         out["vmix"] = f(t["vmix"]).reshape(1)
     return out
@@ -566,8 +626,10 @@ def pack_gla(spec: GLASpec, t: dict, device, act_dtype) -> dict:
     float32 outputs (a1 through the few-row projection, a2 as a float32 matrix)."""
     a = lambda x: x.to(device=device, dtype=act_dtype).contiguous()  # noqa: E731
     f = lambda x: x.to(device=device, dtype=torch.float32).contiguous()  # noqa: E731
-    return dict(w_proj=a(torch.cat([t["q"], t["k"], t["v"], t["g"]], 0)), w_a1=a(t["a1"]), w_a2t=f(t["a2"].float().t()),
-                b_a2=f(t["a2.b"]), norm=f(t["norm"].float().repeat(spec.heads)), w_o=a(t["o"]))
+    out = dict(w_a1=a(t["a1"]), w_a2t=f(t["a2"].float().t()), b_a2=f(t["a2.b"]),
+               norm=f(t["norm"].float().repeat(spec.heads)), w_o=a(t["o"]))
+    _in_proj([t["q"], t["k"], t["v"], t["g"]], t, out, "w_proj", a)
+    return out
 
 
 def pack_retention(spec: RetentionSpec, t: dict, device, act_dtype) -> dict:
@@ -685,23 +747,36 @@ def mix_mlstm(model, li: int, spec: MLSTMSpec, w: dict, h, meta: StepMeta, cache
     return hops.matmul(y, w["w_o"])
 
 
+@dataclass
+class GatedOut:
+    """A sublayer's output together with the pre-activations of its residual gate, which its first projection carried:
+    columns off .. off + d of src."""
+    y: torch.Tensor
+    src: torch.Tensor
+    off: int
+
+
+def _with_gate(y, proj, w: dict):
+    return GatedOut(y, proj, w["rg_off"]) if "rg_off" in w else y
+
+
 def mix_latent_attention(model, li: int, spec: LatentAttentionSpec, w: dict, h, meta: StepMeta, cache: HybridCache):
     T = h.shape[0]
     H, D, R, rank = spec.heads, spec.dim, spec.rot_dim, spec.kv_rank
-    q = hops.matmul(h, w["w_q"]).view(T, H, D + R)
-    dkv = hops.matmul(h, w["w_dkv"])
-    gate = hops.rowdot(h, w["w_g"])
-    hops.latent_prep(q, dkv, meta.pos, meta.tok_seq, meta.block_table, w["dkv_norm"], model.cfg.norm_eps,
-                     model.rope[li], spec.rope_dims, rank, cache.lat[li])
+    nq, nkv = H * (D + R), rank + R
+    proj = hops.matmul(h, w["w_in"])    # q | dkv (| one gate per output column)
+    q = proj[:, :nq].view(T, H, D + R)
+    gate = None if spec.gate_wide else hops.rowdot(h, w["w_g"])
     # the query goes into the latent space (q_u W_uk per head), so a key is the cached row itself; the output
     # comes back through W_uv per head
     qa = torch.empty(T, H, rank + R, device=h.device, dtype=h.dtype)
-    qa[:, :, :rank] = torch.bmm(q[:, :, :D].transpose(0, 1), w["w_uk"]).transpose(0, 1)
-    qa[:, :, rank:] = q[:, :, D:]
+    hops.latent_prep(q, proj[:, nq:nq + nkv], meta.pos, meta.tok_seq, meta.block_table, w["dkv_norm"], model.cfg.norm_eps,
+                     model.rope.get(li), spec.rope_dims, rank, cache.lat[li], qa, spec.rope_interleaved)
+    hops.head_matmul(q[:, :, :D], w["w_uk"], qa[:, :, :rank])
     oa = hops.latent_attention(qa, cache.lat[li], meta.block_table, meta.q_start, meta.pos, gate, spec.scale, rank,
-                               model.act_dtype, meta.max_q)
-    ov = torch.bmm(oa.transpose(0, 1), w["w_uv"].transpose(1, 2)).transpose(0, 1).reshape(T, H * spec.vdim)
-    return hops.matmul(ov, w["w_o"])
+                               model.act_dtype, meta.max_q, spec.window, spec.two_term)
+    ov = hops.head_matmul(oa, w["w_uv"], None, proj if spec.gate_wide else None, nq + nkv)
+    return _with_gate(hops.matmul(ov.view(T, H * spec.vdim), w["w_o"]), proj, w)
 
 
 def mix_window_attention(model, li, spec: WindowAttentionSpec, w: dict, h, meta: StepMeta, cache: HybridCache):
@@ -724,7 +799,7 @@ def mix_window_attention(model, li, spec: WindowAttentionSpec, w: dict, h, meta:
                               gate, spec.scale, spec.window, spec.keep_first, H, model.act_dtype, meta.max_q,
                               spec.chunk, spec.pool if pooled else 0, cache.kp.get(li), cache.vp.get(li), v_tab,
                               (H + G) * D + G * Dv if spec.gate and spec.gate_wide else -1)
-    return hops.matmul(o, w["w_o"])
+    return _with_gate(hops.matmul(o, w["w_o"], w.get("b_o")), qkv, w)
 
 
 def mix_retention(model, li, spec: RetentionSpec, w: dict, h, meta: StepMeta, cache: HybridCache):
@@ -798,8 +873,8 @@ def mix_gla(model, li: int, spec: GLASpec, w: dict, h, meta: StepMeta, cache: Hy
     decay = hops.decay_pow(z, 1.0 / spec.tau)
     o = hops.linear_scan(proj, 0, H * D, 2 * H * D, None, None, D ** -0.5, decay, None, meta.q_start, meta.pos0,
                          meta.slots, cache.S[li], H, H, D, Dv)
-    return hops.matmul(hops.head_norm_gate(o, proj, 2 * H * D + H * Dv, w["norm"], model.cfg.norm_eps, True,
-                                           model.act_dtype), w["w_o"])
+    o = hops.head_norm_gate(o, proj, 2 * H * D + H * Dv, w["norm"], model.cfg.norm_eps, True, model.act_dtype)
+    return _with_gate(hops.matmul(o, w["w_o"]), proj, w)
 
 
 def ff_glu(model, spec: GluFFSpec, w: dict, h):
@@ -830,6 +905,12 @@ def ff_dense(model, spec: DenseFFSpec, w: dict, h):
     return hops.matmul(hops.act_inplace(hops.matmul(h, w["w_up"]), spec.act), w["w_down"])
 
 
+def ff_poly(model, spec: PolyFFSpec, w: dict, h):
+    z = hops.matmul(h, w["w_up"])
+    return _with_gate(hops.matmul(hops.poly_norm(z, spec.ff, w["act"], model.cfg.norm_eps, model.act_dtype), w["w_down"]),
+                      z, w)
+
+
 def ff_moe(model, spec: MoEFFSpec, w: dict, h):
     """Returns the routed experts' sum and, with a shared expert, (sum, shared output): the stream's join adds both."""
     idx, wt = hops.moe_route(h, w["w_router"], w["correction"], spec.top)
@@ -844,7 +925,7 @@ MIXERS = {"mlstm": (mix_mlstm, pack_mlstm), "latent_attention": (mix_latent_atte
           "delta_rule": (mix_delta_rule, pack_delta_rule), "gla": (mix_gla, pack_gla),
           "mamba2": (mix_mamba2, pack_mamba2), "rglru": (mix_rglru, pack_rglru),
           "retention": (mix_retention, pack_retention), "parallel": (mix_parallel, pack_parallel)}
-FEED_FORWARDS = {"dense": (ff_dense, pack_dense), "moe": (ff_moe, pack_moe), "glu": (ff_glu, pack_glu),
+FEED_FORWARDS = {"dense": (ff_dense, pack_dense), "poly": (ff_poly, pack_poly), "moe": (ff_moe, pack_moe), "glu": (ff_glu, pack_glu),
                  "moe_glu": (ff_moe_glu, pack_moe_glu), "moe_group_glu": (ff_moe_group_glu, pack_moe_group_glu)}
 RECURRENT_MIXERS = ("mlstm", "delta_rule", "gla", "mamba2", "rglru", "retention")
 
@@ -908,6 +989,14 @@ class HybridDecoder:
             raise ValueError(f"unknown residual rule {cfg.residual!r}")
         if cfg.token_side and cfg.residual != "pre_norm":
             raise ValueError("the per-layer token input is part of the pre-norm stream's join")
+        if cfg.norm not in ("rms", "tanh"):
+            raise ValueError(f"unknown norm {cfg.norm!r}")
+        self.gated_stream = cfg.norm == "tanh" or cfg.residual_gate or cfg.depth_average or cfg.residual_mult != 1.0
+        if self.gated_stream and (cfg.residual != "pre_norm" or cfg.token_side):
+            raise ValueError("Dynamic Tanh norms, a residual multiplier, residual gates and depth averages belong to the "
+                             "pre-norm stream, without a per-layer token input")
+        if cfg.depth_average and (cfg.loop or cfg.share is not None):
+            raise ValueError("a depth average weighs the layers' results one by one: layers may not repeat")
 
     # ---- what the engine calls --------------------------------------------------------------------------------
     def make_cache(self, num_blocks: int, block_size: int, slots: int, kv_dtype: str = "bf16", k_scale: float = 1.0,
@@ -968,7 +1057,9 @@ class HybridDecoder:
         cfg, w, at = self.cfg, self.w, self.act_dtype
         meta = self._meta(sb)
         x, h = hops.embed_rows(meta.ids, w.embed, at, cfg.embed_scale, cfg.residual not in ("pre_norm", "sandwich"))
-        if cfg.residual == "pre_norm":
+        if self.gated_stream:
+            self._forward_gated(x, meta, cache)
+        elif cfg.residual == "pre_norm":
             self._forward_pre_norm(x, meta, cache)
         elif cfg.residual == "sandwich":
             self._forward_sandwich(x, meta, cache)
@@ -985,6 +1076,8 @@ class HybridDecoder:
         xs = x.index_select(0, meta.last_idx)
         if cfg.residual == "out_norm":
             xn = hops.layer_norm(xs, w.final_norm, cfg.norm_eps, at)
+        elif cfg.norm == "tanh":
+            xn = hops.dyn_tanh(xs, w.final_norm, at)
         else:
             xn = hops.rms_norm(xs, w.final_norm, cfg.norm_eps, at, cfg.norm_groups if cfg.residual == "sandwich" else 1)
         logits = hops.matmul(xn, w.head).float()
@@ -1018,6 +1111,43 @@ class HybridDecoder:
                                       emit=not last)
             else:
                 h = hops.add_rms_norm(y, x, nxt, eps, at, y2, g2, emit=not last)
+            if self.layer_tap is not None:
+                self.layer_tap(ri, x)
+
+    def _forward_gated(self, x, meta: StepMeta, cache: HybridCache) -> None:
+        """x <- x + m g1 * mixer(h), h = norm1(x); x <- x + m g2 * ff(h), h = norm2(x); then, with a depth average,
+        x <- sum_j dwa[j] X_j over the embedding output and the layers' own results so far.  g1, g2: sigmoid of a
+        projection of h (its rows ride in the sublayer's own first projection).  One join kernel per sublayer gates,
+        scales and adds the sublayer's output, averages at a layer's end and emits the next norm."""
+        cfg, w, at = self.cfg, self.w, self.act_dtype
+        runs, hist = cfg.runs, None
+        if cfg.depth_average and runs:   # X_0 .. X_(last - 1): the last layer's own result is needed by nobody else
+            hist = torch.empty(len(runs), *x.shape, device=x.device, dtype=torch.float32)
+            hist[0].copy_(x)
+        tanh = cfg.norm == "tanh"
+        norm = lambda wn: hops.dyn_tanh(x, wn, at) if tanh else hops.rms_norm(x, wn, cfg.norm_eps, at)  # noqa: E731
+
+        def join(out, h, gate, wn, ri, dwa):
+            if isinstance(out, (tuple, PairOut)):
+                raise NotImplementedError("a sublayer with a separate part on a gated pre-norm stream")
+            y, src, off = (out.y, out.src, out.off) if isinstance(out, GatedOut) else (out, None, -1)
+            if cfg.residual_gate and src is None:
+                src, off = hops.matmul(h, gate["w"]), 0
+            hn = hops.gated_join(y, x, src, off, gate.get("b"), cfg.residual_mult, wn if tanh else None, at, hist, ri, dwa,
+                                 tanh and wn is not None)
+            return hn if tanh or wn is None else norm(wn)
+
+        h = norm(w.layers[runs[0]].norm1) if runs else None
+        for ri, li in enumerate(runs):
+            spec, lw = cfg.layers[li], w.layers[li]
+            nxt = w.layers[runs[ri + 1]].norm1 if ri + 1 < len(runs) else None   # the last run emits nothing
+            y = MIXERS[spec.mixer.kind][0](self, ri, spec.mixer, lw.mix, h, meta, cache)
+            if spec.ff is not None:
+                h = join(y, h, lw.gate1, lw.norm2, ri, None)
+                y = FEED_FORWARDS[spec.ff.kind][0](self, spec.ff, lw.ff, h)
+                h = join(y, h, lw.gate2, nxt, ri, lw.dwa)
+            else:
+                h = join(y, h, lw.gate1, nxt, ri, lw.dwa)
             if self.layer_tap is not None:
                 self.layer_tap(ri, x)
 

@@ -191,6 +191,29 @@ def _vogerax_presets():
     return list(vogerax.PRESETS)
 
 
+def _lalasun_build(name, device, tp, seed, is_path, max_position, weight_dtype, dtype):
+    from . import lalasun
+
+    if tp.world > 1:
+        raise NotImplementedError("Lalasun runs on full-weight ranks (data-parallel replicas)")
+    if weight_dtype != "bf16":
+        raise NotImplementedError("Lalasun weights are served in the activation dtype (no fp8 projections)")
+    return lalasun.build(name, device, seed, DTYPES[dtype], max_position)
+
+
+def _lalasun_is_checkpoint(path: str) -> bool:
+    from . import lalasun
+
+    return lalasun.is_checkpoint(path)
+
+
+def _lalasun_presets():
+    from . import lalasun
+
+    return list(lalasun.PRESETS)
+
+
+register(Family("lalasun", _lalasun_presets, _lalasun_is_checkpoint, _lalasun_build, ("bf16", "fp32")))
 register(Family("vogerax", _vogerax_presets, _vogerax_is_checkpoint, _vogerax_build, ("bf16", "fp32")))
 register(Family("tugovik", _tugovik_presets, _tugovik_is_checkpoint, _tugovik_build, ("bf16", "fp32")))
 register(Family("kalesun", _kalesun_presets, _kalesun_is_checkpoint, _kalesun_build, ("bf16", "fp32")))

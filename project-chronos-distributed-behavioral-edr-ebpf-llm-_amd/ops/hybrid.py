@@ -109,18 +109,36 @@ def mlstm_out(o, proj, g_off: int, norm_w, eps: float, act_dtype):
     return ref.mlstm_out(o, proj, g_off, norm_w, eps, act_dtype)
 
 
-def latent_prep(q, dkv, pos, tok_seq, block_table, w_norm, eps: float, cos_sin, dims: int, rank: int, cache) -> None:
+def latent_prep(q, dkv, pos, tok_seq, block_table, w_norm, eps: float, cos_sin, dims: int, rank: int, cache, qa=None,
+                interleaved: bool = False) -> None:
+    """``qa``: where the rotated query columns go (its last R columns per head; default: in place); ``interleaved``:
+    neighbouring columns form the rotated pairs.  q and dkv may be column ranges of one wider projection."""
     if _gpu(q):
-        _k().hy_latent_prep(q, dkv, pos, tok_seq, block_table, w_norm, eps, cos_sin, dims, rank, cache)
+        _k().hy_latent_prep(q, dkv, pos, tok_seq, block_table, w_norm, eps, cos_sin if dims else None, dims, rank, cache,
+                            qa, interleaved)
     else:
-        ref.latent_prep(q, dkv, pos, tok_seq, block_table, w_norm, eps, cos_sin, dims, rank, cache)
+        ref.latent_prep(q, dkv, pos, tok_seq, block_table, w_norm, eps, cos_sin, dims, rank, cache, qa, interleaved)
 
 
-def latent_attention(qa, cache, block_table, q_start, pos, gate, scale: float, rank: int, act_dtype, max_q: int):
-    """``max_q``: the most tokens any sequence brings in this step (sizes the launch grid)."""
+def head_matmul(a, w, out=None, gate_src=None, g_off: int = -1):
+    """Per-head products a[t, h] @ w[h].T (a [T, H, K], w [H, N, K]) into ``out`` [T, H, N] (a view with wider rows is
+    fine), optionally times sigmoid of H N gate columns."""
+    if _gpu(a):
+        if out is None:
+            out = torch.empty(a.shape[0], a.shape[1], w.shape[1], device=a.device, dtype=a.dtype)
+        _k().hy_head_matmul(a, w, out, gate_src, g_off)
+        return out
+    return ref.head_matmul(a, w, out, gate_src, g_off)
+
+
+def latent_attention(qa, cache, block_table, q_start, pos, gate, scale: float, rank: int, act_dtype, max_q: int,
+                     window: int = 0, two_term: bool = False):
+    """``max_q``: the most tokens any sequence brings in this step (sizes the launch grid).  ``window`` > 0: a query
+    sees only the last ``window`` positions.  ``two_term``: the matrix-core kernel feeds every softmax weight as a sum
+    of two bfloat16 terms (float32 weights to about 2^-17)."""
     if _gpu(qa):
-        return _k().hy_latent_attention(qa, cache, block_table, q_start, pos, gate, scale, rank, max_q)
-    return ref.latent_attention(qa, cache, block_table, q_start, pos, gate, scale, rank, act_dtype)
+        return _k().hy_latent_attention(qa, cache, block_table, q_start, pos, gate, scale, rank, max_q, window, two_term)
+    return ref.latent_attention(qa, cache, block_table, q_start, pos, gate, scale, rank, act_dtype, window)
 
 
 def moe_route(h, w_router, correction, top: int):
@@ -348,3 +366,32 @@ def rotate_qk(proj, q_off: int, k_off: int, HQ: int, HK: int, D: int, dims: int,
         _k().hy_rotate_qk(proj, q_off, k_off, HQ, HK, D, dims if cos_sin is not None else 0, cos_sin, pos, q_mul, k_mul)
     else:
         ref.rotate_qk(proj, q_off, k_off, HQ, HK, D, dims, cos_sin, pos, q_mul, k_mul)
+
+
+# ---- pre-norm stream with Dynamic Tanh norms, gated residuals and depth averages; PolyNorm ---------------------------
+
+
+def dyn_tanh(x, wba, act_dtype):
+    """tanh(alpha x) * w + b of the float32 stream; wba = w | b | alpha."""
+    if _gpu(x):
+        return _k().hy_dyn_tanh(x, wba, _f32(act_dtype))
+    return ref.dyn_tanh(x, wba, act_dtype)
+
+
+def gated_join(y, x, gate_src, g_off: int, gate_b, mult: float, wba, act_dtype, hist=None, run: int = -1, dwa=None,
+               emit: bool = True):
+    """x (float32 residual, in place) <- x + mult * sigmoid(gate) * y and, with ``dwa``, the weighted sum of that and
+    the earlier layers' results in ``hist`` (where the layer's own result is kept).  Returns dyn_tanh(x, wba), or None
+    when ``emit`` is off."""
+    if _gpu(x):
+        h = _k().hy_gated_join(y, x, gate_src, g_off, gate_b, mult, wba if emit else None, hist if dwa is not None else None,
+                               run, dwa)
+        return h if emit else None
+    return ref.gated_join(y, x, gate_src, g_off, gate_b, mult, wba, act_dtype, hist, run, dwa, emit)
+
+
+def poly_norm(z, F: int, abce, eps: float, act_dtype):
+    """The PolyNorm activation of the first F columns of z [T, >= F]; returns [T, F]."""
+    if _gpu(z):
+        return _k().hy_poly_norm(z, F, abce, eps)
+    return ref.poly_norm(z, F, abce, eps, act_dtype)

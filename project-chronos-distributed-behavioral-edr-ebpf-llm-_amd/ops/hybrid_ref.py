@@ -101,42 +101,60 @@ def mlstm_out(o, proj, g_off, norm_w, eps, act_dtype):
     return y.to(act_dtype)
 
 
-def rotate_half_rows(x, cos_sin, pos, dims):
-    """Rotary position on the first ``dims`` entries of the last axis (entry i pairs with i + dims/2); cos_sin
-    [P, dims]: cos | sin of position x frequency, float32."""
+def rotate_half_rows(x, cos_sin, pos, dims, interleaved=False):
+    """Rotary position on the first ``dims`` entries of the last axis (entry i pairs with i + dims/2, or with
+    ``interleaved`` entry 2i with 2i + 1); cos_sin [P, dims]: cos | sin of position x frequency, float32."""
     half = dims // 2
     cs = cos_sin[pos.long()]
     shape = [x.shape[0]] + [1] * (x.dim() - 2) + [half]
     c, s = cs[:, :half].view(shape), cs[:, half:].view(shape)
-    u, v = x[..., :half].float(), x[..., half:dims].float()
+    iu, iv = (slice(0, dims, 2), slice(1, dims, 2)) if interleaved else (slice(0, half), slice(half, dims))
+    u, v = x[..., iu].float(), x[..., iv].float()
     out = x.float().clone()
-    out[..., :half] = u * c - v * s
-    out[..., half:dims] = v * c + u * s
+    out[..., iu] = u * c - v * s
+    out[..., iv] = v * c + u * s
     return out
 
 
-def latent_prep(q, dkv, pos, tok_seq, block_table, w_norm, eps, cos_sin, dims, rank, cache):
+def latent_prep(q, dkv, pos, tok_seq, block_table, w_norm, eps, cos_sin, dims, rank, cache, qa=None, interleaved=False):
     """Latent-attention cache write and query rotation.  dkv [T, rank + R]: the first rank columns are RMS-normed
-    (times w_norm) into the latent, the last R rotated; both are written to cache [NB, BS, rank + R] at the token's
-    page and slot.  q [T, H, D + R]: the last R columns of every head are rotated in place."""
+    (times w_norm) into the latent, the last R rotated (on their leading ``dims`` columns; none with dims 0); both are
+    written to cache [NB, BS, rank + R] at the token's page and slot.  q [T, H, D + R] (a view whose rows may be part of
+    a wider projection, like dkv): the last R columns of every head are rotated, into the last R columns of qa
+    [T, H, rank + R] when that is given (q is then left as it is), else in place."""
     T = q.shape[0]
     R = dkv.shape[1] - rank
     D = q.shape[2] - R
     c = dkv[:, :rank].float()
     c = c * torch.rsqrt(c.pow(2).mean(-1, keepdim=True) + eps) * w_norm.float()
-    kr = rotate_half_rows(dkv[:, rank:], cos_sin, pos, dims)
-    row = torch.cat([c, kr], 1).to(cache.dtype)
+    rot = lambda x: rotate_half_rows(x, cos_sin, pos, dims, interleaved) if dims else x.float()  # noqa: E731
+    row = torch.cat([c, rot(dkv[:, rank:])], 1).to(cache.dtype)
     bs = cache.shape[1]
     blk = block_table[tok_seq.long(), (pos // bs).long()].long()
     cache[blk, (pos % bs).long()] = row
-    q[:, :, D:] = rotate_half_rows(q[:, :, D:], cos_sin, pos, dims).to(q.dtype)
+    (q[:, :, D:] if qa is None else qa[:, :, rank:]).copy_(rot(q[:, :, D:]).to(q.dtype))
 
 
-def latent_attention(qa, cache, block_table, q_start, pos, gate, scale, rank, act_dtype):
+def head_matmul(a, w, out=None, gate_src=None, g_off=-1):
+    """Every head's own small product: out[t, h] = a[t, h] @ w[h].T with a [T, H, K] and out [T, H, N] views whose rows
+    may be part of wider ones, w [H, N, K]; float32 accumulation.  With ``gate_src`` the result is multiplied element
+    by element with sigmoid of gate_src[:, g_off : g_off + H N]."""
+    T, H, _ = a.shape
+    N = w.shape[1]
+    y = torch.einsum("thk,hnk->thn", a.float(), w.float())
+    if gate_src is not None:
+        y = y * torch.sigmoid(gate_src[:, g_off:g_off + H * N].float()).view(T, H, N)
+    if out is None:
+        return y.to(a.dtype).contiguous()
+    out.copy_(y.to(out.dtype))
+    return out
+
+
+def latent_attention(qa, cache, block_table, q_start, pos, gate, scale, rank, act_dtype, window=0):
     """Causal softmax attention of H query heads over ONE shared key row per token: key = the cached row (rank + R
     columns), value = its first rank columns.  qa [T, H, rank + R]; token t of sequence b sits at pos[t] and sees the
-    cached rows 0..pos[t] of its sequence; gate f32 [T, H] or None: the output of head h is multiplied by
-    sigmoid(gate).  Returns [T, H, rank]."""
+    cached rows 0..pos[t] of its sequence (``window`` > 0: only the last ``window`` of them); gate f32 [T, H] or None:
+    the output of head h is multiplied by sigmoid(gate).  Returns [T, H, rank]."""
     T, H, DK = qa.shape
     out = torch.zeros(T, H, rank, dtype=torch.float32, device=qa.device)
     bs = cache.shape[1]
@@ -150,7 +168,10 @@ def latent_attention(qa, cache, block_table, q_start, pos, gate, scale, rank, ac
         nblk = (ctx + bs - 1) // bs
         keys = cache[block_table[b, :nblk].long()].reshape(nblk * bs, DK)[:ctx].float()
         sc = torch.einsum("thk,jk->thj", qa[t0:t1].float(), keys) * scale
-        mask = torch.arange(ctx, device=qa.device)[None, :] > p[:, None]
+        j = torch.arange(ctx, device=qa.device)[None, :]
+        mask = j > p[:, None]
+        if window:
+            mask = mask | (p[:, None] - j >= window)
         sc = sc.masked_fill(mask[:, None, :], float("-inf"))
         a = torch.softmax(sc, -1)
         out[t0:t1] = torch.einsum("thj,jr->thr", a, keys[:, :rank])
@@ -603,3 +624,43 @@ def rotate_qk(proj, q_off, k_off, HQ, HK, D, dims, cos_sin, pos, q_mul, k_mul):
         x = proj[:, off:off + n * D].view(T, n, D)
         xf = rotate_half_rows(x, cos_sin, pos, dims) if (cos_sin is not None and dims) else x.float()
         x.copy_((xf * mul).to(x.dtype))
+
+
+# ---- pre-norm stream with Dynamic Tanh norms, gated residuals and depth averages; PolyNorm ---------------------------
+
+
+def dyn_tanh(x, wba, act_dtype):
+    """Dynamic Tanh in place of a norm (no statistic): tanh(alpha x) * w + b; ``wba`` f32 [2 d + 1] = w | b | alpha."""
+    d = x.shape[-1]
+    w, b, alpha = wba[:d].float(), wba[d:2 * d].float(), wba[2 * d].float()
+    return (torch.tanh(alpha * x.float()) * w + b).to(act_dtype)
+
+
+def gated_join(y, x, gate_src, g_off, gate_b, mult, wba, act_dtype, hist=None, run=-1, dwa=None, emit=True):
+    """x (float32 residual, in place) <- x + mult * sigmoid(g) * y, g = gate_src[:, g_off : g_off + d] (+ gate_b); no
+    gate when gate_src is None.  With ``dwa`` (f32 [run + 2]) the updated rows X are then kept as hist[run + 1] (hist
+    f32 [runs, T, d]; hist[0] the embedding output; the last run's X is not kept) and the stream becomes
+    sum_j<=run dwa[j] hist[j] + dwa[run + 1] X.  Returns dyn_tanh(x, wba) in the activation dtype, or None when
+    ``emit`` is off."""
+    v = y.float()
+    if gate_src is not None:
+        g = gate_src[:, g_off:g_off + x.shape[1]].float()
+        v = v * torch.sigmoid(g if gate_b is None else g + gate_b.float())
+    x.add_(mult * v)
+    if dwa is not None:
+        acc = dwa[run + 1] * x
+        for j in range(run + 1):
+            acc = acc + dwa[j] * hist[j]
+        if run + 1 < hist.shape[0]:
+            hist[run + 1].copy_(x)
+        x.copy_(acc)
+    return dyn_tanh(x, wba, act_dtype) if emit else None
+
+
+def poly_norm(z, F, abce, eps, act_dtype):
+    """a N(z) + b N(z^2) + c N(z^3) + e on the first F columns of z, powers element by element, N = division by the
+    row's root mean square; ``abce`` f32 [4]."""
+    zf = z[:, :F].float()
+    n = lambda v: v * torch.rsqrt(v.pow(2).mean(-1, keepdim=True) + eps)  # noqa: E731
+    a, b, c, e = (abce[i].float() for i in range(4))
+    return (a * n(zf) + b * n(zf * zf) + c * n(zf * zf * zf) + e).to(act_dtype)
