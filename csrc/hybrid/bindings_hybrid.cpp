@@ -22,10 +22,18 @@ void launch_hy_mlstm_scan(const void*, int, const float*, const int32_t*, const 
                           float*, float*, float*, float*, float*, int, int, int, int, float, bool, hipStream_t);
 void launch_hy_mlstm_out(const float*, const void*, int, int, const float*, void*, int, int, int, float, bool,
                          hipStream_t);
-void launch_hy_latent_prep(void*, const void*, const int32_t*, const int32_t*, const int32_t*, int, const float*, float,
-                           const float*, int, int, int, int, int, void*, int, int, bool, hipStream_t);
+void launch_hy_latent_prep(void*, int64_t, const void*, int64_t, const int32_t*, const int32_t*, const int32_t*, int,
+                           const float*, float, const float*, int, bool, int, int, int, int, void*, int, void*, int, bool,
+                           hipStream_t);
+void launch_hy_head_matmul(const void*, int64_t, int64_t, const void*, void*, int64_t, int64_t, const void*, int64_t, int,
+                           int, int, int, bool, hipStream_t);
+void launch_hy_dyn_tanh(const float*, const float*, void*, int, int, bool, hipStream_t);
+void launch_hy_gated_join(const void*, float*, const void*, int64_t, const float*, float, const float*, void*, float*,
+                          const float*, int, bool, int, int, bool, hipStream_t);
+void launch_hy_poly_norm(const void*, int64_t, const float*, void*, int, int, float, bool, hipStream_t);
 bool launch_hy_latent_attention(const void*, const void*, const int32_t*, int, const int32_t*, const int32_t*,
-                                const float*, void*, int, int, int, int, int, int, float, bool, int, float*, float*, int64_t,
+                                const float*, void*, int, int, int, int, int, int, float, int, bool, bool, int, float*,
+                                float*, int64_t,
                                 hipStream_t);
 bool hy_latent_use_mfma(bool, int, int);
 int hy_latent_nsplit(int, int);
@@ -202,27 +210,113 @@ Tensor hy_mlstm_out(const Tensor& o, const Tensor& proj, int64_t g_off, const Te
 }
 
 void hy_latent_prep(Tensor& q, const Tensor& dkv, const Tensor& pos, const Tensor& tok_seq, const Tensor& block_table,
-                    const Tensor& w_norm, double eps, const Tensor& cos_sin, int64_t dims, int64_t rank, Tensor& cache) {
+                    const Tensor& w_norm, double eps, const c10::optional<Tensor>& cos_sin, int64_t dims, int64_t rank,
+                    Tensor& cache, c10::optional<Tensor> qa, bool interleaved) {
     c10::hip::HIPGuardMasqueradingAsCUDA g(q.device());
     same_act(q, dkv, "latent_prep: q and dkv in one activation dtype");
     same_act(q, cache, "latent_prep: the cache holds the activation dtype");
-    need(q.dim() == 3 && q.is_contiguous() && dkv.dim() == 2 && dkv.is_contiguous() && cache.dim() == 3 && cache.is_contiguous(), "latent_prep: layouts");
+    need(q.dim() == 3 && dkv.dim() == 2 && cache.dim() == 3 && cache.is_contiguous(), "latent_prep: layouts");
     const int64_t T = q.size(0), H = q.size(1), DK = dkv.size(1), R = DK - rank, D = q.size(2) - R;
+    // rows may be column ranges of a wider projection: a token's heads side by side, unit column stride
+    need(q.stride(2) == 1 && q.stride(1) == q.size(2) && q.stride(0) >= H * q.size(2), "latent_prep: q rows");
+    need(dkv.stride(1) == 1 && dkv.stride(0) >= DK, "latent_prep: dkv rows");
     need(dkv.size(0) == T && rank >= 1 && R >= 0 && D >= 0 && cache.size(2) == DK, "latent_prep: sizes");
-    need(dims % 2 == 0 && dims <= R, "latent_prep: rotated columns");
+    need(dims % 2 == 0 && dims >= 0 && dims <= R, "latent_prep: rotated columns");
     i32(pos, "latent_prep: pos"); i32(tok_seq, "latent_prep: tok_seq"); i32(block_table, "latent_prep: block_table");
     need(pos.numel() == T && tok_seq.numel() == T && block_table.dim() == 2, "latent_prep: per-token metadata");
-    flt(w_norm, "latent_prep: float32 norm weight"); flt(cos_sin, "latent_prep: float32 cos/sin table");
-    need(w_norm.numel() == rank && cos_sin.dim() == 2 && cos_sin.size(1) == dims, "latent_prep: norm weight / table width");
-    chronos::launch_hy_latent_prep(q.data_ptr(), dkv.data_ptr(), pos.data_ptr<int32_t>(), tok_seq.data_ptr<int32_t>(),
-                                   block_table.data_ptr<int32_t>(), (int)block_table.size(1), w_norm.data_ptr<float>(),
-                                   (float)eps, cos_sin.data_ptr<float>(), (int)dims, (int)rank, (int)R, (int)H, (int)D,
-                                   cache.data_ptr(), (int)cache.size(1), (int)T, f32(q), stream());
+    flt(w_norm, "latent_prep: float32 norm weight");
+    need(w_norm.numel() == rank, "latent_prep: norm weight");
+    need(dims == 0 || cos_sin.has_value(), "latent_prep: rotated columns need their table");
+    if (cos_sin) {
+        flt(*cos_sin, "latent_prep: float32 cos/sin table");
+        need(cos_sin->dim() == 2 && cos_sin->size(1) == dims, "latent_prep: table width");
+    }
+    if (qa) {
+        same_act(q, *qa, "latent_prep: qa in the activation dtype");
+        need(qa->is_contiguous() && qa->dim() == 3 && qa->size(0) == T && qa->size(1) == H && qa->size(2) == DK, "latent_prep: qa [T, H, rank + R]");
+    }
+    chronos::launch_hy_latent_prep(q.data_ptr(), q.stride(0), dkv.data_ptr(), dkv.stride(0), pos.data_ptr<int32_t>(),
+                                   tok_seq.data_ptr<int32_t>(), block_table.data_ptr<int32_t>(), (int)block_table.size(1),
+                                   w_norm.data_ptr<float>(), (float)eps, cos_sin ? cos_sin->data_ptr<float>() : nullptr,
+                                   (int)dims, interleaved, (int)rank, (int)R, (int)H, (int)D, cache.data_ptr(),
+                                   (int)cache.size(1), qa ? qa->data_ptr() : nullptr, (int)T, f32(q), stream());
+}
+
+// the first gate column of row 0 of a [T, C] activation tensor, after checking that columns off .. off + n exist
+const void* gate_cols(const Tensor& like, const c10::optional<Tensor>& src, int64_t off, int64_t T, int64_t n, const char* what) {
+    if (!src) return nullptr;
+    same_act(like, *src, what);
+    need(src->dim() == 2 && src->stride(1) == 1 && src->size(0) == T && off >= 0 && off + n <= src->size(1), what);
+    return static_cast<const char*>(src->data_ptr()) + off * src->element_size();
+}
+
+void hy_head_matmul(const Tensor& a, const Tensor& w, Tensor& out, const c10::optional<Tensor>& gate_src, int64_t g_off) {
+    c10::hip::HIPGuardMasqueradingAsCUDA g(a.device());
+    same_act(a, w, "head_matmul: operands in one activation dtype");
+    same_act(a, out, "head_matmul: output in the activation dtype");
+    need(a.dim() == 3 && w.dim() == 3 && out.dim() == 3 && w.is_contiguous(), "head_matmul: layouts");
+    const int64_t T = a.size(0), H = a.size(1), K = a.size(2), N = w.size(1);
+    need(w.size(0) == H && w.size(2) == K && K >= 1 && out.size(0) == T && out.size(1) == H && out.size(2) == N, "head_matmul: shapes");
+    need(H <= 65535 && a.stride(2) == 1 && out.stride(2) == 1 && out.stride(1) >= N && out.stride(0) >= (H - 1) * out.stride(1) + N,
+         "head_matmul: unit column strides, output rows that do not overlap");
+    const void* gp = gate_cols(a, gate_src, g_off, T, H * N, "head_matmul: gate columns");
+    chronos::launch_hy_head_matmul(a.data_ptr(), a.stride(0), a.stride(1), w.data_ptr(), out.data_ptr(), out.stride(0),
+                                   out.stride(1), gp, gate_src ? gate_src->stride(0) : 0, (int)T, (int)H, (int)N, (int)K,
+                                   f32(a), stream());
+}
+
+Tensor hy_dyn_tanh(const Tensor& x, const Tensor& wba, bool out_f32) {
+    c10::hip::HIPGuardMasqueradingAsCUDA g(x.device());
+    flt(x, "dyn_tanh: float32 rows");
+    flt(wba, "dyn_tanh: float32 weights");
+    need(x.dim() == 2 && wba.numel() == 2 * x.size(1) + 1 && x.numel() < (int64_t)1 << 31, "dyn_tanh: x [T, d], weights w | b | alpha");
+    auto h = at::empty_like(x, x.options().dtype(out_f32 ? at::kFloat : at::kBFloat16));
+    chronos::launch_hy_dyn_tanh(x.data_ptr<float>(), wba.data_ptr<float>(), h.data_ptr(), (int)x.size(0), (int)x.size(1),
+                                out_f32, stream());
+    return h;
+}
+
+Tensor hy_gated_join(const Tensor& y, Tensor& x, const c10::optional<Tensor>& gate_src, int64_t g_off,
+                     const c10::optional<Tensor>& gate_b, double mult, const c10::optional<Tensor>& wba,
+                     c10::optional<Tensor> hist, int64_t run, const c10::optional<Tensor>& dwa) {
+    c10::hip::HIPGuardMasqueradingAsCUDA g(x.device());
+    flt(x, "gated_join: float32 residual");
+    need(x.dim() == 2 && is_act(y) && y.is_contiguous() && y.sizes() == x.sizes() && x.numel() < (int64_t)1 << 31, "gated_join: y [T, d] in the activation dtype");
+    const int64_t T = x.size(0), d = x.size(1);
+    const void* gp = gate_cols(y, gate_src, g_off, T, d, "gated_join: gate columns");
+    if (gate_b) { flt(*gate_b, "gated_join: float32 gate bias"); need(gate_src.has_value() && gate_b->numel() == d, "gated_join: gate bias [d]"); }
+    if (wba) { flt(*wba, "gated_join: float32 norm weights"); need(wba->numel() == 2 * d + 1, "gated_join: norm weights w | b | alpha"); }
+    bool keep = false;
+    if (dwa) {
+        need(hist.has_value() && run >= 0, "gated_join: a depth average needs the earlier results");
+        flt(*dwa, "gated_join: float32 depth weights");
+        flt(*hist, "gated_join: float32 history");
+        need(hist->dim() == 3 && hist->size(1) == T && hist->size(2) == d && run < hist->size(0) && dwa->numel() == run + 2, "gated_join: history [runs, T, d], weights [run + 2]");
+        keep = run + 1 < hist->size(0);
+    }
+    Tensor h = wba ? at::empty({T, d}, y.options()) : at::empty({0}, y.options());
+    chronos::launch_hy_gated_join(y.data_ptr(), x.data_ptr<float>(), gp, gate_src ? gate_src->stride(0) : 0,
+                                  gate_b ? gate_b->data_ptr<float>() : nullptr, (float)mult,
+                                  wba ? wba->data_ptr<float>() : nullptr, wba ? h.data_ptr() : nullptr,
+                                  dwa ? hist->data_ptr<float>() : nullptr, dwa ? dwa->data_ptr<float>() : nullptr, (int)run,
+                                  keep, (int)T, (int)d, f32(y), stream());
+    return h;
+}
+
+Tensor hy_poly_norm(const Tensor& z, int64_t F, const Tensor& abce, double eps) {
+    c10::hip::HIPGuardMasqueradingAsCUDA g(z.device());
+    need(is_act(z) && z.dim() == 2 && z.is_contiguous() && F >= 1 && F <= z.size(1), "poly_norm: z [T, >= F]");
+    flt(abce, "poly_norm: float32 coefficients");
+    need(abce.numel() == 4, "poly_norm: four coefficients");
+    auto out = at::empty({z.size(0), F}, z.options());
+    chronos::launch_hy_poly_norm(z.data_ptr(), z.size(1), abce.data_ptr<float>(), out.data_ptr(), (int)z.size(0), (int)F,
+                                 (float)eps, f32(z), stream());
+    return out;
 }
 
 Tensor hy_latent_attention(const Tensor& qa, const Tensor& cache, const Tensor& block_table, const Tensor& q_start,
                            const Tensor& pos, const c10::optional<Tensor>& gate, double scale, int64_t rank,
-                           int64_t max_q) {
+                           int64_t max_q, int64_t window, bool two_term) {
     c10::hip::HIPGuardMasqueradingAsCUDA g(qa.device());
     same_act(qa, cache, "latent_attention: queries and cache in one activation dtype");
     need(qa.dim() == 3 && qa.is_contiguous() && cache.dim() == 3 && cache.is_contiguous(), "latent_attention: layouts");
@@ -231,7 +325,7 @@ Tensor hy_latent_attention(const Tensor& qa, const Tensor& cache, const Tensor& 
     need(f32(qa) || DK % 2 == 0, "latent_attention: bf16 rows need an even width");
     i32(block_table, "latent_attention: block_table"); i32(q_start, "latent_attention: q_start"); i32(pos, "latent_attention: pos");
     const int64_t B = q_start.numel() - 1;
-    need(block_table.dim() == 2 && block_table.size(0) >= B && pos.numel() == T, "latent_attention: metadata");
+    need(block_table.dim() == 2 && block_table.size(0) >= B && pos.numel() == T && window >= 0, "latent_attention: metadata");
     if (gate) { flt(*gate, "latent_attention: float32 gate"); need(gate->numel() == T * H, "latent_attention: gate [T, H]"); }
     auto out = at::empty({T, H, rank}, qa.options());
     if (T == 0 || B <= 0) return out;
@@ -241,7 +335,9 @@ Tensor hy_latent_attention(const Tensor& qa, const Tensor& cache, const Tensor& 
     int nsplit = 1;
     Tensor part_o, part_ml;
     if (chronos::hy_latent_use_mfma(f32(qa), (int)DK, (int)rank)) {
-        nsplit = chronos::hy_latent_nsplit((int)(B * ((mq * H + 63) / 64)), (int)(block_table.size(1) * cache.size(1)));
+        int64_t span = block_table.size(1) * cache.size(1);   // keys a row block walks at most
+        if (window > 0) span = std::min<int64_t>(span, window + mq);
+        nsplit = chronos::hy_latent_nsplit((int)(B * ((mq * H + 63) / 64)), (int)span);
         if (nsplit > 1) {
             part_o = at::empty({T * H * nsplit, rank}, qa.options().dtype(at::kFloat));
             part_ml = at::empty({T * H * nsplit, 2}, qa.options().dtype(at::kFloat));
@@ -250,7 +346,8 @@ Tensor hy_latent_attention(const Tensor& qa, const Tensor& cache, const Tensor& 
     const bool ok = chronos::launch_hy_latent_attention(
         qa.data_ptr(), cache.data_ptr(), block_table.data_ptr<int32_t>(), (int)block_table.size(1),
         q_start.data_ptr<int32_t>(), pos.data_ptr<int32_t>(), gate ? gate->data_ptr<float>() : nullptr, out.data_ptr(),
-        (int)B, (int)H, (int)DK, (int)rank, (int)cache.size(1), mq, (float)scale, f32(qa), nsplit,
+        (int)B, (int)H, (int)DK, (int)rank, (int)cache.size(1), mq, (float)scale, (int)window,
+        two_term, f32(qa), nsplit,
         nsplit > 1 ? part_o.data_ptr<float>() : nullptr, nsplit > 1 ? part_ml.data_ptr<float>() : nullptr, T * H, stream());
     TORCH_CHECK(ok, "chronos hybrid op: latent_attention has no launch geometry for heads=", H, " row width=", DK,
                 " rank=", rank, " (rank <= 512; 16 keys and 4 query rows must fit the LDS)");
@@ -819,9 +916,15 @@ TORCH_LIBRARY_FRAGMENT(chronos, m) {
           "Tensor(b!) n, Tensor(c!) m, int H, int D, int Dv, float cap) -> Tensor");
     m.def("hy_mlstm_out(Tensor o, Tensor proj, int g_off, Tensor w, float eps, bool out_f32) -> Tensor");
     m.def("hy_latent_prep(Tensor(a!) q, Tensor dkv, Tensor pos, Tensor tok_seq, Tensor block_table, Tensor w_norm, "
-          "float eps, Tensor cos_sin, int dims, int rank, Tensor(b!) cache) -> ()");
+          "float eps, Tensor? cos_sin, int dims, int rank, Tensor(b!) cache, Tensor(c!)? qa=None, "
+          "bool interleaved=False) -> ()");
+    m.def("hy_head_matmul(Tensor a, Tensor w, Tensor(a!) out, Tensor? gate_src, int g_off) -> ()");
+    m.def("hy_dyn_tanh(Tensor x, Tensor wba, bool out_f32) -> Tensor");
+    m.def("hy_gated_join(Tensor y, Tensor(a!) x, Tensor? gate_src, int g_off, Tensor? gate_b, float mult, Tensor? wba, "
+          "Tensor(b!)? hist, int run, Tensor? dwa) -> Tensor");
+    m.def("hy_poly_norm(Tensor z, int F, Tensor abce, float eps) -> Tensor");
     m.def("hy_latent_attention(Tensor qa, Tensor cache, Tensor block_table, Tensor q_start, Tensor pos, Tensor? gate, "
-          "float scale, int rank, int max_q) -> Tensor");
+          "float scale, int rank, int max_q, int window=0, bool two_term=False) -> Tensor");
     m.def("hy_moe_route(Tensor h, Tensor w, Tensor corr, int top) -> (Tensor, Tensor)");
     m.def("hy_moe_ffn(Tensor h, Tensor idx, Tensor wt, Tensor w_up, Tensor w_down, int act) -> Tensor");
     m.def("hy_rms_norm(Tensor x, Tensor w, float eps, bool out_f32) -> Tensor");
@@ -872,6 +975,10 @@ TORCH_LIBRARY_IMPL(chronos, CUDA, m) {
     m.impl("hy_mlstm_scan", &hy_mlstm_scan);
     m.impl("hy_mlstm_out", &hy_mlstm_out);
     m.impl("hy_latent_prep", &hy_latent_prep);
+    m.impl("hy_head_matmul", &hy_head_matmul);
+    m.impl("hy_dyn_tanh", &hy_dyn_tanh);
+    m.impl("hy_gated_join", &hy_gated_join);
+    m.impl("hy_poly_norm", &hy_poly_norm);
     m.impl("hy_latent_attention", &hy_latent_attention);
     m.impl("hy_moe_route", &hy_moe_route);
     m.impl("hy_moe_ffn", &hy_moe_ffn);

@@ -8,12 +8,16 @@
 // key width rank + R and value width rank).
 //
 //   latent_prep       per token: RMS norm of the latent columns (float), rotation of the shared key part and of
-//                     every head's rotated query columns (cos / sin from a float table made in double precision),
-//                     cache write at the token's page and slot.
+//                     every head's rotated query columns (cos / sin from a float table made in double precision; pairs
+//                     are columns i and i + dims / 2, or 2i and 2i + 1), cache write at the token's page and slot.  The
+//                     projections' rows may be wider than what is read of them, and the rotated query columns go in
+//                     place or straight to their columns of the latent query.
 //   latent_attention  one workgroup per (sequence, block of up to 64 (token, head) rows): the rows are split
 //                     over 4 waves; 64-key tiles of the cache are staged in LDS; lanes are keys for the scores
 //                     (float accumulation, causal mask by each row's own position, online softmax in float) and
 //                     latent columns for the output.  Serves prefill chunks and decode rows (a tile of one token).
+//                     With window > 0 a row sees only the last `window` positions up to its own: the walk starts at
+//                     the tile of the first row's first visible key, and each row masks by its own position.
 #include <cstdlib>
 
 #include "hybrid_common.h"
@@ -23,16 +27,17 @@ namespace hy {
 
 template <typename T>
 __global__ void __launch_bounds__(256) latent_prep_kernel(
-        T* __restrict__ q, const T* __restrict__ dkv, const int32_t* __restrict__ pos, const int32_t* __restrict__ tok_seq,
-        const int32_t* __restrict__ block_table, int max_blocks, const float* __restrict__ w_norm, float eps,
-        const float* __restrict__ cos_sin, int dims, int rank, int R, int H, int D, T* __restrict__ cache, int BS) {
+        T* q, int64_t ldq, const T* __restrict__ dkv, int64_t ldkv, const int32_t* __restrict__ pos,
+        const int32_t* __restrict__ tok_seq, const int32_t* __restrict__ block_table, int max_blocks,
+        const float* __restrict__ w_norm, float eps, const float* __restrict__ cos_sin, int dims, int inter, int rank,
+        int R, int H, int D, T* __restrict__ cache, int BS, T* __restrict__ qa) {
     __shared__ float red[16];
     const int64_t t = blockIdx.x;
     const int p = pos[t];
     const int blk = block_table[(int64_t)tok_seq[t] * max_blocks + p / BS];
     const int DK = rank + R;
     T* crow = cache + ((int64_t)blk * BS + p % BS) * DK;
-    const T* drow = dkv + t * DK;
+    const T* drow = dkv + t * ldkv;
     float ss = 0.f;
     for (int i = threadIdx.x; i < rank; i += 256) {
         const float v = ld<T>(drow + i);
@@ -42,20 +47,23 @@ __global__ void __launch_bounds__(256) latent_prep_kernel(
     for (int i = threadIdx.x; i < rank; i += 256) st<T>(crow + i, ld<T>(drow + i) * inv * w_norm[i]);
     const int half = dims / 2;
     const float* cs = cos_sin + (int64_t)p * dims;
-    // the shared key part: pairs (i, i + half) rotated, the columns past `dims` copied
-    for (int i = threadIdx.x; i < R; i += 256) {
-        float v = ld<T>(drow + rank + i);
-        if (i < half) v = v * cs[i] - ld<T>(drow + rank + i + half) * cs[half + i];
-        else if (i < dims) v = v * cs[i - half] + ld<T>(drow + rank + i - half) * cs[i];
-        st<T>(crow + rank + i, v);
+    // rows to rotate: the shared key part (row 0) and every head's rotated query columns.  Each thread owns whole pairs
+    // (columns lo and hi), so rotating in place reads nothing another thread writes; columns past `dims` are copied.
+    for (int i = threadIdx.x; i < (H + 1) * half; i += 256) {
+        const int row = i / half, k = i % half;
+        const int lo = inter ? 2 * k : k, hi = inter ? 2 * k + 1 : k + half;
+        const T* src = row == 0 ? drow + rank : q + t * ldq + (int64_t)(row - 1) * (D + R) + D;
+        T* dst = row == 0 ? crow + rank : qa != nullptr ? qa + (t * H + row - 1) * DK + rank
+                                                        : q + t * ldq + (int64_t)(row - 1) * (D + R) + D;
+        const float u = ld<T>(src + lo), v = ld<T>(src + hi), c = cs[k], s = cs[half + k];
+        st<T>(dst + lo, u * c - v * s);
+        st<T>(dst + hi, v * c + u * s);
     }
-    // every head's rotated query columns, in place: each thread owns whole pairs
-    for (int i = threadIdx.x; i < H * half; i += 256) {
-        const int hd = i / half, k = i % half;
-        T* qr = q + (t * H + hd) * (D + R) + D;
-        const float u = ld<T>(qr + k), v = ld<T>(qr + k + half);
-        st<T>(qr + k, u * cs[k] - v * cs[half + k]);
-        st<T>(qr + k + half, v * cs[k] + u * cs[half + k]);
+    const int rest = R - dims;
+    for (int i = threadIdx.x; i < (qa != nullptr ? H + 1 : 1) * rest; i += 256) {
+        const int row = i / rest, k = dims + i % rest;
+        if (row == 0) crow[rank + k] = drow[rank + k];
+        else qa[(t * H + row - 1) * DK + rank + k] = q[t * ldq + (int64_t)(row - 1) * (D + R) + D + k];
     }
 }
 
@@ -79,7 +87,7 @@ template <typename T, int DVL>
 __global__ void __launch_bounds__(256) latent_attention_kernel(
         const T* __restrict__ qa, const T* __restrict__ cache, const int32_t* __restrict__ block_table, int max_blocks,
         const int32_t* __restrict__ q_start, const int32_t* __restrict__ pos, const float* __restrict__ gate,
-        T* __restrict__ out, int H, int DK, int rank, int BS, int RBLK, int KT, int kstride, float scale) {
+        T* __restrict__ out, int H, int DK, int rank, int BS, int RBLK, int KT, int kstride, float scale, int window) {
     constexpr int E = Word<T>::E, RB = 4, RWMAX = 16;
     extern __shared__ __attribute__((aligned(16))) uint32_t smem[];
     const int b = blockIdx.x;
@@ -113,7 +121,8 @@ __global__ void __launch_bounds__(256) latent_attention_kernel(
     }
     float* pw = ps + wv * 64 * RB;
     const int32_t* bt = block_table + (int64_t)b * max_blocks;
-    for (int k0 = 0; k0 <= pmax; k0 += KT) {
+    const int k_lo = window > 0 ? max(0, pos[t0 + rb0 / H] - window + 1) / KT * KT : 0;  // (positions grow along the rows)
+    for (int k0 = k_lo; k0 <= pmax; k0 += KT) {
         __syncthreads();  // everyone is done with the previous key tile (and the query rows are staged)
         const int nk = min(KT, pmax + 1 - k0);
         // one wave per key row in turn (no index arithmetic per element; the page lookup is wave-uniform); 16-byte
@@ -158,7 +167,7 @@ __global__ void __launch_bounds__(256) latent_attention_kernel(
 #pragma unroll
                 for (int u = 0; u < RB; ++u) {
                     const int i = g * RB + u;
-                    const bool seen = lane < nk && k0 + lane <= prow[i];
+                    const bool seen = lane < nk && k0 + lane <= prow[i] && (window <= 0 || prow[i] - (k0 + lane) < window);
                     const float s = seen ? sc[u] * scale : -INFINITY;
                     const float mn = fmaxf(mrow[i], wave_max(s));
                     // a row that has seen no key yet keeps m = -inf: every weight 0, nothing to rescale
@@ -214,12 +223,14 @@ __global__ void __launch_bounds__(256) latent_attention_kernel(
 
 }  // namespace hy
 
-void launch_hy_latent_prep(void* q, const void* dkv, const int32_t* pos, const int32_t* tok_seq, const int32_t* bt,
-                           int max_blocks, const float* w_norm, float eps, const float* cos_sin, int dims, int rank,
-                           int R, int H, int D, void* cache, int BS, int T, bool f32, hipStream_t s) {
+// ldq, ldkv: row strides of q and dkv in elements.  qa == nullptr: queries are rotated in place.
+void launch_hy_latent_prep(void* q, int64_t ldq, const void* dkv, int64_t ldkv, const int32_t* pos, const int32_t* tok_seq,
+                           const int32_t* bt, int max_blocks, const float* w_norm, float eps, const float* cos_sin, int dims,
+                           bool inter, int rank, int R, int H, int D, void* cache, int BS, void* qa, int T, bool f32,
+                           hipStream_t s) {
     if (T == 0) return;
-    if (f32) hy::latent_prep_kernel<float><<<T, 256, 0, s>>>((float*)q, (const float*)dkv, pos, tok_seq, bt, max_blocks, w_norm, eps, cos_sin, dims, rank, R, H, D, (float*)cache, BS);
-    else hy::latent_prep_kernel<uint16_t><<<T, 256, 0, s>>>((uint16_t*)q, (const uint16_t*)dkv, pos, tok_seq, bt, max_blocks, w_norm, eps, cos_sin, dims, rank, R, H, D, (uint16_t*)cache, BS);
+    if (f32) hy::latent_prep_kernel<float><<<T, 256, 0, s>>>((float*)q, ldq, (const float*)dkv, ldkv, pos, tok_seq, bt, max_blocks, w_norm, eps, cos_sin, dims, inter, rank, R, H, D, (float*)cache, BS, (float*)qa);
+    else hy::latent_prep_kernel<uint16_t><<<T, 256, 0, s>>>((uint16_t*)q, ldq, (const uint16_t*)dkv, ldkv, pos, tok_seq, bt, max_blocks, w_norm, eps, cos_sin, dims, inter, rank, R, H, D, (uint16_t*)cache, BS, (uint16_t*)qa);
 }
 
 // Launch geometry of latent_attention for these sizes: RBLK (token, head) rows per workgroup (<= 64), KT keys per
@@ -247,7 +258,7 @@ bool hy_latent_geometry(int H, int DK, int esize, int max_q, int lds_limit, int*
 template <typename T, int DVL>
 static void latent_attn_t(const T* qa, const T* cache, const int32_t* bt, int max_blocks, const int32_t* q_start,
                           const int32_t* pos, const float* gate, T* out, int B, int H, int DK, int rank, int BS,
-                          int max_q, int RBLK, int KT, int kstride, int bytes, float scale, hipStream_t s) {
+                          int max_q, int RBLK, int KT, int kstride, int bytes, float scale, int window, hipStream_t s) {
     auto kern = hy::latent_attention_kernel<T, DVL>;
     static int set_bytes = 0;
     if (bytes > set_bytes) {  // raise the dynamic-LDS ceiling of this instantiation once per size
@@ -255,12 +266,12 @@ static void latent_attn_t(const T* qa, const T* cache, const int32_t* bt, int ma
         set_bytes = bytes;
     }
     const dim3 grid(B, (max_q * H + RBLK - 1) / RBLK);
-    kern<<<grid, 256, bytes, s>>>(qa, cache, bt, max_blocks, q_start, pos, gate, out, H, DK, rank, BS, RBLK, KT, kstride, scale);
+    kern<<<grid, 256, bytes, s>>>(qa, cache, bt, max_blocks, q_start, pos, gate, out, H, DK, rank, BS, RBLK, KT, kstride, scale, window);
 }
 
 bool launch_hy_latent_attention_mfma(const uint16_t*, const uint16_t*, const int32_t*, int, const int32_t*, const int32_t*,
-                                     const float*, uint16_t*, int, int, int, int, int, int, float, int, float*, float*,
-                                     int64_t, hipStream_t);
+                                     const float*, uint16_t*, int, int, int, int, int, int, float, int, bool, int, float*,
+                                     float*, int64_t, hipStream_t);
 bool hy_latent_mfma_ok(int DK, int rank);
 
 // whether this call goes to the matrix-core kernel (bfloat16 at its sizes; CHRONOS_LATENT_MFMA=0 keeps the general
@@ -275,16 +286,16 @@ bool hy_latent_use_mfma(bool f32, int DK, int rank) {
 
 bool launch_hy_latent_attention(const void* qa, const void* cache, const int32_t* bt, int max_blocks,
                                 const int32_t* q_start, const int32_t* pos, const float* gate, void* out, int B, int H,
-                                int DK, int rank, int BS, int max_q, float scale, bool f32, int nsplit, float* part_o,
-                                float* part_ml, int64_t total_rows, hipStream_t s) {
+                                int DK, int rank, int BS, int max_q, float scale, int window, bool two_term, bool f32,
+                                int nsplit, float* part_o, float* part_ml, int64_t total_rows, hipStream_t s) {
     if (B == 0 || max_q == 0) return true;
     if (hy_latent_use_mfma(f32, DK, rank))
         return launch_hy_latent_attention_mfma((const uint16_t*)qa, (const uint16_t*)cache, bt, max_blocks, q_start, pos, gate,
-                                               (uint16_t*)out, B, H, DK, rank, BS, max_q, scale, nsplit, part_o, part_ml,
-                                               total_rows, s);
+                                               (uint16_t*)out, B, H, DK, rank, BS, max_q, scale, window, two_term, nsplit,
+                                               part_o, part_ml, total_rows, s);
     int RBLK, KT, kstride, bytes;
     if (rank > 512 || !hy_latent_geometry(H, DK, f32 ? 4 : 2, max_q, 160 * 1024, &RBLK, &KT, &kstride, &bytes)) return false;
-#define HY_LA(TT, DVL) latent_attn_t<TT, DVL>((const TT*)qa, (const TT*)cache, bt, max_blocks, q_start, pos, gate, (TT*)out, B, H, DK, rank, BS, max_q, RBLK, KT, kstride, bytes, scale, s)
+#define HY_LA(TT, DVL) latent_attn_t<TT, DVL>((const TT*)qa, (const TT*)cache, bt, max_blocks, q_start, pos, gate, (TT*)out, B, H, DK, rank, BS, max_q, RBLK, KT, kstride, bytes, scale, window, s)
     const int dvl = (rank + 63) / 64;
     if (f32) {
         if (dvl <= 1) HY_LA(float, 1); else if (dvl <= 2) HY_LA(float, 2); else if (dvl <= 4) HY_LA(float, 4); else HY_LA(float, 8);

@@ -13,8 +13,12 @@
 //     reductions over the 4 lane groups by two shuffles;
 //   * sum  O^T = V^T P^T : the lane's 8 weights of two neighbouring 16-key tiles ARE a B operand (the k index is a
 //     fixed permutation of the 32 keys, the same one the transposed value image is read with), so the weights never
-//     leave registers.  Accumulators: rank / 16 tiles x 4 registers.
-// Sizes: DK % 32 == 0, rank % 16 == 0, DK <= 576, rank <= 512.  Everything else takes latent_attention.hip.
+//     leave registers.  Accumulators: rank / 16 tiles x 4 registers.  Optionally each weight enters as two
+//     bfloat16 terms (rounded value + remainder), which keeps the float softmax weights nearly exact.
+// With a window a row sees only its last `window` positions: the walk starts at the tile of the first row's first
+// visible key and every row masks by its own position.
+// Sizes: DK % 8 == 0 (the last 32-column step of the scores is zero-filled), rank % 16 == 0, DK <= 576, rank <= 512.
+// Everything else takes latent_attention.hip.
 #include <cstdlib>
 
 #include "hybrid_common.h"
@@ -29,12 +33,13 @@ constexpr int MKT = 64;  // keys per tile at most
 // other multiplies).
 // NW: waves per workgroup, 4 or 8 (16 query rows each): with 8 a staged key tile serves 128 rows and every SIMD holds two
 // waves, so one wave's softmax and staging run beside the other's MFMAs.
-template <int NS, int NCT, int KT, int NW>
+// TT: weights as two bfloat16 terms.
+template <int NS, int NCT, int KT, int NW, bool TT>
 __global__ void __launch_bounds__(64 * NW) latent_attention_mfma_kernel(
         const uint16_t* __restrict__ qa, const uint16_t* __restrict__ cache, const int32_t* __restrict__ block_table,
         int max_blocks, const int32_t* __restrict__ q_start, const int32_t* __restrict__ pos,
         const float* __restrict__ gate, uint16_t* __restrict__ out, int H, int DK, int rank, int BS, float scale,
-        int nsplit, float* __restrict__ part_o, float* __restrict__ part_ml, int bs_shift) {
+        int window, int nsplit, float* __restrict__ part_o, float* __restrict__ part_ml, int bs_shift) {
     extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
     const int b = blockIdx.x;
     const int t0 = q_start[b], t1 = q_start[b + 1];
@@ -43,8 +48,8 @@ __global__ void __launch_bounds__(64 * NW) latent_attention_mfma_kernel(
     const int rb0 = blockIdx.y * RPB;
     if (rb0 >= rows_total) return;
     const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6, g = lane >> 4, qi = lane & 15;
-    const int ns = DK / 32, nct = rank / 16;
-    const int krs = DK * 2 + 16;            // row-major image: bytes per key row
+    const int ns = (DK + 31) / 32, nct = rank / 16;
+    const int krs = ns * 64 + 16;           // row-major image: bytes per key row
     constexpr int vts = KT * 2 + 8;         // transposed image: bytes per value column
     constexpr int PP = KT / 2;              // key pairs per tile
     __shared__ int krow[MKT];  // cache row (page * page size + slot) of each key of the tile
@@ -58,19 +63,30 @@ __global__ void __launch_bounds__(64 * NW) latent_attention_mfma_kernel(
     const int prow = rok ? pos[t0 + rc / H] : -1;
     const int last_row = min(rows_total, rb0 + RPB) - 1;
     const int pmax = pos[t0 + last_row / H];                // positions grow along the sequence
+    const int k_lo = window > 0 ? max(0, pos[t0 + rb0 / H] - window + 1) / KT * KT : 0;
+    const int row_lo = window > 0 ? prow - window + 1 : 0;  // the first key this lane's row sees
     bf16x8 qf[NS];
 #pragma unroll
     for (int s = 0; s < NS; ++s)
-        if (s < ns) qf[s] = *reinterpret_cast<const bf16x8*>(qa + grow * DK + 32 * s + 8 * g);
+        if (s < ns) {
+            const u16x8 z = {0, 0, 0, 0, 0, 0, 0, 0};
+            qf[s] = 32 * s + 8 * g < DK ? *reinterpret_cast<const bf16x8*>(qa + grow * DK + 32 * s + 8 * g)
+                                        : __builtin_bit_cast(bf16x8, z);
+        }
     f32x4 O[NCT];
 #pragma unroll
     for (int c = 0; c < NCT; ++c) O[c] = f32x4{0.f, 0.f, 0.f, 0.f};
     float mrow = -INFINITY, lrow = 0.f;
     const int32_t* bt = block_table + (int64_t)b * max_blocks;
     const int chunks = DK / 8, vchunks = rank / 8;
+    const int padc = ns * 4 - chunks;   // zero chunks behind a key row (staging never writes them)
+    for (int it = threadIdx.x; it < KT * padc; it += NT) {
+        const u16x8 z = {0, 0, 0, 0, 0, 0, 0, 0};
+        *reinterpret_cast<u16x8*>(kimg + it / padc * krs + (chunks + it % padc) * 16) = z;
+    }
     // key tiles are dealt round-robin to the nsplit workgroups of this row block (blockIdx.z): the context length is
     // only known on the device, and a split that gets no tile contributes an empty partial
-    for (int k0 = blockIdx.z * KT; k0 <= pmax; k0 += KT * nsplit) {
+    for (int k0 = k_lo + blockIdx.z * KT; k0 <= pmax; k0 += KT * nsplit) {
         __syncthreads();
         // ---- cache rows of the tile's 64 keys (page lookup once per key, not once per staged vector: a lookup in
         // front of every data load made each of them wait for two trips to memory)
@@ -130,7 +146,7 @@ __global__ void __launch_bounds__(64 * NW) latent_attention_mfma_kernel(
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
                 const int key = k0 + 16 * kt + 4 * g + i;
-                const float sv = key <= prow ? S[kt][i] * scale : -INFINITY;
+                const float sv = key <= prow && key >= row_lo ? S[kt][i] * scale : -INFINITY;
                 S[kt][i] = sv;
                 mx = fmaxf(mx, sv);
             }
@@ -153,11 +169,16 @@ __global__ void __launch_bounds__(64 * NW) latent_attention_mfma_kernel(
         mrow = mn;
         // ---- weighted sum of the value columns: k index of step u = [tile 2u keys 4g..4g+3 | tile 2u+1 keys 4g..4g+3]
         constexpr int NU = KT / 32;
-        bf16x8 pf[NU];
+        bf16x8 pf[NU], pl[TT ? NU : 1];
 #pragma unroll
-        for (int u = 0; u < NU; ++u)
+        for (int u = 0; u < NU; ++u) {
             pf[u] = bf16x8{(__bf16)S[2 * u][0], (__bf16)S[2 * u][1], (__bf16)S[2 * u][2], (__bf16)S[2 * u][3],
                            (__bf16)S[2 * u + 1][0], (__bf16)S[2 * u + 1][1], (__bf16)S[2 * u + 1][2], (__bf16)S[2 * u + 1][3]};
+            if constexpr (TT) {
+#pragma unroll
+                for (int e = 0; e < 8; ++e) pl[u][e] = (__bf16)(S[2 * u + (e >> 2)][e & 3] - (float)pf[u][e]);
+            }
+        }
 #pragma unroll
         for (int c = 0; c < NCT; ++c) {
             if (c < nct) {
@@ -169,6 +190,7 @@ __global__ void __launch_bounds__(64 * NW) latent_attention_mfma_kernel(
                     const bf16x4 hi = *reinterpret_cast<const bf16x4*>(vrow + u * 64 + 32);
                     const bf16x8 vf = __builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7);
                     O[c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pf[u], O[c], 0, 0, 0);
+                    if constexpr (TT) O[c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pl[u], O[c], 0, 0, 0);
                 }
             }
         }
@@ -224,13 +246,13 @@ __global__ void __launch_bounds__(256) latent_combine_kernel(const float* __rest
 
 }  // namespace hy
 
-template <int NS, int NCT, int KT, int NW>
+template <int NS, int NCT, int KT, int NW, bool TT>
 static void la_mfma_launch(const uint16_t* qa, const uint16_t* cache, const int32_t* bt, int max_blocks,
                            const int32_t* q_start, const int32_t* pos, const float* gate, uint16_t* out, int B, int H,
-                           int DK, int rank, int BS, int max_q, float scale, int nsplit, float* part_o, float* part_ml,
-                           hipStream_t s) {
-    auto kern = hy::latent_attention_mfma_kernel<NS, NCT, KT, NW>;
-    const int bytes = KT * (DK * 2 + 16) + rank * (KT * 2 + 8);
+                           int DK, int rank, int BS, int max_q, float scale, int window, int nsplit, float* part_o,
+                           float* part_ml, hipStream_t s) {
+    auto kern = hy::latent_attention_mfma_kernel<NS, NCT, KT, NW, TT>;
+    const int bytes = KT * ((DK + 31) / 32 * 64 + 16) + rank * (KT * 2 + 8);
     static int set_bytes = 0;
     if (bytes > set_bytes) {
         (void)hipFuncSetAttribute(reinterpret_cast<const void*>(kern), hipFuncAttributeMaxDynamicSharedMemorySize, bytes);
@@ -238,11 +260,11 @@ static void la_mfma_launch(const uint16_t* qa, const uint16_t* cache, const int3
     }
     const dim3 grid(B, (max_q * H + 16 * NW - 1) / (16 * NW), nsplit);
     const int bs_shift = (BS & (BS - 1)) == 0 ? __builtin_ctz(BS) : -1;
-    kern<<<grid, 64 * NW, bytes, s>>>(qa, cache, bt, max_blocks, q_start, pos, gate, out, H, DK, rank, BS, scale, nsplit, part_o,
-                                  part_ml, bs_shift);
+    kern<<<grid, 64 * NW, bytes, s>>>(qa, cache, bt, max_blocks, q_start, pos, gate, out, H, DK, rank, BS, scale, window,
+                                  nsplit, part_o, part_ml, bs_shift);
 }
 
-bool hy_latent_mfma_ok(int DK, int rank) { return !(DK % 32 || rank % 16 || DK > 576 || rank > 512 || rank > DK); }
+bool hy_latent_mfma_ok(int DK, int rank) { return !(DK % 8 || rank % 16 || DK > 576 || rank > 512 || rank > DK); }
 
 // Splits of the key range (flash-decoding) for a launch of `wgs` workgroups over contexts of at most max_ctx keys:
 // enough workgroups to cover the chip, at least 4 key tiles per split, at most 16.
@@ -258,11 +280,11 @@ int hy_latent_nsplit(int wgs, int max_ctx) {
 // [T * H * nsplit, rank] and part_ml float [T * H * nsplit, 2] scratch.
 bool launch_hy_latent_attention_mfma(const uint16_t* qa, const uint16_t* cache, const int32_t* bt, int max_blocks,
                                      const int32_t* q_start, const int32_t* pos, const float* gate, uint16_t* out, int B,
-                                     int H, int DK, int rank, int BS, int max_q, float scale, int nsplit, float* part_o,
-                                     float* part_ml, int64_t total_rows, hipStream_t s) {
+                                     int H, int DK, int rank, int BS, int max_q, float scale, int window, bool two_term,
+                                     int nsplit, float* part_o, float* part_ml, int64_t total_rows, hipStream_t s) {
     if (!hy_latent_mfma_ok(DK, rank)) return false;
     if (B == 0 || max_q == 0) return true;
-#define HY_LAM(NS, NCT, KT, NW) la_mfma_launch<NS, NCT, KT, NW>(qa, cache, bt, max_blocks, q_start, pos, gate, out, B, H, DK, rank, BS, max_q, scale, nsplit, part_o, part_ml, s)
+#define HY_LAM(NS, NCT, KT, NW, TT) la_mfma_launch<NS, NCT, KT, NW, TT>(qa, cache, bt, max_blocks, q_start, pos, gate, out, B, H, DK, rank, BS, max_q, scale, window, nsplit, part_o, part_ml, s)
     // 64-key tiles (32-key tiles measured slower at every size: the per-tile softmax and barriers weigh more than the
     // second workgroup per CU gains; CHRONOS_LATENT_KT=32 keeps them for A/B).  8 waves per workgroup when a sequence
     // brings more than 64 rows (CHRONOS_LATENT_NW=4 / 8 forces one).
@@ -272,8 +294,9 @@ bool launch_hy_latent_attention_mfma(const uint16_t* qa, const uint16_t* cache, 
     const bool nw8 = force_nw == 8 || (force_nw != 4 && max_q * H > 64);
 #define HY_LAM_T(NS, NCT)                                                            \
     do {                                                                             \
-        if (kt32) { if (nw8) HY_LAM(NS, NCT, 32, 8); else HY_LAM(NS, NCT, 32, 4); }   \
-        else { if (nw8) HY_LAM(NS, NCT, 64, 8); else HY_LAM(NS, NCT, 64, 4); }       \
+        if (two_term) { if (nw8) HY_LAM(NS, NCT, 64, 8, true); else HY_LAM(NS, NCT, 64, 4, true); }         \
+        else if (kt32) { if (nw8) HY_LAM(NS, NCT, 32, 8, false); else HY_LAM(NS, NCT, 32, 4, false); }      \
+        else { if (nw8) HY_LAM(NS, NCT, 64, 8, false); else HY_LAM(NS, NCT, 64, 4, false); }                \
     } while (0)
     if (DK <= 128 && rank <= 64) HY_LAM_T(4, 4);
     else if (DK <= 320 && rank <= 256) HY_LAM_T(10, 16);
