@@ -1,13 +1,14 @@
-"""Throughput of a hybrid design (Zokunex, Kalesun, Tugovik, Vogerax) beside the framework's other models at equal width and depth:
+"""Throughput of a hybrid design (Zokunex, Kalesun, Tugovik, Vogerax, Lalasun) beside the framework's other models at equal width and depth:
 whole-model prefill and decode steps, and each of the design's kernels beside its closest existing kernel with the
 fraction of its roofline it reaches.
 
-``python bench.py --design-compare [--design zokunex|kalesun|tugovik|vogerax] [--design-sizes 1k,2k,4k]`` prints one JSON line
+``python bench.py --design-compare [--design zokunex|kalesun|tugovik|vogerax|lalasun] [--design-sizes 1k,2k,4k]`` prints one JSON line
 (the default benchmark and its output line are untouched).  Zokunex stands beside Llama; Kalesun beside Zokunex (the
 closest family: recurrent layers, attention and mixtures of experts on a float32 stream) and Llama; Tugovik beside
 Kalesun (masked grouped-query attention over paged keys and values, linear-state scans behind a short convolution,
 gated experts, RMS norms on the stream) and Llama; Vogerax beside Kalesun too (windowed and causal sink attention on
-the same kernels, a linear-state scan, RMS norms joined to a float32 stream) and Llama.  Weights are random; every number is measured on the GPU this
+the same kernels, a linear-state scan, RMS norms joined to a float32 stream) and Llama; Lalasun beside Kalesun (masked
+sink attention, gated linear attention, dense feed-forwards), Zokunex (latent attention) and Llama.  Weights are random; every number is measured on the GPU this
 process runs on.
 
 Rooflines: HBM 8 TB/s for kernels bound by the bytes they must move, 2.5 PFLOP/s dense bf16 for the matrix-shaped
@@ -126,6 +127,29 @@ def vogerax_config(size: dict) -> dict:
     layers = [dict(mix_a, mlp=dense), dict(mix_p, mlp=moe), dict(mix_a, mlp=moe), dict(mix_p, mlp=dense)][:LAYERS]
     return dict(architecture="Vogerax", vocab=VOCAB, width=size["width"], norm=dict(eps=1e-6, groups=size["groups"]),
                 embedding=dict(scale=8.0), layers=layers)
+
+
+# Lalasun: width -> (attention heads, kv heads, dim, vdim, chunk | latent heads, dim, rot, vdim, rank, window |
+#                    gla heads, dim, vdim | dense ff)
+LALASUN_SIZES = {
+    "1k": dict(width=1024, a=(8, 2, 128, 128, 512), l=(8, 64, 32, 64, 256, 512), g=(4, 128, 256), ff=4096),
+    "2k": dict(width=2048, a=(16, 4, 128, 128, 1024), l=(16, 128, 64, 128, 512, 1024), g=(8, 128, 256), ff=8192),
+    "4k": dict(width=4096, a=(32, 8, 128, 128, 1024), l=(32, 128, 64, 128, 512, 1024), g=(16, 128, 256), ff=14336),
+}
+
+
+def lalasun_config(size: dict) -> dict:
+    ah, ag, ad, av, chunk = size["a"]
+    lh, ld, lr, lv, rank, win = size["l"]
+    gh, gd, gv = size["g"]
+    mix_a = dict(type="attention", mixer=dict(heads=ah, kv_heads=ag, dim=ad, vdim=av, scale=ad ** -0.5, mask=dict(size=chunk),
+                                              rot=dict(base=5e5, dims=ad)))
+    mix_l = dict(type="latent_attention", mixer=dict(heads=lh, dim=ld, rot_dim=lr, vdim=lv, kv_rank=rank, scale=(ld + lr) ** -0.5,
+                                                     mask=dict(size=win), rot=dict(base=1e5, dims=lr)))
+    mix_g = dict(type="gla", mixer=dict(heads=gh, dim=gd, vdim=gv, tau=16.0, rank=16))
+    mlp = dict(kind="dense", ff=size["ff"])
+    layers = [dict(m, mlp=mlp) for m in (mix_g, mix_l, mix_a, mix_l)][:LAYERS]
+    return dict(architecture="Lalasun", vocab=VOCAB, width=size["width"], residual_mult=0.4, norm=dict(eps=1e-6), layers=layers)
 
 
 def _say(msg: str) -> None:
@@ -824,6 +848,217 @@ def run_vogerax(sizes: list, seqs: int = 4, plen: int = 2048, rows: int = 64, ct
                 dtype="bf16", data="synthetic", sizes=res)
 
 
+def _kernels_lalasun(size: dict, ksize: dict, zsize: dict, dev, T: int, ctx: int, rows: int) -> dict:
+    """Lalasun's kernels and their closest existing kernels at this size: seconds, and the fraction of the roofline
+    reached.  ``ksize``, ``zsize``: the Kalesun and Zokunex sizes of the same width (for the kernels it stands beside)."""
+    from chronos import ops
+    from chronos.models.hybrid import rope_cos_sin
+    from chronos.ops import hybrid as hops
+
+    out = {}
+    bf = torch.bfloat16
+    d = size["width"]
+    g = torch.Generator(device=dev).manual_seed(1)
+    rnd = lambda *s, dt=bf, sc=1.0: (torch.randn(*s, device=dev, generator=g) * sc).to(dt)  # noqa: E731
+    f32 = lambda *s, sc=1.0: rnd(*s, dt=torch.float32, sc=sc)  # noqa: E731
+    i32 = dict(dtype=torch.int32, device=dev)
+
+    def rec(name, secs, nbytes=0.0, flops=0.0):
+        roof = max(nbytes / HBM_BPS, flops / BF16_FLOPS)
+        _say(f"  {name}: {secs * 1e6:.1f} us, roofline {roof * 1e6:.2f} us")
+        out[name] = dict(us=round(secs * 1e6, 1), roofline_us=round(roof * 1e6, 2), of_roofline=round(roof / secs, 4))
+
+    bs = 16
+    seqs = max(1, T // ctx)
+    n = seqs * ctx
+    per = ctx // bs + 1
+    nb = max(seqs, rows) * per + 1
+    bt = torch.arange(1, 1 + seqs * per, **i32).view(seqs, per)
+    qs = torch.arange(0, (seqs + 1) * ctx, ctx, **i32)
+    pos = torch.arange(ctx, **i32).repeat(seqs)
+    tseq = torch.arange(seqs, **i32).repeat_interleave(ctx)
+    btd = torch.arange(1, 1 + rows * per, **i32).view(rows, per)
+    qsd = torch.arange(rows + 1, **i32)
+    posd = torch.full((rows,), ctx, **i32)
+    NS = max(seqs, rows) + 1
+    p0, sl, sld = torch.zeros(seqs, **i32), torch.arange(seqs, **i32), torch.arange(rows, **i32)
+    full_pairs = n * (ctx + 1) / 2
+    # ---- the stream's joins (gate, multiply, add, next norm; at a layer's end also the depth average)
+    y, x32, w1 = rnd(T, d), f32(T, d), f32(d)
+    wba, gb = torch.cat([w1, f32(d, sc=0.1), torch.tensor([0.7], device=dev)]), f32(d, sc=0.1)
+    F = size["ff"]
+    src = rnd(T, F + d)   # the gate's columns lie behind the feed-forward's up-projection
+    for run in (0, 2):
+        hist, dwa = f32(LAYERS, T, d), f32(run + 2, sc=0.3)
+        rec(f"gated_join.depth_average_{run + 2}", _time(lambda: hops.gated_join(y, x32, src, F, gb, 0.4, wba, bf, hist, run, dwa)),
+            T * d * (2 + 2 + 4 + 4 + 2 + 4 * (run + 1) + 4))
+    del hist
+    rec("gated_join", _time(lambda: hops.gated_join(y, x32, src, F, gb, 0.4, wba, bf)), T * d * (2 + 2 + 4 + 4 + 2))
+    yd, xd, srcd = rnd(rows, d), f32(rows, d), rnd(rows, F + d)
+    rec("gated_join.decode", _time(lambda: hops.gated_join(yd, xd, srcd, F, gb, 0.4, wba, bf)), rows * d * 14.0)
+    rec("kalesun.scale_add_rms_norm.decode", _time(lambda: hops.scale_add_rms_norm(yd, xd, w1, 1.0, 1e-6, bf)), rows * d * 12.0)
+    rec("dyn_tanh", _time(lambda: hops.dyn_tanh(x32, wba, bf)), T * d * (4 + 2))
+    rec("rms_norm", _time(lambda: hops.rms_norm(x32, w1, 1e-6, bf)), T * d * (4 + 2))
+    rec("kalesun.scale_add_rms_norm", _time(lambda: hops.scale_add_rms_norm(y, x32, w1, 1.0, 1e-6, bf)), T * d * (2 + 4 + 4 + 2))
+    rec("zokunex.add_layer_norm", _time(lambda: hops.add_layer_norm(y, x32, w1, 1e-6, bf)), T * d * (2 + 4 + 4 + 2))
+    xb, wb = rnd(T, d), rnd(d)
+    rec("llama.add_rmsnorm", _time(lambda: ops.add_rmsnorm(y, xb, wb, 1e-5)), T * d * (2 + 2 + 2 + 2))
+    # ---- chunked attention with one added to the denominator beside Kalesun's window of the same span and Llama's
+    H, G, D, Dv, chunk = size["a"]
+    kc, vc = rnd(nb, bs, G, D, sc=0.3), rnd(nb, bs, G, Dv, sc=0.3)
+    C = (H + G) * D + G * Dv + d    # (the residual gate's rows ride along)
+    qkv, qkvd = rnd(n, C, sc=0.3), rnd(rows, C, sc=0.3)
+    tab = rope_cos_sin(5e5, D, ctx + 2, dev)
+    zero = torch.zeros(H, device=dev)
+    vis = sum(i % chunk + 1 for i in range(ctx))
+    rec("chunk_attention.prefill", _time(lambda: hops.window_attention(qkv, kc, vc, bt, qs, pos, zero, None, D ** -0.5, 0, 0, H, bf, ctx, chunk), iters=3, warm=1),
+        flops=2.0 * seqs * vis * H * (D + Dv))
+    posc = torch.full((rows,), (ctx // chunk) * chunk - 1, **i32)   # the last position of a chunk: all of it is visible
+    rec("chunk_attention.decode", _time(lambda: hops.window_attention(qkvd, kc, vc, btd, qsd, posc, zero, None, D ** -0.5, 0, 0, H, bf, 1, chunk)),
+        nbytes=rows * chunk * G * (D + Dv) * 2.0)
+    rec("window_prep.rotated.prefill", _time(lambda: hops.window_prep(qkv, H, G, D, Dv, None, None, pos, tseq, bt, None, None, 1e-5, tab, D, kc, vc, False)),
+        nbytes=n * (2 * (H + G) * D + 2 * G * Dv) * 2.0)
+    kH, kG, kD, kDv, kwin, keep = ksize["a"]
+    kkc, kvc = rnd(nb, bs, kG, kD, sc=0.3), rnd(nb, bs, kG, kDv, sc=0.3)
+    kqkv, kqkvd = rnd(n, (kH + kG) * kD + kG * kDv, sc=0.3), rnd(rows, (kH + kG) * kD + kG * kDv, sc=0.3)
+    kgate, kgated, ksink = f32(n, kH), f32(rows, kH), f32(kH)
+    qn, kn, ktab = f32(kD), f32(kD), rope_cos_sin(5e5, kD // 2, ctx + 2, dev)
+    kvis = sum(min(i + 1, kwin) + max(0, min(keep, i + 1 - kwin)) for i in range(ctx))
+    rec("kalesun.window_attention.prefill", _time(lambda: hops.window_attention(kqkv, kkc, kvc, bt, qs, pos, ksink, kgate, kD ** -0.5, kwin, keep, kH, bf, ctx), iters=3, warm=1),
+        flops=2.0 * seqs * kvis * kH * (kD + kDv))
+    rec("kalesun.window_attention.decode", _time(lambda: hops.window_attention(kqkvd, kkc, kvc, btd, qsd, posd, ksink, kgated, kD ** -0.5, kwin, keep, kH, bf, 1)),
+        nbytes=rows * (min(ctx + 1, kwin) + keep) * kG * (kD + kDv) * 2.0)
+    rec("kalesun.window_prep.prefill", _time(lambda: hops.window_prep(kqkv, kH, kG, kD, kDv, None, None, pos, tseq, bt, qn, kn, 1e-5, ktab, kD // 2, kkc, kvc, False)),
+        nbytes=n * (2 * (kH + kG) * kD + 2 * kG * kDv) * 2.0)
+    hq = d // 128
+    hkv = max(1, hq // 4)
+    akc, avc = rnd(nb, hkv, bs, 128, sc=0.3), rnd(nb, hkv, 128, bs, sc=0.3)
+    q, qd = rnd(n, hq, 128, sc=0.3), rnd(rows, hq, 128, sc=0.3)
+    ctxl, ctxd = torch.full((seqs,), ctx, **i32), torch.full((rows,), ctx + 1, **i32)
+    tiles = torch.tensor(ops.attention_tiles([ctx] * seqs, hq, hkv, 8), **i32).view(-1, 2)
+    rec("llama.attention.prefill", _time(lambda: ops.paged_attention(q, akc, avc, bt, qs, ctxl, tiles, tiles.shape[0], 8, 1), iters=3, warm=1),
+        flops=4.0 * full_pairs * hq * 128)
+    ns = ops.pick_nsplit(rows * hkv, ctx + 1)
+    rec("llama.attention.decode", _time(lambda: ops.paged_attention(qd, akc, avc, btd, qsd, ctxd, None, rows, 1, ns)),
+        nbytes=rows * (ctx + 1) * hkv * 128 * 2 * 2.0)
+    del kc, vc, kkc, kvc, akc, avc, qkv, kqkv, q
+    # ---- latent attention through a window (two-term weights) beside Zokunex's causal latent attention
+    H, D, R, Dv, rank, win = size["l"]
+    DK, nq = rank + R, H * (D + R)
+    lat = rnd(nb, bs, DK, sc=0.3)
+    Cl = nq + DK + H * Dv + d
+    proj, projd = rnd(n, Cl, sc=0.3), rnd(rows, Cl, sc=0.3)
+    qa, qad = rnd(n, H, DK, sc=0.3), rnd(rows, H, DK, sc=0.3)
+    ltab, wn = rope_cos_sin(1e5, R, ctx + 2, dev), f32(rank)
+    wvis = sum(min(i + 1, win) for i in range(ctx))
+    rec("latent_window.prefill", _time(lambda: hops.latent_attention(qa, lat, bt, qs, pos, None, 0.1, rank, bf, ctx, win, True), iters=3, warm=1),
+        flops=2.0 * seqs * wvis * H * (DK + rank))
+    rec("latent_window.prefill.one_term", _time(lambda: hops.latent_attention(qa, lat, bt, qs, pos, None, 0.1, rank, bf, ctx, win, False), iters=3, warm=1),
+        flops=2.0 * seqs * wvis * H * (DK + rank))
+    rec("latent_window.decode", _time(lambda: hops.latent_attention(qad, lat, btd, qsd, posd, None, 0.1, rank, bf, 1, win, True)),
+        nbytes=rows * min(ctx + 1, win) * DK * 2.0)
+    rec("latent_prep.prefill", _time(lambda: hops.latent_prep(proj[:, :nq].view(n, H, D + R), proj[:, nq:nq + DK], pos, tseq, bt, wn, 1e-5, ltab, R, rank, lat, qa, True)),
+        nbytes=n * (2 * DK + 2 * H * R) * 2.0)
+    zH, zD, zR, zDv, zrank = zsize["a"]
+    zlat = rnd(nb, bs, zrank + zR, sc=0.3)
+    zqa, zqad = rnd(n, zH, zrank + zR, sc=0.3), rnd(rows, zH, zrank + zR, sc=0.3)
+    zg, zgd = f32(n, zH), f32(rows, zH)
+    rec("zokunex.latent_attention.prefill", _time(lambda: hops.latent_attention(zqa, zlat, bt, qs, pos, zg, 0.1, zrank, bf, ctx), iters=3, warm=1),
+        flops=2.0 * full_pairs * zH * (2 * zrank + zR))
+    rec("zokunex.latent_attention.decode", _time(lambda: hops.latent_attention(zqad, zlat, btd, qsd, posd, zgd, 0.1, zrank, bf, 1)),
+        nbytes=rows * (ctx + 1) * (zrank + zR) * 2.0)
+    # per-head products beside the library's batched product (which leaves the result in another layout)
+    wuk, wuv = rnd(H, rank, D, sc=D ** -0.5), rnd(H, Dv, rank, sc=rank ** -0.5)
+    ukt, uvt = wuk.transpose(1, 2).contiguous(), wuv.transpose(1, 2).contiguous()
+    for name, m, pr, qx in (("prefill", n, proj, qa), ("decode", rows, projd, qad)):
+        qv = pr[:, :nq].view(m, H, D + R)[:, :, :D]
+        oa = rnd(m, H, rank)
+        nb1, fl = (m * H * (D + rank) + H * D * rank) * 2.0, 2.0 * m * H * D * rank
+        rec(f"head_matmul.to_latent.{name}", _time(lambda: hops.head_matmul(qv, wuk, qx[:, :, :rank])), nbytes=nb1, flops=fl)
+        rec(f"library.bmm.to_latent.{name}", _time(lambda: torch.bmm(qv.transpose(0, 1), ukt)), nbytes=nb1, flops=fl)
+        nb2 = (m * H * (2 * Dv + rank) + H * Dv * rank) * 2.0
+        rec(f"head_matmul.from_latent_gated.{name}", _time(lambda: hops.head_matmul(oa, wuv, None, pr, nq + DK)), nbytes=nb2, flops=2.0 * m * H * Dv * rank)
+        rec(f"library.bmm.from_latent.{name}", _time(lambda: torch.bmm(oa.transpose(0, 1), uvt)), nbytes=nb2 - m * H * Dv * 2.0, flops=2.0 * m * H * Dv * rank)
+    del lat, zlat, proj, qa, zqa, oa
+    # ---- gated linear attention: Kalesun's kernels
+    gh, gd, gv = size["g"]
+    S = torch.zeros(NS, gh, gd, gv, device=dev)
+    gproj, gprojd = rnd(n, 2 * gh * gd + 2 * gh * gv + d, sc=0.5), rnd(rows, 2 * gh * gd + 2 * gh * gv + d, sc=0.5)
+    gdec, gdecd = torch.rand(n, gh, gd, device=dev), torch.rand(rows, gh, gd, device=dev)
+    rec("linear_scan.gla.prefill", _time(lambda: hops.linear_scan(gproj, 0, gh * gd, 2 * gh * gd, None, None, gd ** -0.5, gdec, None, qs, p0, sl, S, gh, gh, gd, gv), iters=3, warm=1),
+        nbytes=n * (2 * gh * gd + gh * gv) * 2.0, flops=n * gh * gd * gv * 4.0)
+    rec("linear_scan.gla.decode", _time(lambda: hops.linear_scan(gprojd, 0, gh * gd, 2 * gh * gd, None, None, gd ** -0.5, gdecd, None, qsd, posd, sld, S, gh, gh, gd, gv)),
+        nbytes=rows * gh * gd * gv * 4 * 2.0)
+    kgh, kgd, kgv = ksize["g"]
+    kS = torch.zeros(NS, kgh, kgd, kgv, device=dev)
+    kproj = rnd(n, 2 * kgh * kgd + 2 * kgh * kgv, sc=0.5)
+    kdec = torch.rand(n, kgh, kgd, device=dev)
+    rec("kalesun.linear_scan.gla.prefill", _time(lambda: hops.linear_scan(kproj, 0, kgh * kgd, 2 * kgh * kgd, None, None, kgd ** -0.5, kdec, None, qs, p0, sl, kS, kgh, kgh, kgd, kgv), iters=3, warm=1),
+        nbytes=n * (2 * kgh * kgd + kgh * kgv) * 2.0, flops=n * kgh * kgd * kgv * 4.0)
+    # ---- feed-forwards: PolyNorm beside Zokunex's activation in place and Kalesun's gated unit, then whole units
+    abce = torch.tensor([0.6, -0.3, 0.2, 0.1], device=dev)
+    kff, zff, lf = ksize["ff"], zsize["ff"], int(3.5 * d)
+    wup, wdn = rnd(F + d, d, sc=d ** -0.5), rnd(d, F, sc=F ** -0.5)
+    kgu, kdn = rnd(2 * kff, d, sc=d ** -0.5), rnd(d, kff, sc=kff ** -0.5)
+    zup, zdn = rnd(zff, d, sc=d ** -0.5), rnd(d, zff, sc=zff ** -0.5)
+    lgu, ldn = rnd(2 * lf, d, sc=d ** -0.5), rnd(d, lf, sc=lf ** -0.5)
+    for name, tk in (("prefill", T), ("decode", rows)):
+        h, z, kz = rnd(tk, d), rnd(tk, F + d), rnd(tk, 2 * kff)
+        zz = rnd(tk, zff)
+        rec(f"poly_norm.{name}", _time(lambda: hops.poly_norm(z, F, abce, 1e-6, bf)), nbytes=tk * F * 4.0)
+        rec(f"zokunex.act.{name}", _time(lambda: hops.act_inplace(zz, hops.ACT_RELU2)), nbytes=tk * zff * 4.0)
+        rec(f"kalesun.glu.{name}", _time(lambda: hops.glu(kz, 7.0, 1.702, 1.0, bf)), nbytes=tk * kff * 6.0)
+        rec(f"poly_ff.{name}", _time(lambda: hops.matmul(hops.poly_norm(hops.matmul(h, wup), F, abce, 1e-6, bf), wdn), iters=3, warm=1),
+            nbytes=(2 * F + d) * d * 2.0 + tk * d * 4.0, flops=tk * 2.0 * (2 * F + d) * d)
+        rec(f"zokunex.dense_ff.{name}", _time(lambda: hops.matmul(hops.act_inplace(hops.matmul(h, zup), hops.ACT_RELU2), zdn), iters=3, warm=1),
+            nbytes=2 * zff * d * 2.0 + tk * d * 4.0, flops=tk * 4.0 * zff * d)
+        rec(f"kalesun.glu_ff.{name}", _time(lambda: hops.matmul(hops.glu(hops.matmul(h, kgu), 7.0, 1.702, 1.0, bf), kdn), iters=3, warm=1),
+            nbytes=3 * kff * d * 2.0 + tk * d * 4.0, flops=tk * 6.0 * kff * d)
+        rec(f"llama.mlp.{name}", _time(lambda: ops.linear(ops.gate_up_silu(h, lgu), ldn), iters=3, warm=1),
+            nbytes=3 * lf * d * 2.0 + tk * d * 4.0, flops=tk * 6.0 * lf * d)
+    return out
+
+
+def run_lalasun(sizes: list, seqs: int = 4, plen: int = 2048, rows: int = 64, ctx: int = 2048, device: str = "cuda") -> dict:
+    from chronos import ops
+    from chronos.models import kalesun, lalasun, llama, zokunex
+    from chronos.models.hybrid import HybridDecoder
+
+    dev = torch.device(device if ":" in device else device + ":0")
+    torch.cuda.set_device(dev)
+    ops.load()
+    ops.device_init()
+    res = {}
+    P = ctx + plen + 16
+    for name in sizes:
+        size, ksize, zsize = LALASUN_SIZES[name], KALESUN_SIZES[name], SIZES[name]
+        t0 = time.time()
+        entry = {}
+        for mod, key, conf in ((lalasun, "lalasun", lalasun_config(size)), (kalesun, "kalesun", kalesun_config(ksize)),
+                               (zokunex, "zokunex", zokunex_config(zsize))):
+            cfg = mod.config_from_dict(conf, name=f"{key}-{name}", max_position=P)
+            m = HybridDecoder(cfg, mod.pack_weights(cfg, mod.random_tensors(cfg, 0), dev, torch.bfloat16), dev, P, torch.bfloat16)
+            entry[key] = dict(params=cfg.param_count(), **_model_steps(m, dev, seqs, plen, rows, ctx))
+            _say(f"size {name}: {key} {entry[key]}")
+            del m
+        d = size["width"]
+        lc = llama.LlamaConfig(name=f"llama-{name}", vocab_size=VOCAB, hidden_size=d, intermediate_size=int(3.5 * d),
+                               num_layers=LAYERS, num_heads=d // 128, num_kv_heads=max(1, d // 512), max_position=P)
+        lm = llama.LlamaModel(lc, llama.random_weights(lc, None, dev, 0), None, dev, P)
+        entry["llama"] = dict(params=lc.param_count(), **_model_steps(lm, dev, seqs, plen, rows, ctx))
+        _say(f"  llama {entry['llama']}")
+        del lm
+        torch.cuda.empty_cache()
+        entry["kernels"] = _kernels_lalasun(size, ksize, zsize, dev, seqs * plen, ctx, rows)
+        entry["seconds"] = round(time.time() - t0, 1)
+        res[name] = entry
+        torch.cuda.empty_cache()
+    return dict(metric="design_compare", design="lalasun", beside="kalesun, zokunex and llama (equal width and depth)",
+                layers=LAYERS, workload=dict(prefill=f"{seqs} x {plen} tokens in one step",
+                                             decode=f"{rows} rows at context {ctx}"),
+                dtype="bf16", data="synthetic", sizes=res)
+
+
 def run_kalesun(sizes: list, seqs: int = 4, plen: int = 2048, rows: int = 64, ctx: int = 2048, device: str = "cuda") -> dict:
     from chronos import ops
     from chronos.models import kalesun, llama, zokunex
@@ -906,7 +1141,8 @@ def run(sizes: list, seqs: int = 4, plen: int = 2048, rows: int = 64, ctx: int =
 
 def main(a) -> int:
     sizes = [s for s in a.design_sizes.split(",") if s]
-    fn = {"kalesun": run_kalesun, "tugovik": run_tugovik, "vogerax": run_vogerax}.get(getattr(a, "design", "zokunex"), run)
+    fn = {"kalesun": run_kalesun, "tugovik": run_tugovik, "vogerax": run_vogerax,
+          "lalasun": run_lalasun}.get(getattr(a, "design", "zokunex"), run)
     out = fn(sizes, device=a.device)
     print(json.dumps(out), flush=True)
     return 0
