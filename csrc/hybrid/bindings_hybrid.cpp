@@ -36,7 +36,7 @@ bool launch_hy_latent_attention(const void*, const void*, const int32_t*, int, c
                                 float*, int64_t,
                                 hipStream_t);
 bool hy_latent_use_mfma(bool, int, int);
-int hy_latent_nsplit(int, int);
+int hy_latent_nsplit(int, int, bool);
 void launch_hy_moe_route(const void*, const void*, const float*, float*, int32_t*, float*, int, int, int, int, bool,
                          hipStream_t);
 void launch_hy_moe_ffn_token(const void*, const int32_t*, const float*, const void*, const void*, void*, int, int, int,
@@ -337,7 +337,7 @@ Tensor hy_latent_attention(const Tensor& qa, const Tensor& cache, const Tensor& 
     if (chronos::hy_latent_use_mfma(f32(qa), (int)DK, (int)rank)) {
         int64_t span = block_table.size(1) * cache.size(1);   // keys a row block walks at most
         if (window > 0) span = std::min<int64_t>(span, window + mq);
-        nsplit = chronos::hy_latent_nsplit((int)(B * ((mq * H + 63) / 64)), (int)span);
+        nsplit = chronos::hy_latent_nsplit((int)(B * ((mq * H + 63) / 64)), (int)span, window > 0);
         if (nsplit > 1) {
             part_o = at::empty({T * H * nsplit, rank}, qa.options().dtype(at::kFloat));
             part_ml = at::empty({T * H * nsplit, 2}, qa.options().dtype(at::kFloat));

@@ -267,10 +267,11 @@ static void la_mfma_launch(const uint16_t* qa, const uint16_t* cache, const int3
 bool hy_latent_mfma_ok(int DK, int rank) { return !(DK % 8 || rank % 16 || DK > 576 || rank > 512 || rank > DK); }
 
 // Splits of the key range (flash-decoding) for a launch of `wgs` workgroups over contexts of at most max_ctx keys:
-// enough workgroups to cover the chip, at least 4 key tiles per split, at most 16.
-int hy_latent_nsplit(int wgs, int max_ctx) {
+// enough workgroups to cover the chip, at least 4 key tiles per split (2 behind a window, whose few tiles are all of the
+// walk), at most 16.
+int hy_latent_nsplit(int wgs, int max_ctx, bool windowed) {
     if (wgs >= 128) return 1;
-    int want = (256 + wgs - 1) / wgs, cap = max_ctx / (4 * hy::MKT);
+    int want = (256 + wgs - 1) / wgs, cap = max_ctx / ((windowed ? 2 : 4) * hy::MKT);
     if (want > 16) want = 16;
     if (want > cap) want = cap;
     return want < 1 ? 1 : want;
