@@ -218,29 +218,29 @@ __global__ void __launch_bounds__(64 * NW) latent_attention_mfma_kernel(
         }
 }
 
-// one wave per (token, head) row: out = sum_z exp(m_z - m) O_z / sum_z exp(m_z - m) l_z * sigmoid(gate)
+// one wave per (token, head) row: out = sum_z exp(m_z - m) O_z / sum_z exp(m_z - m) l_z * sigmoid(gate).  Lane z holds
+// split z's maximum and sum (nsplit <= 16); a lane then sums 4 neighbouring columns over the splits, whose loads do not
+// depend on each other.
 __global__ void __launch_bounds__(256) latent_combine_kernel(const float* __restrict__ part_o, const float* __restrict__ part_ml,
                                                              const float* __restrict__ gate, uint16_t* __restrict__ out,
                                                              int64_t rows, int rank, int nsplit) {
     const int lane = threadIdx.x & 63;
     const int64_t r = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
     if (r >= rows) return;
-    float m = -INFINITY;
-    for (int z = 0; z < nsplit; ++z) m = fmaxf(m, part_ml[(r * nsplit + z) * 2]);
-    float l = 0.f;
-    for (int z = 0; z < nsplit; ++z) {
-        const float mz = part_ml[(r * nsplit + z) * 2];
-        if (mz != -INFINITY) l += expf(mz - m) * part_ml[(r * nsplit + z) * 2 + 1];
-    }
-    float f = 1.f / l;
-    if (gate != nullptr) f *= sigmoidf_(gate[r]);
-    for (int c = lane; c < rank; c += 64) {
-        float acc = 0.f;
+    const float mz = lane < nsplit ? part_ml[(r * nsplit + lane) * 2] : -INFINITY;
+    const float lz = lane < nsplit ? part_ml[(r * nsplit + lane) * 2 + 1] : 0.f;
+    const float m = wave_max(mz);
+    float e = mz == -INFINITY ? 0.f : expf(mz - m);   // (a split without a visible key adds nothing)
+    const float l = wave_sum(e * lz);
+    e *= (gate != nullptr ? sigmoidf_(gate[r]) : 1.f) / l;
+    for (int c = lane * 4; c < rank; c += 256) {      // (rank is a multiple of 16)
+        f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
         for (int z = 0; z < nsplit; ++z) {
-            const float mz = part_ml[(r * nsplit + z) * 2];
-            if (mz != -INFINITY) acc += expf(mz - m) * part_o[(r * nsplit + z) * rank + c];
+            const float w = __uint_as_float(__builtin_amdgcn_readlane(__float_as_uint(e), z));
+            acc += w * *reinterpret_cast<const f32x4*>(part_o + (r * nsplit + z) * rank + c);
         }
-        out[r * rank + c] = f2bf(acc * f);
+        *reinterpret_cast<u16x4*>(out + r * rank + c) = u16x4{f2bf(acc[0]), f2bf(acc[1]), f2bf(acc[2]), f2bf(acc[3])};
     }
 }
 
