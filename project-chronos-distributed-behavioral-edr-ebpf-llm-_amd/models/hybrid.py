@@ -4,10 +4,12 @@ linear recurrence, retention, two mixers side by side) and an optional feed-forw
 experts), on a float32 residual stream.
 The stream's rule is a parameter of the configuration: the norm on the sublayer's OUTPUT (``out_norm``:
 x <- x + layer_norm(sublayer(x))), AFTER the sum (``post_norm``: x <- rms_norm(alpha x + sublayer(x))), on the
-sublayer's INPUT (``pre_norm``: x <- x + sublayer(rms_norm(x))) or on both sides (``sandwich``:
-x <- x + norm_b(sublayer(norm_a(x))), RMS norms over ``norm_groups`` equal parts of the row).  A pre-norm stream may
+sublayer's INPUT (``pre_norm``: x <- x + sublayer(rms_norm(x))), on both sides (``sandwich``:
+x <- x + norm_b(sublayer(norm_a(x))), RMS norms over ``norm_groups`` equal parts of the row), or one norm that both
+sublayers of a layer read (``parallel``: x <- x + mixer(h) + ff(h), h = layer_norm(x)).  A pre-norm stream may
 use Dynamic Tanh in place of the RMS norm, scale what it adds, gate every sublayer's result by a projection of what
-the sublayer read, and hand on weighted sums of all earlier layers' results.  A range of layers may repeat, back to back, on shared weights (``loop``), or single layers may name another layer whose weights they use
+the sublayer read, and hand on weighted sums of all earlier layers' results.  A range of layers may repeat, back to
+back, on shared weights (``loop``), or single layers may name another layer whose weights they use
 (``share``); every run has its own pages and state.
 
 This module is the design-independent part: the mixer and feed-forward kinds with their sizes and constants as
@@ -49,9 +51,11 @@ class MLSTMSpec:
 class LatentAttentionSpec:
     """Attention whose keys and values are up-projections of one cached low-rank latent per token, plus a rotated key
     part shared by all heads; through a sliding window or over the whole prefix; a sigmoid output gate (one number per
-    head, or with ``gate_wide`` one per output column).  ``rope_interleaved``: neighbouring columns form the rotated
-    pairs (else column i pairs with i + rope_dims / 2).  ``two_term``: on the matrix cores the softmax weights enter
-    the weighted sum as two bfloat16 terms each."""
+    head, or with ``gate_wide`` one per output column; none with ``gate`` off).  ``rope_interleaved``: neighbouring
+    columns form the rotated pairs (else column i pairs with i + rope_dims / 2).  ``two_term``: on the matrix cores
+    the softmax weights enter the weighted sum as two bfloat16 terms each.  ``q_rank`` > 0: the queries are
+    up-projections of an RMS-normed latent of that size.  ``sink``: a learned softmax sink per head.  ``kv_from``: the
+    layer writes no latents, it reads the pages of that earlier layer (same kv_rank, rot_dim and rotation)."""
     heads: int
     dim: int        # unrotated query / key columns per head
     rot_dim: int    # rotated columns per head (the shared rotated key has as many)
@@ -64,7 +68,20 @@ class LatentAttentionSpec:
     rope_interleaved: bool = False
     gate_wide: bool = False
     two_term: bool = False
+    gate: bool = True
+    q_rank: int = 0
+    sink: bool = False
+    kv_from: Optional[int] = None
+    rope_scaling: Optional[tuple] = None   # see rope_cos_sin
     kind: str = "latent_attention"
+
+    def params(self, d: int) -> int:
+        nq = self.heads * (self.dim + self.rot_dim)
+        n = self.q_rank * (d + 1 + nq) if self.q_rank else d * nq
+        n += d * self.heads * (self.vdim if self.gate_wide else 1) * self.gate + self.heads * self.sink
+        if self.kv_from is None:
+            n += d * (self.kv_rank + self.rot_dim) + self.kv_rank
+        return n + self.kv_rank * self.heads * (self.dim + self.vdim) + self.heads * self.vdim * d
 
 
 @dataclass
@@ -102,9 +119,14 @@ class WindowAttentionSpec:
     first such layer, and a sigmoid output gate (one number per head, or with ``gate_wide`` one per output column).
     ``pool`` > 0 (with a window): beside the window's tokens a query sees one key and value per block of ``pool``
     positions that lies wholly before its window — the means of the block's cached keys and values.  ``v_from_k``:
-    there is no value projection, the values are the keys as projected (before norm and rotation).  ``v_rot``: values
+    there is no value projection, the values are the keys before norm and rotation.  ``v_rot``: values
     are cached rotated by their position over all ``vdim`` columns (frequencies rope_base^(-2m/vdim), unscaled) and
-    every head's output is turned back by the query's position."""
+    every head's output is turned back by the query's position.  ``conv`` > 0: queries, keys and values pass a short
+    causal convolution of that many taps right after the projection.  ``q_temp`` = (coef, every): queries are multiplied
+    by 1 + coef ln(floor((p + 1) / every) + 1) at position p.
+
+    Where keys are values divided by their root mean square (``v_from_k``, a norm without weights, no rotation) only
+    the values are cached, and one float32 number per token and head: ``unit_keys``."""
     heads: int
     kv_heads: int
     dim: int
@@ -128,12 +150,20 @@ class WindowAttentionSpec:
     gate_wide: bool = False  # the sigmoid output gate has heads * vdim rows instead of heads
     sink_fixed: Optional[float] = None  # with ``sink``: every head's sink score is this constant (no weights)
     bias_o: bool = False     # the output projection adds a bias
+    conv: int = 0            # > 0: taps of a causal convolution over time on the projected columns
+    qk_norm_weight: bool = True   # with ``qk_norm``: the norms of queries and keys have weights
+    q_temp: Optional[tuple] = None  # (coef, every): the queries' temperature by position
     kind: str = "window_attention"
+
+    @property
+    def unit_keys(self) -> bool:
+        return self.v_from_k and self.qk_norm and not self.qk_norm_weight and not self.rope_dims and not self.v_rot \
+            and not self.v_mix and not self.pool and self.dim == self.vdim
 
     def params(self, d: int) -> int:
         qkv = self.heads * self.dim + self.kv_heads * (self.dim + (0 if self.v_from_k else self.vdim))
         gate = self.heads * (self.vdim if self.gate_wide else 1) * self.gate
-        return d * (qkv + gate) + 2 * self.dim * self.qk_norm + \
+        return d * (qkv + gate) + qkv * self.conv + 2 * self.dim * (self.qk_norm and self.qk_norm_weight) + \
             (self.heads if self.sink and self.sink_fixed is None else 0) + self.bias_o * d + \
             (1 if self.v_mix and not self.v_mix_first else 0) + \
             self.heads * self.vdim * d + qkv * self.bias
@@ -304,14 +334,16 @@ class HybridConfig:
     architecture: str = "hybrid"
     residual: str = "out_norm"     # "out_norm": x <- x + layer_norm(y);  "post_norm": x <- rms_norm(alpha x + y);
     #                                "pre_norm": x <- x + sublayer(rms_norm(x));
-    #                                "sandwich": x <- x + norm_b(sublayer(norm_a(x)))
+    #                                "sandwich": x <- x + norm_b(sublayer(norm_a(x)));
+    #                                "parallel": x <- x + mixer(h) + ff(h), h = norm(x)
     norm_groups: int = 1           # sandwich: the stream's RMS norms work on this many equal parts of a row
     embed_scale: float = 1.0       # the embedding rows are multiplied by this
     share: Optional[list] = None   # share[i] = j: layer i runs on layer j's weights (j itself has its own)
     residual_alpha: float = 1.0
     tied_head: bool = False        # the logits come from the embedding table
     loop: Optional[tuple] = None   # (start, stop, times): layers [start, stop) run ``times`` times, back to back
-    norm: str = "rms"              # pre_norm: the stream's norms, "rms" or "tanh" (Dynamic Tanh: tanh(alpha x) w + b)
+    norm: str = "rms"              # pre_norm: the stream's norms, "rms" or "tanh" (Dynamic Tanh: tanh(alpha x) w + b);
+    #                                parallel: "layer" (layer norm with weight and bias)
     residual_mult: float = 1.0     # pre_norm: x <- x + residual_mult * sublayer(norm(x))
     residual_gate: bool = False    # pre_norm: a sublayer's result times sigmoid(W h + b), h what the sublayer read
     depth_average: bool = False    # pre_norm: after layer i the stream is sum_j dwa_i[j] X_j over the embedding output
@@ -336,7 +368,8 @@ class HybridConfig:
 
     def param_count(self) -> int:
         d = self.hidden_size
-        n = (1 if self.tied_head else 2) * self.vocab_size * d + d + (d + 1 if self.norm == "tanh" else 0)
+        extra = {"tanh": d + 1, "layer": d}.get(self.norm, 0)     # what a norm carries beside its weight
+        n = (1 if self.tied_head else 2) * self.vocab_size * d + d + extra
         own = set(self.runs)
         for i, l in enumerate(self.layers):
             if i not in own:
@@ -346,19 +379,14 @@ class HybridConfig:
                 n += m.params(d)
             elif m.kind == "mlstm":
                 n += d * (2 * m.heads * m.dim + 2 * m.heads * m.vdim) + 2 * m.heads * (d + 1) + m.heads * m.vdim * (d + 1)
-            else:
-                gates = m.heads * (m.vdim if m.gate_wide else 1)
-                n += d * (m.heads * (m.dim + m.rot_dim) + m.kv_rank + m.rot_dim + gates) + m.kv_rank
-                n += m.kv_rank * m.heads * (m.dim + m.vdim) + m.heads * m.vdim * d
             sub = d * (2 if self.residual == "sandwich" else 1)    # what every sublayer carries beside its own weights
-            if self.norm == "tanh":
-                sub += d + 1
+            sub += extra
             if self.residual_gate:
                 sub += d * (d + 1)
             n += sub + (i + 2 if self.depth_average else 0)
             if l.ff is not None:
                 f = l.ff
-                n += sub
+                n += sub if self.residual != "parallel" else 0     # (one norm for both sublayers)
                 n += {"dense": lambda: 2 * d * f.ff, "poly": lambda: 2 * d * f.ff + 4, "glu": lambda: 3 * d * f.ff,
                       "moe": lambda: (f.experts * f.ff + f.shared_ff) * 2 * d + (f.experts + f.identity) * (d + f.correction),
                       "moe_glu": lambda: f.experts * (3 * d * f.ff + d + 1),
@@ -374,10 +402,17 @@ class HybridConfig:
 # -----------------------------------------------------------------------------------------------------------------
 
 
+def _conv_channels(mx: WindowAttentionSpec) -> int:
+    """Columns that pass an attention layer's short convolution: q | k (| v)."""
+    return (mx.heads + mx.kv_heads) * mx.dim + (0 if mx.v_from_k else mx.kv_heads * mx.vdim)
+
+
 class HybridCache:
-    """Per latent-attention layer run a paged latent cache [NB, BS, kv_rank + rot_dim], per windowed-attention run
+    """Per latent-attention layer run a paged latent cache [NB, BS, kv_rank + rot_dim] (a run that reads another layer's
+    latents names the same tensor), per windowed-attention run
     paged keys [NB, BS, G, D] and values [NB, BS, G, Dv] (with pooled blocks also their means, ``kp`` / ``vp``
-    [NB, ceil(BS / pool), G, .]: block e of a sequence sits in row e % EP of the sequence's page e // EP), all in the
+    [NB, ceil(BS / pool), G, .]: block e of a sequence sits in row e % EP of the sequence's page e // EP; where keys are
+    scaled values no keys but their factors, ``ks`` float32 [NB, BS, G]), all else in the
     activation dtype (block 0 is the engine's scratch block); per recurrent run float32 state rows S [NS, H, D, Dv]
     (the matrix-memory layers also n [NS, H, D] and m [NS, H]; the gated linear recurrence keeps S [NS, width];
     layers with a short convolution also its last conv - 1 inputs, ``hist`` [NS, conv - 1, C] in the activation
@@ -399,6 +434,7 @@ class HybridCache:
         self.vc: dict = {}
         self.kp: dict = {}
         self.vp: dict = {}
+        self.ks: dict = {}
         self.hist: dict = {}
         self._dev, self._at = device, act_dtype
         for li, l in enumerate(cfg.layers[i] for i in cfg.runs):
@@ -409,6 +445,8 @@ class HybridCache:
         if mx.kind == "parallel":
             self._alloc((li, 0), mx.left)
             self._alloc((li, 1), mx.right)
+        elif mx.kind == "latent_attention" and mx.kv_from is not None:
+            self.lat[li] = self.lat[mx.kv_from]
         elif mx.kind == "latent_attention":
             self.lat[li] = torch.zeros(num_blocks, block_size, mx.kv_rank + mx.rot_dim, device=device, dtype=act_dtype)
         elif mx.kind == "mlstm":
@@ -418,7 +456,12 @@ class HybridCache:
             self.m[li] = torch.zeros(slots + 1, mx.heads, **f32)
         elif mx.kind == "window_attention":
             pg = dict(device=device, dtype=act_dtype)
-            self.kc[li] = torch.zeros(num_blocks, block_size, mx.kv_heads, mx.dim, **pg)
+            if mx.unit_keys:
+                self.ks[li] = torch.zeros(num_blocks, block_size, mx.kv_heads, device=device, dtype=torch.float32)
+            else:
+                self.kc[li] = torch.zeros(num_blocks, block_size, mx.kv_heads, mx.dim, **pg)
+            if mx.conv:
+                self.hist[li] = torch.zeros(slots + 1, mx.conv - 1, _conv_channels(mx), **pg)
             self.vc[li] = torch.zeros(num_blocks, block_size, mx.kv_heads, mx.vdim, **pg)
             if mx.pool:
                 ep = (block_size + mx.pool - 1) // mx.pool
@@ -440,17 +483,19 @@ class HybridCache:
     def bytes_per_block(cfg: HybridConfig, block_size: int, act_dtype) -> int:
         eb = 4 if act_dtype == torch.float32 else 2
 
-        def per_page(m) -> int:   # elements one page of this mixer holds
+        def per_page(m) -> int:   # bytes one page of this mixer holds
             if m.kind == "parallel":
                 return per_page(m.left) + per_page(m.right)
             if m.kind == "latent_attention":
-                return block_size * (m.kv_rank + m.rot_dim)
+                return block_size * (m.kv_rank + m.rot_dim) * eb if m.kv_from is None else 0
+            if m.kind == "window_attention" and m.unit_keys:
+                return block_size * m.kv_heads * (m.vdim * eb + 4)
             if m.kind == "window_attention":
                 rows = block_size + ((block_size + m.pool - 1) // m.pool if m.pool else 0)
-                return rows * m.kv_heads * (m.dim + m.vdim)
+                return rows * m.kv_heads * (m.dim + m.vdim) * eb
             return 0
 
-        return max(1, sum(per_page(cfg.layers[i].mixer) for i in cfg.runs) * eb)
+        return max(1, sum(per_page(cfg.layers[i].mixer) for i in cfg.runs))
 
     def move_slots(self, src: torch.Tensor, dst: torch.Tensor) -> None:
         """Slot compaction: the recurrent state rows follow their sequences."""
@@ -500,13 +545,50 @@ class HybridWeights:
         return n
 
 
-def _in_proj(rows: list, t: dict, out: dict, key: str, cast) -> None:
-    """out[key] = the sublayer's first projection: ``rows`` stacked and, when t holds "rg" (a residual gate's rows, which
-    read the same input), those last, from column out["rg_off"] on."""
+def _in_proj(rows: list, t: dict, out: dict, key: str, cast, gate: bool = False) -> None:
+    """out[key] = the sublayer's first projection: ``rows`` stacked and behind them what else reads the same input, each
+    from a column of its own on: with t["rg"] a residual gate's rows (out["rg_off"]); with t["ff"] = (spec, gate and up
+    rows, down) the first projection of a gated feed-forward that runs beside the mixer (out["ff"] = its column and
+    its spec) and, with ``gate``, the per-head gate's rows t["g"] (out["g_off"]).  The latter start on multiples of 8
+    columns and end on one of 16 (rows of zeros between)."""
     if "rg" in t:
         out["rg_off"] = sum(r.shape[0] for r in rows)
         rows = rows + [t["rg"]]
+    if "ff" in t:
+        n, stack = 0, []
+
+        def put(r, unit):
+            nonlocal n
+            stack.append(r)
+            n += r.shape[0]
+            pad = -n % unit
+            if pad:
+                stack.append(torch.zeros(pad, r.shape[1], dtype=r.dtype, device=r.device))
+                n += pad
+
+        for i, r in enumerate(rows):
+            put(r, 8 if i == len(rows) - 1 else 1)
+        spec, gu, _ = t["ff"]
+        out["ff"] = (n, spec)
+        put(gu, 8 if gate else 16)
+        if gate:
+            out["g_off"] = n
+            put(t["g"], 16)
+        rows = stack
     out[key] = cast(rows[0] if len(rows) == 1 else torch.cat(rows, 0))
+
+
+def _out_proj(t: dict, out: dict, cast) -> None:
+    """out["w_o"] = the mixer's output projection; with a feed-forward beside it (t["ff"]) the down projection's columns
+    follow: one product over [mixer output | feed-forward activation] is the sum of the two sublayers."""
+    out["w_o"] = cast(torch.cat([t["o"], t["ff"][2]], 1) if "ff" in t else t["o"])
+
+
+def ff_rides_along(mixer, ff) -> bool:
+    """Can a layer's feed-forward, on a parallel stream, share the mixer's first and last products?  A gated one beside
+    an attention mixer, with both parts of the last product on 16-byte columns."""
+    return ff is not None and ff.kind == "glu" and mixer.kind in ("latent_attention", "window_attention") and \
+        ff.ff % 8 == 0 and mixer.heads * mixer.vdim % 8 == 0
 
 
 def pack_mlstm(spec: MLSTMSpec, t: dict, device, act_dtype) -> dict:
@@ -519,17 +601,26 @@ def pack_mlstm(spec: MLSTMSpec, t: dict, device, act_dtype) -> dict:
 
 
 def pack_latent(spec: LatentAttentionSpec, t: dict, device, act_dtype) -> dict:
-    """t: q, dkv, dkv.norm, uk, uv, g, o.  q | dkv (| g with a gate per output column) are one projection; per-head
+    """t: q (or dq, dq.norm, uq), dkv, dkv.norm (not with kv_from), uk, uv, g, sink, o.  q | dkv (| g with a gate per
+    output column) are one projection, with a query latent dq | dkv are; per-head
     gate rows are a few-row float32-output projection.  The per-head up-projections are kept as [H, rank, D] and
     [H, Dv, rank]: keys are never materialised (the query is carried into the latent space instead) and the value
     up-projection is applied to the attention's latent-space output."""
     a = lambda x: x.to(device=device, dtype=act_dtype).contiguous()  # noqa: E731
     f = lambda x: x.to(device=device, dtype=torch.float32).contiguous()  # noqa: E731
-    out = dict(dkv_norm=f(t["dkv.norm"]), w_o=a(t["o"]),
-               w_uk=a(t["uk"].view(spec.heads, spec.dim, spec.kv_rank).transpose(1, 2)),
+    out = dict(w_uk=a(t["uk"].view(spec.heads, spec.dim, spec.kv_rank).transpose(1, 2)),
                w_uv=a(t["uv"].view(spec.heads, spec.vdim, spec.kv_rank)))
-    _in_proj([t["q"], t["dkv"]] + ([t["g"]] if spec.gate_wide else []), t, out, "w_in", a)
-    if not spec.gate_wide:
+    rows = [t["dq"] if spec.q_rank else t["q"]]
+    if spec.q_rank:
+        out.update(dq_norm=f(t["dq.norm"]), w_uq=a(t["uq"]))
+    if spec.kv_from is None:
+        out["dkv_norm"] = f(t["dkv.norm"])
+        rows.append(t["dkv"])
+    _in_proj(rows + ([t["g"]] if spec.gate and spec.gate_wide else []), t, out, "w_in", a)
+    _out_proj(t, out, a)
+    if spec.sink:
+        out["sink"] = f(t["sink"])
+    if spec.gate and not spec.gate_wide:
         out["w_g"] = a(t["g"])
     return out
 
@@ -561,19 +652,25 @@ def pack_moe(spec: MoEFFSpec, t: dict, device, act_dtype) -> dict:
 
 
 def pack_window_attention(spec: WindowAttentionSpec, t: dict, device, act_dtype) -> dict:
-    """t: q, k, v, q.norm, k.norm, sink, g, o and, in value-mixing layers, vmix.  q | k | v become one projection
+    """t: q, k, v, q.norm, k.norm, sink, g, o, the convolution's taps q.conv, k.conv, v.conv and, in value-mixing
+    layers, vmix.  q | k | v become one projection
     (q | k when the values are the keys; q | k | v | g with a gate per output column); per-head gate rows are a
-    few-row float32-output projection."""
+    few-row float32-output projection (with a feed-forward beside the mixer they end the one projection)."""
     a = lambda x: x.to(device=device, dtype=act_dtype).contiguous()  # noqa: E731
     f = lambda x: x.to(device=device, dtype=torch.float32).contiguous()  # noqa: E731
     rows = [t["q"], t["k"]] + ([] if spec.v_from_k else [t["v"]]) + ([t["g"]] if spec.gate and spec.gate_wide else [])
-    out = dict(w_o=a(t["o"]))
-    _in_proj(rows, t, out, "w_qkv", a)
-    if spec.qk_norm:
-        out.update(q_norm=f(t["q.norm"]), k_norm=f(t["k.norm"]))
+    out = {}
+    few = spec.gate and not spec.gate_wide
+    _in_proj(rows, t, out, "w_qkv", a, few)
+    _out_proj(t, out, a)
+    if spec.conv:
+        out["taps"] = f(torch.cat([t["q.conv"], t["k.conv"]] + ([] if spec.v_from_k else [t["v.conv"]]), 0))
+    if spec.qk_norm and not spec.unit_keys:
+        one = torch.ones(spec.dim)
+        out.update(q_norm=f(t["q.norm"] if spec.qk_norm_weight else one), k_norm=f(t["k.norm"] if spec.qk_norm_weight else one))
     if spec.sink:
         out["sink"] = f(t["sink"] if spec.sink_fixed is None else torch.full((spec.heads,), float(spec.sink_fixed)))
-    if spec.gate and not spec.gate_wide:
+    if few and "g_off" not in out:
         out["w_g"] = a(t["g"])
     if spec.bias:
         rest = out["w_qkv"].shape[0] - spec.heads * spec.dim - spec.kv_heads * (spec.dim + spec.vdim)  # gate rows: none
@@ -715,6 +812,12 @@ def rope_cos_sin(base: float, dims: int, max_pos: int, device, scaling: Optional
     return (torch.cat([fr.cos(), fr.sin()], 1) * mag).float().to(device)
 
 
+def query_temperature(coef: float, every: float, max_pos: int, device) -> torch.Tensor:
+    """[max_pos] float32: 1 + coef ln(floor((p + 1) / every) + 1), in float64 before the rounding."""
+    p = torch.arange(1, max_pos + 1, dtype=torch.float64)
+    return (1.0 + coef * torch.log(torch.floor(p / every) + 1.0)).float().to(device)
+
+
 # -----------------------------------------------------------------------------------------------------------------
 # mixers and feed-forwards (one function per kind: h [T, d] in the activation dtype -> [T, d])
 # -----------------------------------------------------------------------------------------------------------------
@@ -760,46 +863,78 @@ def _with_gate(y, proj, w: dict):
     return GatedOut(y, proj, w["rg_off"]) if "rg_off" in w else y
 
 
+def _wide_out(w: dict, proj, n: int):
+    """Rows for a mixer's output of n columns.  With a feed-forward beside the mixer they are the first n columns of
+    wider ones, whose other columns receive the feed-forward's activation here; the caller's last product takes the
+    wide rows.  Returns (wide rows or None, the mixer's columns or None: the op makes its own)."""
+    if "ff" not in w:
+        return None, None
+    off, ff = w["ff"]
+    wide = torch.empty(proj.shape[0], n + ff.ff, device=proj.device, dtype=proj.dtype)
+    hops.glu_cols(proj, off, ff.ff, ff.limit, ff.slope, ff.shift, wide[:, n:])
+    return wide, wide[:, :n]
+
+
 def mix_latent_attention(model, li: int, spec: LatentAttentionSpec, w: dict, h, meta: StepMeta, cache: HybridCache):
     T = h.shape[0]
     H, D, R, rank = spec.heads, spec.dim, spec.rot_dim, spec.kv_rank
-    nq, nkv = H * (D + R), rank + R
-    proj = hops.matmul(h, w["w_in"])    # q | dkv (| one gate per output column)
-    q = proj[:, :nq].view(T, H, D + R)
-    gate = None if spec.gate_wide else hops.rowdot(h, w["w_g"])
+    eps = model.cfg.norm_eps
+    nq, nkv = spec.q_rank or H * (D + R), rank + R
+    proj = hops.matmul(h, w["w_in"])    # q or its latent | dkv (| one gate per output column)
+    q = proj[:, :nq]
+    if spec.q_rank:
+        q = hops.matmul(hops.norm_cols(proj, 0, nq, w["dq_norm"], eps), w["w_uq"])
+    q = q.view(T, H, D + R)
+    gate = hops.rowdot(h, w["w_g"]) if spec.gate and not spec.gate_wide else None
+    own = spec.kv_from is None
     # the query goes into the latent space (q_u W_uk per head), so a key is the cached row itself; the output
     # comes back through W_uv per head
     qa = torch.empty(T, H, rank + R, device=h.device, dtype=h.dtype)
-    hops.latent_prep(q, proj[:, nq:nq + nkv], meta.pos, meta.tok_seq, meta.block_table, w["dkv_norm"], model.cfg.norm_eps,
-                     model.rope.get(li), spec.rope_dims, rank, cache.lat[li], qa, spec.rope_interleaved)
+    hops.latent_prep(q, proj[:, nq:nq + nkv] if own else None, meta.pos, meta.tok_seq, meta.block_table, w.get("dkv_norm"),
+                     eps, model.rope.get(li), spec.rope_dims, rank, cache.lat[li], qa, spec.rope_interleaved)
     hops.head_matmul(q[:, :, :D], w["w_uk"], qa[:, :, :rank])
     oa = hops.latent_attention(qa, cache.lat[li], meta.block_table, meta.q_start, meta.pos, gate, spec.scale, rank,
-                               model.act_dtype, meta.max_q, spec.window, spec.two_term)
-    ov = hops.head_matmul(oa, w["w_uv"], None, proj if spec.gate_wide else None, nq + nkv)
-    return _with_gate(hops.matmul(ov.view(T, H * spec.vdim), w["w_o"]), proj, w)
+                               model.act_dtype, meta.max_q, spec.window, spec.two_term, w.get("sink"))
+    wide, ov = _wide_out(w, proj, H * spec.vdim)
+    ov = hops.head_matmul(oa, w["w_uv"], None if ov is None else ov.view(T, H, spec.vdim),
+                          proj if spec.gate and spec.gate_wide else None, nq + nkv if own else nq)
+    return _with_gate(hops.matmul(ov.view(T, H * spec.vdim) if wide is None else wide, w["w_o"]), proj, w)
 
 
 def mix_window_attention(model, li, spec: WindowAttentionSpec, w: dict, h, meta: StepMeta, cache: HybridCache):
     H, G, D, Dv = spec.heads, spec.kv_heads, spec.dim, spec.vdim
-    qkv = hops.matmul(h, w["w_qkv"], w.get("b_qkv"))
-    gate = hops.rowdot(h, w["w_g"]) if spec.gate and not spec.gate_wide else None
-    mixes = spec.v_mix and not spec.v_mix_first
-    v_tab = model.rope_v.get(li)
-    v = hops.window_prep(qkv, H, G, D, Dv, meta.shared["v_first"] if mixes else None, w.get("vmix"), meta.pos,
-                         meta.tok_seq, meta.block_table, w.get("q_norm"), w.get("k_norm"), model.cfg.norm_eps,
-                         model.rope.get(li), spec.rope_dims, cache.kc[li], cache.vc[li], spec.v_mix_first,
-                         H * D if spec.v_from_k else -1, v_tab)
-    if spec.v_mix_first:
-        meta.shared["v_first"] = v
+    proj = qkv = hops.matmul(h, w["w_qkv"], w.get("b_qkv"))
+    gate = hops.rowdot(h, w["w_g"]) if "w_g" in w else None
+    temp = model.q_temp.get(li)
+    if spec.conv and spec.unit_keys:
+        # convolution, norms, temperature, cache write and the gate's float32 copy in one pass over the projection
+        qkv, gate_cols = hops.conv_prep(proj, w["taps"], meta.tok_seq, meta.q_start, meta.pos0, meta.slots, cache.hist[li],
+                                        meta.pos, meta.block_table, H, G, D, model.cfg.norm_eps, temp, cache.ks[li],
+                                        cache.vc[li], w.get("g_off", -1), meta.max_q)
+        gate = gate if gate_cols is None else gate_cols
+    else:
+        if spec.conv:
+            qkv = hops.short_conv(proj, w["taps"], meta.tok_seq, meta.q_start, meta.pos0, meta.slots, cache.hist[li], False)
+        if "g_off" in w:
+            gate = proj[:, w["g_off"]:w["g_off"] + H].float()
+        mixes = spec.v_mix and not spec.v_mix_first
+        v = hops.window_prep(qkv, H, G, D, Dv, meta.shared["v_first"] if mixes else None, w.get("vmix"), meta.pos,
+                             meta.tok_seq, meta.block_table, w.get("q_norm"), w.get("k_norm"), model.cfg.norm_eps,
+                             model.rope.get(li), spec.rope_dims, cache.kc.get(li), cache.vc[li], spec.v_mix_first,
+                             H * D if spec.v_from_k else -1, model.rope_v.get(li), temp, cache.ks.get(li))
+        if spec.v_mix_first:
+            meta.shared["v_first"] = v
     pooled = spec.pool > 0 and spec.window > 0
     if pooled:   # the blocks this step's tokens complete get their means before any query of the step looks
         hops.pool_blocks(cache.kc[li], cache.vc[li], cache.kp[li], cache.vp[li], meta.block_table, meta.q_start,
                          meta.pos0, spec.pool, meta.max_q)
-    o = hops.window_attention(qkv, cache.kc[li], cache.vc[li], meta.block_table, meta.q_start, meta.pos, w.get("sink"),
+    wide, out = _wide_out(w, proj, H * Dv)
+    o = hops.window_attention(qkv, cache.kc.get(li), cache.vc[li], meta.block_table, meta.q_start, meta.pos, w.get("sink"),
                               gate, spec.scale, spec.window, spec.keep_first, H, model.act_dtype, meta.max_q,
-                              spec.chunk, spec.pool if pooled else 0, cache.kp.get(li), cache.vp.get(li), v_tab,
-                              (H + G) * D + G * Dv if spec.gate and spec.gate_wide else -1)
-    return _with_gate(hops.matmul(o, w["w_o"], w.get("b_o")), qkv, w)
+                              spec.chunk, spec.pool if pooled else 0, cache.kp.get(li), cache.vp.get(li),
+                              model.rope_v.get(li), (H + G) * D + G * Dv if spec.gate and spec.gate_wide else -1,
+                              cache.ks.get(li), out)
+    return _with_gate(hops.matmul(o if wide is None else wide, w["w_o"], w.get("b_o")), proj, w)
 
 
 def mix_retention(model, li, spec: RetentionSpec, w: dict, h, meta: StepMeta, cache: HybridCache):
@@ -931,12 +1066,13 @@ RECURRENT_MIXERS = ("mlstm", "delta_rule", "gla", "mamba2", "rglru", "retention"
 
 
 def _is_recurrent(mx) -> bool:
-    """Does a sequence hold something beyond the tokens of its own pages?  A recurrent state; or pooled blocks, whose
+    """Does a sequence hold something beyond the tokens of its own pages?  A recurrent state, the last inputs of a short
+    convolution; or pooled blocks, whose
     pair sits in the page e // EP while its tokens may lie on later pages (blocks off the page grid), so that a page
     shared between sequences as a common prefix could be written with one sequence's continuation."""
     if mx.kind == "parallel":
         return _is_recurrent(mx.left) or _is_recurrent(mx.right)
-    return mx.kind in RECURRENT_MIXERS or (mx.kind == "window_attention" and mx.pool > 0 and mx.window > 0)
+    return mx.kind in RECURRENT_MIXERS or (mx.kind == "window_attention" and (mx.conv > 1 or (mx.pool > 0 and mx.window > 0)))
 
 
 # -----------------------------------------------------------------------------------------------------------------
@@ -964,7 +1100,7 @@ class HybridDecoder:
         self.decode_overlap_rows = 0
         P = max_position or cfg.max_position
         # rotation tables by run (the halves of a parallel mixer: (run, 0) and (run, 1)); equal tables are one tensor
-        self.rope, self.rope_v, made = {}, {}, {}
+        self.rope, self.rope_v, self.q_temp, made = {}, {}, {}, {}
 
         def table(base, dims, scaling):
             key = (float(base), int(dims), tuple(scaling) if scaling else None)
@@ -981,15 +1117,33 @@ class HybridDecoder:
                     self.rope[key] = table(mx.rope_base, mx.rope_dims, getattr(mx, "rope_scaling", None))
                 if getattr(mx, "v_rot", False):
                     self.rope_v[key] = table(mx.rope_base, mx.vdim, None)
+                if getattr(mx, "q_temp", None):
+                    tk = tuple(float(v) for v in mx.q_temp)
+                    if tk not in made:
+                        made[tk] = query_temperature(*tk, P, self.device)
+                    self.q_temp[key] = made[tk]
 
         for ri, l in enumerate(cfg.layers[i] for i in cfg.runs):
             tables(ri, l.mixer)
         self.recurrent = any(_is_recurrent(l.mixer) for l in cfg.layers)
-        if cfg.residual not in ("out_norm", "post_norm", "pre_norm", "sandwich"):
+        if cfg.residual not in ("out_norm", "post_norm", "pre_norm", "sandwich", "parallel"):
             raise ValueError(f"unknown residual rule {cfg.residual!r}")
+        if (cfg.residual == "parallel") != (cfg.norm == "layer"):
+            raise ValueError("the parallel stream has layer norms with weight and bias, the others do not")
+        for i, l in enumerate(cfg.layers):
+            src = getattr(l.mixer, "kv_from", None)
+            if src is None:
+                continue
+            m, o = l.mixer, cfg.layers[src].mixer if 0 <= src < i else None
+            if cfg.loop or cfg.share is not None or getattr(o, "kind", "") != "latent_attention" or o.kv_from is not None:
+                raise ValueError(f"layer {i}: kv_from names an earlier latent-attention layer with latents of its own, in "
+                                 "a model whose layers run once")
+            same = lambda a: (a.kv_rank, a.rot_dim, a.rope_base, a.rope_dims, a.rope_scaling, a.rope_interleaved)  # noqa: E731
+            if same(m) != same(o):
+                raise ValueError(f"layer {i}: kv_rank, rot_dim and rotation must be those of layer {src}")
         if cfg.token_side and cfg.residual != "pre_norm":
             raise ValueError("the per-layer token input is part of the pre-norm stream's join")
-        if cfg.norm not in ("rms", "tanh"):
+        if cfg.norm not in ("rms", "tanh", "layer"):
             raise ValueError(f"unknown norm {cfg.norm!r}")
         self.gated_stream = cfg.norm == "tanh" or cfg.residual_gate or cfg.depth_average or cfg.residual_mult != 1.0
         if self.gated_stream and (cfg.residual != "pre_norm" or cfg.token_side):
@@ -1056,13 +1210,15 @@ class HybridDecoder:
         followed by decode rows)."""
         cfg, w, at = self.cfg, self.w, self.act_dtype
         meta = self._meta(sb)
-        x, h = hops.embed_rows(meta.ids, w.embed, at, cfg.embed_scale, cfg.residual not in ("pre_norm", "sandwich"))
+        x, h = hops.embed_rows(meta.ids, w.embed, at, cfg.embed_scale, cfg.residual not in ("pre_norm", "sandwich", "parallel"))
         if self.gated_stream:
             self._forward_gated(x, meta, cache)
         elif cfg.residual == "pre_norm":
             self._forward_pre_norm(x, meta, cache)
         elif cfg.residual == "sandwich":
             self._forward_sandwich(x, meta, cache)
+        elif cfg.residual == "parallel":
+            self._forward_parallel(x, meta, cache)
         else:
             for ri, li in enumerate(cfg.runs):   # the cache is keyed by run, the weights by layer
                 spec, lw = cfg.layers[li], w.layers[li]
@@ -1078,6 +1234,8 @@ class HybridDecoder:
             xn = hops.layer_norm(xs, w.final_norm, cfg.norm_eps, at)
         elif cfg.norm == "tanh":
             xn = hops.dyn_tanh(xs, w.final_norm, at)
+        elif cfg.norm == "layer":
+            xn = hops.layer_norm_join(None, xs, w.final_norm, cfg.norm_eps, at)
         else:
             xn = hops.rms_norm(xs, w.final_norm, cfg.norm_eps, at, cfg.norm_groups if cfg.residual == "sandwich" else 1)
         logits = hops.matmul(xn, w.head).float()
@@ -1174,6 +1332,26 @@ class HybridDecoder:
                 y = FEED_FORWARDS[spec.ff.kind][0](self, spec.ff, lw.ff, h)
                 y, y2 = y if isinstance(y, tuple) else (y, None)
                 h = hops.sandwich_join(y, x, lw.norm2b, nxt, ng, eps, at, y2, None, emit=not last)
+            if self.layer_tap is not None:
+                self.layer_tap(ri, x)
+
+    def _forward_parallel(self, x, meta: StepMeta, cache: HybridCache) -> None:
+        """x <- x + mixer(h) + ff(h), h = layer_norm(x): both sublayers of a layer read one norm.  A feed-forward that
+        rides along in the mixer's first and last products leaves one output to add, any other its own.  One join
+        kernel per layer adds to the float32 stream in place and emits the next layer's norm."""
+        cfg, w, at, eps = self.cfg, self.w, self.act_dtype, self.cfg.norm_eps
+        runs = cfg.runs
+        h = hops.layer_norm_join(None, x, w.layers[runs[0]].norm1, eps, at) if runs else None
+        for ri, li in enumerate(runs):
+            spec, lw = cfg.layers[li], w.layers[li]
+            last = ri + 1 == len(runs)    # the last run emits nothing: the final norm reads the wanted rows only
+            y = MIXERS[spec.mixer.kind][0](self, ri, spec.mixer, lw.mix, h, meta, cache)
+            y2 = None
+            if spec.ff is not None and "ff" not in lw.mix:
+                y2 = FEED_FORWARDS[spec.ff.kind][0](self, spec.ff, lw.ff, h)
+            if isinstance(y, PairOut) or isinstance(y2, tuple):
+                raise NotImplementedError("a sublayer with a separate part on the parallel stream")
+            h = hops.layer_norm_join(y, x, None if last else w.layers[runs[ri + 1]].norm1, eps, at, y2, emit=not last)
             if self.layer_tap is not None:
                 self.layer_tap(ri, x)
 

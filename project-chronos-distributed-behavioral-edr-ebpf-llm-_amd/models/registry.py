@@ -213,6 +213,29 @@ def _lalasun_presets():
     return list(lalasun.PRESETS)
 
 
+def _nubodra_build(name, device, tp, seed, is_path, max_position, weight_dtype, dtype):
+    from . import nubodra
+
+    if tp.world > 1:
+        raise NotImplementedError("Nubodra runs on full-weight ranks (data-parallel replicas)")
+    if weight_dtype != "bf16":
+        raise NotImplementedError("Nubodra weights are served in the activation dtype (no fp8 projections)")
+    return nubodra.build(name, device, seed, DTYPES[dtype], max_position)
+
+
+def _nubodra_is_checkpoint(path: str) -> bool:
+    from . import nubodra
+
+    return nubodra.is_checkpoint(path)
+
+
+def _nubodra_presets():
+    from . import nubodra
+
+    return list(nubodra.PRESETS)
+
+
+register(Family("nubodra", _nubodra_presets, _nubodra_is_checkpoint, _nubodra_build, ("bf16", "fp32")))
 register(Family("lalasun", _lalasun_presets, _lalasun_is_checkpoint, _lalasun_build, ("bf16", "fp32")))
 register(Family("vogerax", _vogerax_presets, _vogerax_is_checkpoint, _vogerax_build, ("bf16", "fp32")))
 register(Family("tugovik", _tugovik_presets, _tugovik_is_checkpoint, _tugovik_build, ("bf16", "fp32")))

@@ -112,7 +112,8 @@ def mlstm_out(o, proj, g_off: int, norm_w, eps: float, act_dtype):
 def latent_prep(q, dkv, pos, tok_seq, block_table, w_norm, eps: float, cos_sin, dims: int, rank: int, cache, qa=None,
                 interleaved: bool = False) -> None:
     """``qa``: where the rotated query columns go (its last R columns per head; default: in place); ``interleaved``:
-    neighbouring columns form the rotated pairs.  q and dkv may be column ranges of one wider projection."""
+    neighbouring columns form the rotated pairs.  q and dkv may be column ranges of one wider projection; dkv None: the
+    cache is another layer's and only the queries are rotated."""
     if _gpu(q):
         _k().hy_latent_prep(q, dkv, pos, tok_seq, block_table, w_norm, eps, cos_sin if dims else None, dims, rank, cache,
                             qa, interleaved)
@@ -132,13 +133,13 @@ def head_matmul(a, w, out=None, gate_src=None, g_off: int = -1):
 
 
 def latent_attention(qa, cache, block_table, q_start, pos, gate, scale: float, rank: int, act_dtype, max_q: int,
-                     window: int = 0, two_term: bool = False):
+                     window: int = 0, two_term: bool = False, sink=None):
     """``max_q``: the most tokens any sequence brings in this step (sizes the launch grid).  ``window`` > 0: a query
     sees only the last ``window`` positions.  ``two_term``: the matrix-core kernel feeds every softmax weight as a sum
-    of two bfloat16 terms (float32 weights to about 2^-17)."""
+    of two bfloat16 terms (float32 weights to about 2^-17).  ``sink`` f32 [H]: joins the softmax denominator."""
     if _gpu(qa):
-        return _k().hy_latent_attention(qa, cache, block_table, q_start, pos, gate, scale, rank, max_q, window, two_term)
-    return ref.latent_attention(qa, cache, block_table, q_start, pos, gate, scale, rank, act_dtype, window)
+        return _k().hy_latent_attention(qa, cache, block_table, q_start, pos, gate, scale, rank, max_q, window, two_term, sink)
+    return ref.latent_attention(qa, cache, block_table, q_start, pos, gate, scale, rank, act_dtype, window, sink)
 
 
 def moe_route(h, w_router, correction, top: int):
@@ -181,15 +182,16 @@ def glu(gu, limit: float, slope: float, shift: float, act_dtype):
 
 
 def window_prep(qkv, H: int, G: int, D: int, Dv: int, v_first, lam, pos, tok_seq, block_table, q_norm, k_norm,
-                eps: float, cos_sin, dims: int, kc, vc, emit_v: bool, v_off: int = -1, v_cos_sin=None):
+                eps: float, cos_sin, dims: int, kc, vc, emit_v: bool, v_off: int = -1, v_cos_sin=None, q_temp=None, ks=None):
     """``v_off`` >= 0: the column of qkv where the values start (default: after the keys); ``v_cos_sin``: a rotation
-    table over all Dv columns that the values pass before they are cached."""
+    table over all Dv columns that the values pass before they are cached; ``q_temp`` f32 [P]: a factor on the queries by
+    position; ``ks`` (kc None): keys are values over their root mean square, only the factor is cached."""
     if _gpu(qkv):
         v = _k().hy_window_prep(qkv, H, G, D, Dv, v_first, lam, pos, tok_seq, block_table, q_norm, k_norm, eps, cos_sin,
-                                dims, kc, vc, emit_v, v_off, v_cos_sin)
+                                dims, kc, vc, emit_v, v_off, v_cos_sin, q_temp, ks)
         return v if emit_v else None
     return ref.window_prep(qkv, H, G, D, Dv, v_first, lam, pos, tok_seq, block_table, q_norm, k_norm, eps, cos_sin,
-                           dims, kc, vc, emit_v, v_off, v_cos_sin)
+                           dims, kc, vc, emit_v, v_off, v_cos_sin, q_temp, ks)
 
 
 def pool_blocks(kc, vc, kp, vp, block_table, q_start, pos0, pool: int, max_q: int) -> None:
@@ -203,20 +205,25 @@ def pool_blocks(kc, vc, kp, vp, block_table, q_start, pos0, pool: int, max_q: in
 
 def window_attention(qkv, kc, vc, block_table, q_start, pos, sink, gate, scale: float, window: int, keep_first: int,
                      H: int, act_dtype, max_q: int, chunk: int = 0, pool: int = 0, kp=None, vp=None, v_cos_sin=None,
-                     g_off: int = -1):
+                     g_off: int = -1, ks=None, out=None):
     """``max_q``: the most tokens any sequence brings in this step (sizes the launch grid).  ``chunk`` > 0: keys
     outside the query's own chunk of that many positions are hidden.  ``pool`` > 0: the pooled pairs of the blocks
     that lie wholly before a query's window join its softmax.  ``v_cos_sin`` [P, Dv]: every head's output is turned
     back by the query's position (the values were cached rotated); ``g_off`` >= 0: the output is multiplied element by
-    element with sigmoid of qkv[:, g_off : g_off + H Dv].  The matrix-core kernel does both in its epilogue."""
+    element with sigmoid of qkv[:, g_off : g_off + H Dv].  The matrix-core kernel does both in its epilogue.
+    ``ks`` f32 [NB, BS, G] (kc None): key j is value j times its factor, one cached row serves both.  ``out``: where the
+    output goes, [T, H Dv] columns of wider rows (not with v_cos_sin or g_off)."""
     if _gpu(qkv):
         return _k().hy_window_attention(qkv, kc, vc, block_table, q_start, pos, sink, gate, scale, window, keep_first,
                                         chunk, H, max_q, pool, kp if pool else None, vp if pool else None, v_cos_sin,
-                                        g_off)
+                                        g_off, ks, out)
     o = ref.window_attention(qkv, kc, vc, block_table, q_start, pos, sink, gate, scale, window, keep_first, H,
-                             act_dtype, chunk, pool, kp, vp)
+                             act_dtype, chunk, pool, kp, vp, ks)
     if v_cos_sin is not None or g_off >= 0:
         o = ref.unrotate_gate(o, pos, v_cos_sin, qkv if g_off >= 0 else None, g_off, H, vc.shape[3], act_dtype)
+    if out is not None:
+        out.copy_(o)
+        return out
     return o
 
 
@@ -395,3 +402,43 @@ def poly_norm(z, F: int, abce, eps: float, act_dtype):
     if _gpu(z):
         return _k().hy_poly_norm(z, F, abce, eps)
     return ref.poly_norm(z, F, abce, eps, act_dtype)
+
+
+# ---- parallel stream: one layer norm per layer, both sublayers in one pair of products -------------------------------
+
+
+def layer_norm_join(y, x, wb, eps: float, act_dtype, y2=None, emit: bool = True):
+    """x (float32 residual, in place) <- x + y (+ y2), y None: x stays.  Returns layer_norm(x) * w + b (wb = w | b), or
+    None when ``emit`` is off."""
+    if _gpu(x):
+        h = _k().hy_layer_norm_join(y, y2, x, wb if emit else None, eps, _f32(act_dtype))
+        return h if emit else None
+    return ref.layer_norm_join(y, x, wb, eps, act_dtype, y2, emit)
+
+
+def glu_cols(src, off: int, F: int, limit: float, slope: float, shift: float, out) -> None:
+    """The gated unit on columns off .. off + 2 F of src, into ``out`` [T, F] (a column range of wider rows)."""
+    if _gpu(src):
+        _k().hy_glu_cols(src, off, F, limit, slope, shift, out)
+    else:
+        ref.glu_cols(src, off, F, limit, slope, shift, out)
+
+
+def norm_cols(src, off: int, n: int, w, eps: float):
+    """RMS norm of n columns of src from ``off`` on, times w; [T, n] in src's dtype."""
+    if _gpu(src):
+        return _k().hy_norm_cols(src, off, n, w, eps)
+    return ref.norm_cols(src, off, n, w, eps)
+
+
+def conv_prep(proj, taps, tok_seq, q_start, pos0, slots, hist, pos, block_table, H: int, G: int, D: int, eps: float,
+              q_temp, ks, vc, g_off: int, max_q: int):
+    """Convolution, norms, temperature and cache write of an attention layer whose keys are values over their root mean
+    square.  ``max_q``: the most tokens any sequence brings in this step (with 1 the history is rewritten in the same
+    pass).  Returns (queries [T, H D], float32 gate columns [T, H] or None)."""
+    if _gpu(proj):
+        q, gate = _k().hy_conv_prep(proj, taps, tok_seq, q_start, pos0, slots, hist, pos, block_table, H, G, D, eps, q_temp,
+                                    ks, vc, g_off, max_q)
+        return q, (gate if g_off >= 0 else None)
+    return ref.conv_prep(proj, taps, q_start, pos0, slots, hist, pos, tok_seq, block_table, H, G, D, eps, q_temp, ks, vc,
+                         g_off)

@@ -121,17 +121,18 @@ def latent_prep(q, dkv, pos, tok_seq, block_table, w_norm, eps, cos_sin, dims, r
     (times w_norm) into the latent, the last R rotated (on their leading ``dims`` columns; none with dims 0); both are
     written to cache [NB, BS, rank + R] at the token's page and slot.  q [T, H, D + R] (a view whose rows may be part of
     a wider projection, like dkv): the last R columns of every head are rotated, into the last R columns of qa
-    [T, H, rank + R] when that is given (q is then left as it is), else in place."""
-    T = q.shape[0]
-    R = dkv.shape[1] - rank
+    [T, H, rank + R] when that is given (q is then left as it is), else in place.  dkv None: the cache is another
+    layer's and stays as it is."""
+    R = cache.shape[2] - rank
     D = q.shape[2] - R
-    c = dkv[:, :rank].float()
-    c = c * torch.rsqrt(c.pow(2).mean(-1, keepdim=True) + eps) * w_norm.float()
     rot = lambda x: rotate_half_rows(x, cos_sin, pos, dims, interleaved) if dims else x.float()  # noqa: E731
-    row = torch.cat([c, rot(dkv[:, rank:])], 1).to(cache.dtype)
-    bs = cache.shape[1]
-    blk = block_table[tok_seq.long(), (pos // bs).long()].long()
-    cache[blk, (pos % bs).long()] = row
+    if dkv is not None:
+        c = dkv[:, :rank].float()
+        c = c * torch.rsqrt(c.pow(2).mean(-1, keepdim=True) + eps) * w_norm.float()
+        row = torch.cat([c, rot(dkv[:, rank:])], 1).to(cache.dtype)
+        bs = cache.shape[1]
+        blk = block_table[tok_seq.long(), (pos // bs).long()].long()
+        cache[blk, (pos % bs).long()] = row
     (q[:, :, D:] if qa is None else qa[:, :, rank:]).copy_(rot(q[:, :, D:]).to(q.dtype))
 
 
@@ -150,11 +151,12 @@ def head_matmul(a, w, out=None, gate_src=None, g_off=-1):
     return out
 
 
-def latent_attention(qa, cache, block_table, q_start, pos, gate, scale, rank, act_dtype, window=0):
+def latent_attention(qa, cache, block_table, q_start, pos, gate, scale, rank, act_dtype, window=0, sink=None):
     """Causal softmax attention of H query heads over ONE shared key row per token: key = the cached row (rank + R
     columns), value = its first rank columns.  qa [T, H, rank + R]; token t of sequence b sits at pos[t] and sees the
     cached rows 0..pos[t] of its sequence (``window`` > 0: only the last ``window`` of them); gate f32 [T, H] or None:
-    the output of head h is multiplied by sigmoid(gate).  Returns [T, H, rank]."""
+    the output of head h is multiplied by sigmoid(gate); sink f32 [H] or None: exp(sink_h) joins the softmax denominator
+    (no key, no value).  Returns [T, H, rank]."""
     T, H, DK = qa.shape
     out = torch.zeros(T, H, rank, dtype=torch.float32, device=qa.device)
     bs = cache.shape[1]
@@ -173,7 +175,9 @@ def latent_attention(qa, cache, block_table, q_start, pos, gate, scale, rank, ac
         if window:
             mask = mask | (p[:, None] - j >= window)
         sc = sc.masked_fill(mask[:, None, :], float("-inf"))
-        a = torch.softmax(sc, -1)
+        if sink is not None:
+            sc = torch.cat([sc, sink.float()[None, :, None].expand(t1 - t0, H, 1)], -1)
+        a = torch.softmax(sc, -1)[:, :, :ctx]
         out[t0:t1] = torch.einsum("thj,jr->thr", a, keys[:, :rank])
     if gate is not None:
         out = out * torch.sigmoid(gate.float())[:, :, None]
@@ -242,14 +246,15 @@ def glu(gu, limit, slope, shift, act_dtype):
 
 
 def window_prep(qkv, H, G, D, Dv, v_first, lam, pos, tok_seq, block_table, q_norm, k_norm, eps, cos_sin, dims, kc, vc,
-                emit_v, v_off=-1, v_cos_sin=None):
+                emit_v, v_off=-1, v_cos_sin=None, q_temp=None, ks=None):
     """qkv [T, H D + G D + G Dv]: per-head RMS norm (weights q_norm / k_norm [D], float32 math; both None: no
     norm) and rotation of the query and key heads, queries in place; values mixed with ``v_first`` [T, G Dv] as (1 - lam) v + lam v_first when
     given; keys and (mixed) values written to the paged caches kc [NB, BS, G, D], vc [NB, BS, G, Dv].  Returns the
     values as read from the projection [T, G Dv] when ``emit_v`` (the source of later layers' mixing), else None.
     ``v_off`` >= 0: the values start at that column of qkv instead of after the keys (at H D they are the keys as
     projected).  ``v_cos_sin`` [P, Dv]: the values are rotated by their position over all Dv columns before the
-    write."""
+    write.  ``q_temp`` f32 [P]: queries are multiplied by the entry at their position.  ``ks`` f32 [NB, BS, G] (with
+    kc None): keys are the values divided by their root mean square, and only that factor is written."""
     T = qkv.shape[0]
     q = qkv[:, :H * D].view(T, H, D)
     k = qkv[:, H * D:(H + G) * D].view(T, G, D)
@@ -263,18 +268,24 @@ def window_prep(qkv, H, G, D, Dv, v_first, lam, pos, tok_seq, block_table, q_nor
             xf = xf * torch.rsqrt(xf.pow(2).mean(-1, keepdim=True) + eps) * w.float()
         return rotate_half_rows(xf, cos_sin, pos, dims) if dims else xf
 
+    if ks is not None:
+        q_norm = torch.ones(D, device=qkv.device)
     qn = norm_rot(q, q_norm)
-    kn = norm_rot(k, k_norm)
+    if q_temp is not None:
+        qn = qn * q_temp[pos.long()][:, None, None]
     vf = v.float()
     if v_first is not None:
         l = lam.float().reshape(())
         vf = (1.0 - l) * vf + l * v_first.view(T, G, Dv).float()
     if v_cos_sin is not None:
         vf = rotate_half_rows(vf, v_cos_sin, pos, Dv)
-    bs = kc.shape[1]
+    bs = vc.shape[1]
     blk = block_table[tok_seq.long(), (pos // bs).long()].long()
-    kc[blk, (pos % bs).long()] = kn.to(kc.dtype)
     vc[blk, (pos % bs).long()] = vf.to(vc.dtype)
+    if ks is not None:
+        ks[blk, (pos % bs).long()] = torch.rsqrt(vf.to(vc.dtype).float().pow(2).mean(-1) + eps)
+    else:
+        kc[blk, (pos % bs).long()] = norm_rot(k, k_norm).to(kc.dtype)
     q.copy_(qn.to(q.dtype))
     return out_v
 
@@ -298,7 +309,7 @@ def pool_blocks(kc, vc, kp, vp, block_table, q_start, pos0, pool):
 
 
 def window_attention(qkv, kc, vc, block_table, q_start, pos, sink, gate, scale, window, keep_first, H, act_dtype,
-                     chunk=0, pool=0, kp=None, vp=None):
+                     chunk=0, pool=0, kp=None, vp=None, ks=None):
     """Causal softmax attention over a paged cache through a sliding window that also keeps a sequence's first
     tokens: the query at position i sees key j <= i when i - j < window or j < keep_first (window 0: every j <= i).
     ``chunk`` > 0 further hides every key outside the query's own chunk of that many positions (the chunk grid
@@ -307,12 +318,14 @@ def window_attention(qkv, kc, vc, block_table, q_start, pos, sink, gate, scale, 
     None: head h's output times sigmoid(gate).  Queries are the first H D columns of qkv; query head h reads
     key/value head h // (H / G).  ``pool`` > 0 (with a window): the query at i also sees the pooled pair of every
     block e with e pool + pool - 1 <= i - window (kp / vp as :func:`pool_blocks` leaves them), in the same softmax.
+    ``ks`` f32 [NB, BS, G] (kc None): key j is value j times its factor.
     Returns [T, H Dv]."""
     T = qkv.shape[0]
-    G, D, Dv = kc.shape[2], kc.shape[3], vc.shape[3]
+    G, Dv = vc.shape[2], vc.shape[3]
+    D = Dv if kc is None else kc.shape[3]
     q = qkv[:, :H * D].view(T, H, D).float()
     out = torch.zeros(T, H, Dv, dtype=torch.float32, device=qkv.device)
-    bs = kc.shape[1]
+    bs = vc.shape[1]
     qs = q_start.tolist()
     rep = H // G
     for b in range(len(qs) - 1):
@@ -323,8 +336,10 @@ def window_attention(qkv, kc, vc, block_table, q_start, pos, sink, gate, scale, 
         ctx = int(p.max()) + 1
         nblk = (ctx + bs - 1) // bs
         pages = block_table[b, :nblk].long()
-        keys = kc[pages].reshape(nblk * bs, G, D)[:ctx].float().repeat_interleave(rep, 1)
-        vals = vc[pages].reshape(nblk * bs, G, Dv)[:ctx].float().repeat_interleave(rep, 1)
+        vals = vc[pages].reshape(nblk * bs, G, Dv)[:ctx].float()
+        keys = kc[pages].reshape(nblk * bs, G, D)[:ctx].float() if ks is None else \
+            vals * ks[pages].reshape(nblk * bs, G, 1)[:ctx]
+        keys, vals = keys.repeat_interleave(rep, 1), vals.repeat_interleave(rep, 1)
         sc = torch.einsum("thd,jhd->thj", q[t0:t1], keys) * scale
         j = torch.arange(ctx, device=qkv.device)[None, :]
         hidden = j > p[:, None]
@@ -664,3 +679,40 @@ def poly_norm(z, F, abce, eps, act_dtype):
     n = lambda v: v * torch.rsqrt(v.pow(2).mean(-1, keepdim=True) + eps)  # noqa: E731
     a, b, c, e = (abce[i].float() for i in range(4))
     return (a * n(zf) + b * n(zf * zf) + c * n(zf * zf * zf) + e).to(act_dtype)
+
+
+# ---- parallel stream: one layer norm per layer, both sublayers in one pair of products -------------------------------
+
+
+def layer_norm_join(y, x, wb, eps, act_dtype, y2=None, emit=True):
+    """x (float32 residual, in place) <- x + y (+ y2); y None: x stays.  Returns layer_norm(x) * w + b in the activation
+    dtype (``wb`` f32 [2 d] = w | b; the variance is the mean of the squared deviations), or None when ``emit`` is off."""
+    if y is not None:
+        x.add_(y.float() if y2 is None else y.float() + y2.float())
+    if not emit:
+        return None
+    d = x.shape[-1]
+    c = x - x.mean(-1, keepdim=True)
+    return (c * torch.rsqrt(c.pow(2).mean(-1, keepdim=True) + eps) * wb[:d] + wb[d:]).to(act_dtype)
+
+
+def glu_cols(src, off, F, limit, slope, shift, out):
+    """The gated unit of :func:`glu` on columns of wider rows: gate columns off .. off + F of src, up columns the next F;
+    into ``out`` [T, F], a column range of wider rows too."""
+    out.copy_(glu(src[:, off:off + 2 * F], limit, slope, shift, out.dtype))
+
+
+def norm_cols(src, off, n, w, eps):
+    """rms_norm of columns off .. off + n of src [T, C], times w [n]; in src's dtype."""
+    return rms_norm(src[:, off:off + n], w, eps, src.dtype)
+
+
+def conv_prep(proj, taps, q_start, pos0, slots, hist, pos, tok_seq, block_table, H, G, D, eps, q_temp, ks, vc, g_off):
+    """What an attention layer needs of its projection when keys are values over their root mean square: short
+    convolution of the query and key heads (the first (H + G) D columns; see :func:`short_conv`), queries scaled to unit
+    RMS per head and multiplied by q_temp at their position, values (the convolved keys) and their factors written to
+    the pages.  Returns (queries [T, H D], float32 copy of the H gate columns from g_off on, or None)."""
+    qk = short_conv(proj, taps, q_start, pos0, slots, hist, False)
+    window_prep(qk, H, G, D, D, None, None, pos, tok_seq, block_table, None, None, eps, None, 0, None, vc, False, H * D,
+                None, q_temp, ks)
+    return qk[:, :H * D].contiguous(), (proj[:, g_off:g_off + H].float() if g_off >= 0 else None)
