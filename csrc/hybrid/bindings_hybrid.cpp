@@ -33,8 +33,7 @@ void launch_hy_gated_join(const void*, float*, const void*, int64_t, const float
 void launch_hy_poly_norm(const void*, int64_t, const float*, void*, int, int, float, bool, hipStream_t);
 bool launch_hy_latent_attention(const void*, const void*, const int32_t*, int, const int32_t*, const int32_t*,
                                 const float*, void*, int, int, int, int, int, int, float, int, bool, bool, int, float*,
-                                float*, int64_t,
-                                hipStream_t);
+                                float*, int64_t, const float*, hipStream_t);
 bool hy_latent_use_mfma(bool, int, int);
 int hy_latent_nsplit(int, int, bool);
 void launch_hy_moe_route(const void*, const void*, const float*, float*, int32_t*, float*, int, int, int, int, bool,
@@ -45,13 +44,18 @@ int hy_moe_max_tiles(int, int);
 void launch_hy_moe_grouped(const uint16_t*, const int32_t*, const float*, const uint16_t*, const uint16_t*, uint16_t*,
                            int32_t*, uint16_t*, uint16_t*, int, int, int, int, int, int, hipStream_t);
 void launch_hy_rms_norm(const void*, float*, const float*, void*, bool, int, int, float, float, hipStream_t);
-void launch_hy_glu(const void*, void*, int64_t, int, float, float, float, bool, hipStream_t);
+void launch_hy_glu(const void*, int64_t, void*, int64_t, int64_t, int, float, float, float, bool, hipStream_t);
+void launch_hy_layer_norm_join(const void*, const void*, float*, const float*, void*, int, int, float, bool, hipStream_t);
+void launch_hy_norm_cols(const void*, int64_t, const float*, void*, int, int, float, bool, hipStream_t);
+void launch_hy_conv_prep(const void*, int64_t, const float*, int, const int32_t*, const int32_t*, const int32_t*,
+                         const int32_t*, void*, const int32_t*, const int32_t*, int, int, int, int, int, int, float,
+                         const float*, float*, void*, int, void*, float*, int, bool, bool, hipStream_t);
 void launch_hy_decay_pow(float*, int64_t, float, hipStream_t);
 void launch_hy_head_norm_gate(const float*, const void*, int, int, const float*, void*, int, int, int, float, bool, bool,
                               hipStream_t);
 void launch_hy_window_prep(void*, int, int, int, int, int, const void*, const float*, const int32_t*, const int32_t*,
                            const int32_t*, int, const float*, const float*, float, const float*, int, void*, void*, int,
-                           void*, int, const float*, int, bool, hipStream_t);
+                           void*, int, const float*, const float*, float*, int, bool, hipStream_t);
 void launch_hy_pool_blocks(const void*, const void*, void*, void*, const int32_t*, int, const int32_t*, const int32_t*, int,
                            int, int, int, int, int, int, bool, hipStream_t);
 void launch_hy_sandwich_join(const void*, const void*, float*, const float*, const float*, const float*, const float*,
@@ -64,7 +68,8 @@ void launch_hy_unrotate_gate(const void*, const int32_t*, const float*, const vo
 int hy_window_rows_cap(int, int, int, bool);
 void launch_hy_window_attention(const void*, int, const void*, const void*, const int32_t*, int, const int32_t*,
                                 const int32_t*, const float*, const float*, void*, int, int, int, int, int, int, int, float,
-                                int, int, int, bool, int, float*, float*, int64_t, int, int, const void*, const void*, const float*, int, hipStream_t);
+                                int, int, int, bool, int, float*, float*, int64_t, int, int, const void*, const void*, const float*, int,
+                                const float*, int64_t, hipStream_t);
 int hy_window_nsplit(bool, int, int, int, int, int, int, int, int, int, int, int, int);
 void launch_hy_short_conv(const void*, int, const float*, const float*, const int32_t*, const int32_t*, const int32_t*,
                           const int32_t*, void*, void*, int, int, int, int, bool, bool, hipStream_t);
@@ -209,23 +214,27 @@ Tensor hy_mlstm_out(const Tensor& o, const Tensor& proj, int64_t g_off, const Te
     return y;
 }
 
-void hy_latent_prep(Tensor& q, const Tensor& dkv, const Tensor& pos, const Tensor& tok_seq, const Tensor& block_table,
-                    const Tensor& w_norm, double eps, const c10::optional<Tensor>& cos_sin, int64_t dims, int64_t rank,
-                    Tensor& cache, c10::optional<Tensor> qa, bool interleaved) {
+void hy_latent_prep(Tensor& q, const c10::optional<Tensor>& dkv, const Tensor& pos, const Tensor& tok_seq,
+                    const Tensor& block_table, const c10::optional<Tensor>& w_norm, double eps,
+                    const c10::optional<Tensor>& cos_sin, int64_t dims, int64_t rank, Tensor& cache, c10::optional<Tensor> qa,
+                    bool interleaved) {
     c10::hip::HIPGuardMasqueradingAsCUDA g(q.device());
-    same_act(q, dkv, "latent_prep: q and dkv in one activation dtype");
     same_act(q, cache, "latent_prep: the cache holds the activation dtype");
-    need(q.dim() == 3 && dkv.dim() == 2 && cache.dim() == 3 && cache.is_contiguous(), "latent_prep: layouts");
-    const int64_t T = q.size(0), H = q.size(1), DK = dkv.size(1), R = DK - rank, D = q.size(2) - R;
+    need(q.dim() == 3 && cache.dim() == 3 && cache.is_contiguous(), "latent_prep: layouts");
+    const int64_t T = q.size(0), H = q.size(1), DK = cache.size(2), R = DK - rank, D = q.size(2) - R;
     // rows may be column ranges of a wider projection: a token's heads side by side, unit column stride
     need(q.stride(2) == 1 && q.stride(1) == q.size(2) && q.stride(0) >= H * q.size(2), "latent_prep: q rows");
-    need(dkv.stride(1) == 1 && dkv.stride(0) >= DK, "latent_prep: dkv rows");
-    need(dkv.size(0) == T && rank >= 1 && R >= 0 && D >= 0 && cache.size(2) == DK, "latent_prep: sizes");
+    need(rank >= 1 && R >= 0 && D >= 0, "latent_prep: sizes");
+    if (dkv) {
+        same_act(q, *dkv, "latent_prep: q and dkv in one activation dtype");
+        need(dkv->dim() == 2 && dkv->size(0) == T && dkv->size(1) == DK && dkv->stride(1) == 1 && dkv->stride(0) >= DK, "latent_prep: dkv rows");
+        need(w_norm.has_value(), "latent_prep: the latent needs its norm weight");
+        flt(*w_norm, "latent_prep: float32 norm weight");
+        need(w_norm->numel() == rank, "latent_prep: norm weight");
+    }
     need(dims % 2 == 0 && dims >= 0 && dims <= R, "latent_prep: rotated columns");
     i32(pos, "latent_prep: pos"); i32(tok_seq, "latent_prep: tok_seq"); i32(block_table, "latent_prep: block_table");
     need(pos.numel() == T && tok_seq.numel() == T && block_table.dim() == 2, "latent_prep: per-token metadata");
-    flt(w_norm, "latent_prep: float32 norm weight");
-    need(w_norm.numel() == rank, "latent_prep: norm weight");
     need(dims == 0 || cos_sin.has_value(), "latent_prep: rotated columns need their table");
     if (cos_sin) {
         flt(*cos_sin, "latent_prep: float32 cos/sin table");
@@ -235,11 +244,12 @@ void hy_latent_prep(Tensor& q, const Tensor& dkv, const Tensor& pos, const Tenso
         same_act(q, *qa, "latent_prep: qa in the activation dtype");
         need(qa->is_contiguous() && qa->dim() == 3 && qa->size(0) == T && qa->size(1) == H && qa->size(2) == DK, "latent_prep: qa [T, H, rank + R]");
     }
-    chronos::launch_hy_latent_prep(q.data_ptr(), q.stride(0), dkv.data_ptr(), dkv.stride(0), pos.data_ptr<int32_t>(),
-                                   tok_seq.data_ptr<int32_t>(), block_table.data_ptr<int32_t>(), (int)block_table.size(1),
-                                   w_norm.data_ptr<float>(), (float)eps, cos_sin ? cos_sin->data_ptr<float>() : nullptr,
-                                   (int)dims, interleaved, (int)rank, (int)R, (int)H, (int)D, cache.data_ptr(),
-                                   (int)cache.size(1), qa ? qa->data_ptr() : nullptr, (int)T, f32(q), stream());
+    chronos::launch_hy_latent_prep(q.data_ptr(), q.stride(0), dkv ? dkv->data_ptr() : nullptr, dkv ? dkv->stride(0) : 0,
+                                   pos.data_ptr<int32_t>(), tok_seq.data_ptr<int32_t>(), block_table.data_ptr<int32_t>(),
+                                   (int)block_table.size(1), dkv ? w_norm->data_ptr<float>() : nullptr, (float)eps,
+                                   cos_sin ? cos_sin->data_ptr<float>() : nullptr, (int)dims, interleaved, (int)rank, (int)R,
+                                   (int)H, (int)D, cache.data_ptr(), (int)cache.size(1), qa ? qa->data_ptr() : nullptr, (int)T,
+                                   f32(q), stream());
 }
 
 // the first gate column of row 0 of a [T, C] activation tensor, after checking that columns off .. off + n exist
@@ -316,7 +326,7 @@ Tensor hy_poly_norm(const Tensor& z, int64_t F, const Tensor& abce, double eps) 
 
 Tensor hy_latent_attention(const Tensor& qa, const Tensor& cache, const Tensor& block_table, const Tensor& q_start,
                            const Tensor& pos, const c10::optional<Tensor>& gate, double scale, int64_t rank,
-                           int64_t max_q, int64_t window, bool two_term) {
+                           int64_t max_q, int64_t window, bool two_term, const c10::optional<Tensor>& sink) {
     c10::hip::HIPGuardMasqueradingAsCUDA g(qa.device());
     same_act(qa, cache, "latent_attention: queries and cache in one activation dtype");
     need(qa.dim() == 3 && qa.is_contiguous() && cache.dim() == 3 && cache.is_contiguous(), "latent_attention: layouts");
@@ -327,6 +337,7 @@ Tensor hy_latent_attention(const Tensor& qa, const Tensor& cache, const Tensor& 
     const int64_t B = q_start.numel() - 1;
     need(block_table.dim() == 2 && block_table.size(0) >= B && pos.numel() == T && window >= 0, "latent_attention: metadata");
     if (gate) { flt(*gate, "latent_attention: float32 gate"); need(gate->numel() == T * H, "latent_attention: gate [T, H]"); }
+    if (sink) { flt(*sink, "latent_attention: float32 sinks"); need(sink->numel() == H, "latent_attention: sink [H]"); }
     auto out = at::empty({T, H, rank}, qa.options());
     if (T == 0 || B <= 0) return out;
     // few workgroups over long contexts (decode rows, a lone short portion): split the key range over more workgroups
@@ -348,7 +359,8 @@ Tensor hy_latent_attention(const Tensor& qa, const Tensor& cache, const Tensor& 
         q_start.data_ptr<int32_t>(), pos.data_ptr<int32_t>(), gate ? gate->data_ptr<float>() : nullptr, out.data_ptr(),
         (int)B, (int)H, (int)DK, (int)rank, (int)cache.size(1), mq, (float)scale, (int)window,
         two_term, f32(qa), nsplit,
-        nsplit > 1 ? part_o.data_ptr<float>() : nullptr, nsplit > 1 ? part_ml.data_ptr<float>() : nullptr, T * H, stream());
+        nsplit > 1 ? part_o.data_ptr<float>() : nullptr, nsplit > 1 ? part_ml.data_ptr<float>() : nullptr, T * H,
+        sink ? sink->data_ptr<float>() : nullptr, stream());
     TORCH_CHECK(ok, "chronos hybrid op: latent_attention has no launch geometry for heads=", H, " row width=", DK,
                 " rank=", rank, " (rank <= 512; 16 keys and 4 query rows must fit the LDS)");
     return out;
@@ -430,9 +442,81 @@ Tensor hy_glu(const Tensor& gu, double limit, double slope, double shift) {
     c10::hip::HIPGuardMasqueradingAsCUDA g(gu.device());
     need(is_act(gu) && gu.dim() == 2 && gu.is_contiguous() && gu.size(1) % 2 == 0, "glu: [T, 2F] activation tensor");
     auto y = at::empty({gu.size(0), gu.size(1) / 2}, gu.options());
-    chronos::launch_hy_glu(gu.data_ptr(), y.data_ptr(), gu.size(0), (int)(gu.size(1) / 2), (float)limit, (float)slope,
-                           (float)shift, f32(gu), stream());
+    chronos::launch_hy_glu(gu.data_ptr(), gu.size(1), y.data_ptr(), y.size(1), gu.size(0), (int)(gu.size(1) / 2),
+                           (float)limit, (float)slope, (float)shift, f32(gu), stream());
     return y;
+}
+
+void hy_glu_cols(const Tensor& src, int64_t off, int64_t F, double limit, double slope, double shift, Tensor& out) {
+    c10::hip::HIPGuardMasqueradingAsCUDA g(src.device());
+    same_act(src, out, "glu_cols: one activation dtype");
+    need(src.dim() == 2 && out.dim() == 2 && src.stride(1) == 1 && out.stride(1) == 1 && src.stride(0) >= src.size(1) &&
+             out.stride(0) >= F, "glu_cols: rows with unit column stride");
+    need(F >= 1 && off >= 0 && off + 2 * F <= src.size(1) && out.size(0) == src.size(0) && out.size(1) == F, "glu_cols: columns");
+    chronos::launch_hy_glu(static_cast<const char*>(src.data_ptr()) + off * src.element_size(), src.stride(0), out.data_ptr(),
+                           out.stride(0), src.size(0), (int)F, (float)limit, (float)slope, (float)shift, f32(src), stream());
+}
+
+Tensor hy_layer_norm_join(const c10::optional<Tensor>& y, const c10::optional<Tensor>& y2, Tensor& x,
+                          const c10::optional<Tensor>& wb, double eps, bool out_f32) {
+    c10::hip::HIPGuardMasqueradingAsCUDA g(x.device());
+    flt(x, "layer_norm_join: float32 residual");
+    need(x.dim() == 2, "layer_norm_join: x [T, d]");
+    const int64_t T = x.size(0), d = x.size(1);
+    if (y) need(is_act(*y) && f32(*y) == out_f32 && y->is_contiguous() && y->sizes() == x.sizes(), "layer_norm_join: y [T, d] in the activation dtype");
+    if (y2) need(y.has_value() && y2->scalar_type() == y->scalar_type() && y2->is_contiguous() && y2->sizes() == x.sizes(), "layer_norm_join: y2 like y");
+    if (wb) { flt(*wb, "layer_norm_join: float32 weights"); need(wb->numel() == 2 * d, "layer_norm_join: weights w | b"); }
+    const auto o = x.options().dtype(out_f32 ? at::kFloat : at::kBFloat16);
+    Tensor h = wb ? at::empty({T, d}, o) : at::empty({0}, o);
+    chronos::launch_hy_layer_norm_join(y ? y->data_ptr() : nullptr, y2 ? y2->data_ptr() : nullptr, x.data_ptr<float>(),
+                                       wb ? wb->data_ptr<float>() : nullptr, wb ? h.data_ptr() : nullptr, (int)T, (int)d,
+                                       (float)eps, out_f32, stream());
+    return h;
+}
+
+Tensor hy_norm_cols(const Tensor& src, int64_t off, int64_t n, const Tensor& w, double eps) {
+    c10::hip::HIPGuardMasqueradingAsCUDA g(src.device());
+    need(is_act(src) && src.dim() == 2 && src.stride(1) == 1 && off >= 0 && n >= 1 && off + n <= src.size(1), "norm_cols: columns off .. off + n of [T, C]");
+    flt(w, "norm_cols: float32 weight");
+    need(w.numel() == n, "norm_cols: weight [n]");
+    auto out = at::empty({src.size(0), n}, src.options());
+    chronos::launch_hy_norm_cols(static_cast<const char*>(src.data_ptr()) + off * src.element_size(), src.stride(0),
+                                 w.data_ptr<float>(), out.data_ptr(), (int)src.size(0), (int)n, (float)eps, f32(src), stream());
+    return out;
+}
+
+std::tuple<Tensor, Tensor> hy_conv_prep(const Tensor& proj, const Tensor& taps, const Tensor& tok_seq, const Tensor& q_start,
+                                        const Tensor& pos0, const Tensor& slots, Tensor& hist, const Tensor& pos,
+                                        const Tensor& block_table, int64_t H, int64_t G, int64_t D, double eps,
+                                        const c10::optional<Tensor>& q_temp, Tensor& ks, Tensor& vc, int64_t g_off,
+                                        int64_t max_q) {
+    c10::hip::HIPGuardMasqueradingAsCUDA g(proj.device());
+    same_act(proj, hist, "conv_prep: the history holds the activation dtype");
+    same_act(proj, vc, "conv_prep: the cache holds the activation dtype");
+    flt(taps, "conv_prep: float32 taps");
+    flt(ks, "conv_prep: float32 key factors");
+    need(proj.dim() == 2 && proj.is_contiguous() && taps.dim() == 2 && hist.dim() == 3 && hist.is_contiguous() &&
+             vc.dim() == 4 && vc.is_contiguous(), "conv_prep: layouts");
+    const int64_t T = proj.size(0), C = (H + G) * D, K = taps.size(1), B = slots.numel();
+    need(H >= 1 && G >= 1 && D >= 1 && D <= 256 && C <= proj.size(1) && taps.size(0) == C && K >= 1, "conv_prep: heads, D <= 256, taps [C, K]");
+    need(hist.size(1) == K - 1 && hist.size(2) == C, "conv_prep: history [slots, K - 1, C]");
+    need(vc.size(2) == G && vc.size(3) == D && ks.dim() == 3 && ks.size(0) == vc.size(0) && ks.size(1) == vc.size(1) && ks.size(2) == G, "conv_prep: cache [NB, BS, G, D], factors [NB, BS, G]");
+    i32(tok_seq, "conv_prep: tok_seq"); i32(q_start, "conv_prep: q_start"); i32(pos0, "conv_prep: pos0"); i32(slots, "conv_prep: slots");
+    i32(pos, "conv_prep: pos"); i32(block_table, "conv_prep: block_table");
+    need(tok_seq.numel() == T && pos.numel() == T && q_start.numel() == B + 1 && pos0.numel() == B && block_table.dim() == 2 &&
+             block_table.size(0) >= B, "conv_prep: metadata");
+    need(g_off < 0 || g_off + H <= proj.size(1), "conv_prep: gate columns");
+    if (q_temp) flt(*q_temp, "conv_prep: float32 temperatures");
+    auto q = at::empty({T, H * D}, proj.options());
+    auto gate = at::empty({g_off >= 0 ? T : 0, H}, proj.options().dtype(at::kFloat));
+    chronos::launch_hy_conv_prep(proj.data_ptr(), proj.size(1), taps.data_ptr<float>(), (int)K, tok_seq.data_ptr<int32_t>(),
+                                 q_start.data_ptr<int32_t>(), pos0.data_ptr<int32_t>(), slots.data_ptr<int32_t>(),
+                                 hist.data_ptr(), pos.data_ptr<int32_t>(), block_table.data_ptr<int32_t>(),
+                                 (int)block_table.size(1), (int)T, (int)B, (int)H, (int)G, (int)D, (float)eps,
+                                 q_temp ? q_temp->data_ptr<float>() : nullptr, ks.data_ptr<float>(), vc.data_ptr(),
+                                 (int)vc.size(1), q.data_ptr(), g_off >= 0 ? gate.data_ptr<float>() : nullptr, (int)g_off,
+                                 max_q == 1, f32(proj), stream());
+    return {q, gate};
 }
 
 void hy_decay_pow(Tensor& z, double p) {
@@ -458,12 +542,13 @@ Tensor hy_head_norm_gate(const Tensor& o, const Tensor& src, int64_t g_off, cons
 Tensor hy_window_prep(Tensor& qkv, int64_t H, int64_t G, int64_t D, int64_t Dv, const c10::optional<Tensor>& v_first,
                       const c10::optional<Tensor>& lam, const Tensor& pos, const Tensor& tok_seq, const Tensor& block_table,
                       const c10::optional<Tensor>& q_norm, const c10::optional<Tensor>& k_norm, double eps,
-                      const c10::optional<Tensor>& cos_sin, int64_t dims, Tensor& kc, Tensor& vc, bool emit_v,
-                      int64_t v_off, const c10::optional<Tensor>& v_cos_sin) {
+                      const c10::optional<Tensor>& cos_sin, int64_t dims, c10::optional<Tensor> kc, Tensor& vc, bool emit_v,
+                      int64_t v_off, const c10::optional<Tensor>& v_cos_sin, const c10::optional<Tensor>& q_temp,
+                      c10::optional<Tensor> ks) {
     c10::hip::HIPGuardMasqueradingAsCUDA g(qkv.device());
-    same_act(qkv, kc, "window_prep: the caches hold the activation dtype");
+    need(kc.has_value() != ks.has_value(), "window_prep: a key cache, or the keys' factors");
     same_act(qkv, vc, "window_prep: the caches hold the activation dtype");
-    need(qkv.dim() == 2 && qkv.is_contiguous() && kc.dim() == 4 && vc.dim() == 4 && kc.is_contiguous() && vc.is_contiguous(), "window_prep: layouts");
+    need(qkv.dim() == 2 && qkv.is_contiguous() && vc.dim() == 4 && vc.is_contiguous(), "window_prep: layouts");
     const int64_t T = qkv.size(0);
     if (v_off < 0) v_off = (H + G) * D;   // the values follow the keys
     need(H >= 1 && G >= 1 && H % G == 0 && D >= 1 && Dv >= 1 && qkv.size(1) >= (H + G) * D && v_off + G * Dv <= qkv.size(1), "window_prep: qkv width");
@@ -471,7 +556,17 @@ Tensor hy_window_prep(Tensor& qkv, int64_t H, int64_t G, int64_t D, int64_t Dv, 
         flt(*v_cos_sin, "window_prep: float32 cos/sin table of the values");
         need(Dv % 2 == 0 && v_cos_sin->dim() == 2 && v_cos_sin->size(1) == Dv, "window_prep: the values' table is [P, Dv], Dv even");
     }
-    need(kc.size(2) == G && kc.size(3) == D && vc.size(2) == G && vc.size(3) == Dv && vc.size(0) == kc.size(0) && vc.size(1) == kc.size(1), "window_prep: cache shapes");
+    need(vc.size(2) == G && vc.size(3) == Dv, "window_prep: cache shapes");
+    if (kc) {
+        same_act(qkv, *kc, "window_prep: the caches hold the activation dtype");
+        need(kc->dim() == 4 && kc->is_contiguous() && kc->size(2) == G && kc->size(3) == D && vc.size(0) == kc->size(0) && vc.size(1) == kc->size(1), "window_prep: cache shapes");
+    } else {
+        flt(*ks, "window_prep: float32 key factors");
+        need(ks->dim() == 3 && ks->size(0) == vc.size(0) && ks->size(1) == vc.size(1) && ks->size(2) == G, "window_prep: key factors [NB, BS, G]");
+        need(!q_norm.has_value() && dims == 0 && !v_first.has_value() && !v_cos_sin.has_value() && D == Dv && v_off == H * D,
+             "window_prep: unit keys are plain values over their root mean square");
+    }
+    if (q_temp) flt(*q_temp, "window_prep: float32 temperatures");
     i32(pos, "window_prep: pos"); i32(tok_seq, "window_prep: tok_seq"); i32(block_table, "window_prep: block_table");
     need(pos.numel() == T && tok_seq.numel() == T && block_table.dim() == 2, "window_prep: per-token metadata");
     need(q_norm.has_value() == k_norm.has_value(), "window_prep: queries and keys are normed together or not at all");
@@ -498,18 +593,29 @@ Tensor hy_window_prep(Tensor& qkv, int64_t H, int64_t G, int64_t D, int64_t Dv, 
                                    pos.data_ptr<int32_t>(), tok_seq.data_ptr<int32_t>(), block_table.data_ptr<int32_t>(),
                                    (int)block_table.size(1), q_norm ? q_norm->data_ptr<float>() : nullptr,
                                    k_norm ? k_norm->data_ptr<float>() : nullptr, (float)eps,
-                                   dims > 0 ? cos_sin->data_ptr<float>() : nullptr, (int)dims, kc.data_ptr(), vc.data_ptr(),
-                                   (int)kc.size(1), emit_v ? v_out.data_ptr() : nullptr, (int)v_off,
-                                   v_cos_sin ? v_cos_sin->data_ptr<float>() : nullptr, (int)T, f32(qkv), stream());
+                                   dims > 0 ? cos_sin->data_ptr<float>() : nullptr, (int)dims, kc ? kc->data_ptr() : nullptr,
+                                   vc.data_ptr(), (int)vc.size(1), emit_v ? v_out.data_ptr() : nullptr, (int)v_off,
+                                   v_cos_sin ? v_cos_sin->data_ptr<float>() : nullptr,
+                                   q_temp ? q_temp->data_ptr<float>() : nullptr, ks ? ks->data_ptr<float>() : nullptr, (int)T,
+                                   f32(qkv), stream());
     return v_out;
 }
 
-Tensor hy_window_attention(const Tensor& qkv, const Tensor& kc, const Tensor& vc, const Tensor& block_table,
+// out_cols (optional): where the output goes, [T, H Dv] columns of wider rows; the returned tensor is then empty
+Tensor hy_window_attention(const Tensor& qkv, const c10::optional<Tensor>& kc_in, const Tensor& vc, const Tensor& block_table,
                            const Tensor& q_start, const Tensor& pos, const c10::optional<Tensor>& sink,
                            const c10::optional<Tensor>& gate, double scale, int64_t window, int64_t keep, int64_t chunk,
                            int64_t H, int64_t max_q, int64_t pool, const c10::optional<Tensor>& kp,
-                           const c10::optional<Tensor>& vp, const c10::optional<Tensor>& v_cos_sin, int64_t g_off) {
+                           const c10::optional<Tensor>& vp, const c10::optional<Tensor>& v_cos_sin, int64_t g_off,
+                           const c10::optional<Tensor>& ks, c10::optional<Tensor> out_cols) {
     c10::hip::HIPGuardMasqueradingAsCUDA g(qkv.device());
+    need(kc_in.has_value() != ks.has_value(), "window_attention: a key cache, or the keys' factors");
+    const Tensor& kc = kc_in ? *kc_in : vc;   // unit keys: the value cache is read as both
+    if (ks) {
+        flt(*ks, "window_attention: float32 key factors");
+        need(vc.dim() == 4 && ks->dim() == 3 && ks->size(0) == vc.size(0) && ks->size(1) == vc.size(1) && ks->size(2) == vc.size(2) && pool == 0,
+             "window_attention: key factors [NB, BS, G], no pooled blocks");
+    }
     same_act(qkv, kc, "window_attention: queries and caches in one activation dtype");
     same_act(qkv, vc, "window_attention: queries and caches in one activation dtype");
     need(qkv.dim() == 2 && qkv.is_contiguous() && kc.dim() == 4 && vc.dim() == 4 && kc.is_contiguous() && vc.is_contiguous(), "window_attention: layouts");
@@ -537,7 +643,13 @@ Tensor hy_window_attention(const Tensor& qkv, const Tensor& kc, const Tensor& vc
         need(Dv % 2 == 0 && v_cos_sin->dim() == 2 && v_cos_sin->size(1) == Dv, "window_attention: the values' table is [P, Dv], Dv even");
     }
     need(g_off < 0 || g_off + H * Dv <= qkv.size(1), "window_attention: the gate columns lie in the projection's row");
-    auto out = at::empty({T, H * Dv}, qkv.options());
+    if (out_cols) {
+        same_act(qkv, *out_cols, "window_attention: output in the activation dtype");
+        need(out_cols->dim() == 2 && out_cols->size(0) == T && out_cols->size(1) == H * Dv && out_cols->stride(1) == 1 &&
+                 out_cols->stride(0) >= H * Dv && !v_cos_sin.has_value() && g_off < 0, "window_attention: output columns [T, H Dv]");
+        need(reinterpret_cast<uintptr_t>(out_cols->data_ptr()) % 8 == 0, "window_attention: output columns start on 8 bytes");
+    }
+    auto out = at::empty({out_cols ? 0 : T, H * Dv}, qkv.options());
     if (T == 0 || B <= 0) return out;
     const int mq = (int)std::max<int64_t>(1, max_q);
     const int nsplit = chronos::hy_window_nsplit(f32(qkv), (int)qkv.size(1), (int)B, mq, (int)H, (int)G, (int)D, (int)Dv,
@@ -552,12 +664,14 @@ Tensor hy_window_attention(const Tensor& qkv, const Tensor& kc, const Tensor& vc
                                         block_table.data_ptr<int32_t>(), (int)block_table.size(1),
                                         q_start.data_ptr<int32_t>(), pos.data_ptr<int32_t>(),
                                         sink ? sink->data_ptr<float>() : nullptr, gate ? gate->data_ptr<float>() : nullptr,
-                                        out.data_ptr(), (int)B, mq, (int)H, (int)G, (int)D, (int)Dv, (int)kc.size(1),
+                                        out_cols ? out_cols->data_ptr() : out.data_ptr(), (int)B, mq, (int)H, (int)G, (int)D,
+                                        (int)Dv, (int)kc.size(1),
                                         (float)scale, (int)window, (int)keep, (int)chunk, f32(qkv), nsplit,
                                         nsplit > 1 ? part_o.data_ptr<float>() : nullptr,
                                         nsplit > 1 ? part_ml.data_ptr<float>() : nullptr, T * H, (int)pool, (int)EP,
                                         pool > 0 ? kp->data_ptr() : nullptr, pool > 0 ? vp->data_ptr() : nullptr,
                                         v_cos_sin ? v_cos_sin->data_ptr<float>() : nullptr, g_off >= 0 ? (int)g_off : -1,
+                                        ks ? ks->data_ptr<float>() : nullptr, out_cols ? out_cols->stride(0) : H * Dv,
                                         stream());
     return out;
 }
@@ -915,7 +1029,7 @@ TORCH_LIBRARY_FRAGMENT(chronos, m) {
     m.def("hy_mlstm_scan(Tensor proj, Tensor gate_pre, Tensor q_start, Tensor pos0, Tensor slots, Tensor(a!) S, "
           "Tensor(b!) n, Tensor(c!) m, int H, int D, int Dv, float cap) -> Tensor");
     m.def("hy_mlstm_out(Tensor o, Tensor proj, int g_off, Tensor w, float eps, bool out_f32) -> Tensor");
-    m.def("hy_latent_prep(Tensor(a!) q, Tensor dkv, Tensor pos, Tensor tok_seq, Tensor block_table, Tensor w_norm, "
+    m.def("hy_latent_prep(Tensor(a!) q, Tensor? dkv, Tensor pos, Tensor tok_seq, Tensor block_table, Tensor? w_norm, "
           "float eps, Tensor? cos_sin, int dims, int rank, Tensor(b!) cache, Tensor(c!)? qa=None, "
           "bool interleaved=False) -> ()");
     m.def("hy_head_matmul(Tensor a, Tensor w, Tensor(a!) out, Tensor? gate_src, int g_off) -> ()");
@@ -924,20 +1038,28 @@ TORCH_LIBRARY_FRAGMENT(chronos, m) {
           "Tensor(b!)? hist, int run, Tensor? dwa) -> Tensor");
     m.def("hy_poly_norm(Tensor z, int F, Tensor abce, float eps) -> Tensor");
     m.def("hy_latent_attention(Tensor qa, Tensor cache, Tensor block_table, Tensor q_start, Tensor pos, Tensor? gate, "
-          "float scale, int rank, int max_q, int window=0, bool two_term=False) -> Tensor");
+          "float scale, int rank, int max_q, int window=0, bool two_term=False, Tensor? sink=None) -> Tensor");
     m.def("hy_moe_route(Tensor h, Tensor w, Tensor corr, int top) -> (Tensor, Tensor)");
     m.def("hy_moe_ffn(Tensor h, Tensor idx, Tensor wt, Tensor w_up, Tensor w_down, int act) -> Tensor");
     m.def("hy_rms_norm(Tensor x, Tensor w, float eps, bool out_f32) -> Tensor");
     m.def("hy_scale_add_rms_norm(Tensor y, Tensor(a!) x, Tensor w, float alpha, float eps, bool out_f32) -> Tensor");
     m.def("hy_glu(Tensor gu, float limit, float slope, float shift) -> Tensor");
+    m.def("hy_glu_cols(Tensor src, int off, int F, float limit, float slope, float shift, Tensor(a!) out) -> ()");
+    m.def("hy_layer_norm_join(Tensor? y, Tensor? y2, Tensor(a!) x, Tensor? wb, float eps, bool out_f32) -> Tensor");
+    m.def("hy_norm_cols(Tensor src, int off, int n, Tensor w, float eps) -> Tensor");
+    m.def("hy_conv_prep(Tensor proj, Tensor taps, Tensor tok_seq, Tensor q_start, Tensor pos0, Tensor slots, Tensor(a!) hist, "
+          "Tensor pos, Tensor block_table, int H, int G, int D, float eps, Tensor? q_temp, Tensor(b!) ks, Tensor(c!) vc, "
+          "int g_off, int max_q) -> (Tensor, Tensor)");
     m.def("hy_decay_pow(Tensor(a!) z, float p) -> ()");
     m.def("hy_head_norm_gate(Tensor o, Tensor src, int g_off, Tensor w, float eps, bool silu_gate, bool out_f32) -> Tensor");
     m.def("hy_window_prep(Tensor(a!) qkv, int H, int G, int D, int Dv, Tensor? v_first, Tensor? lam, Tensor pos, "
           "Tensor tok_seq, Tensor block_table, Tensor? q_norm, Tensor? k_norm, float eps, Tensor? cos_sin, int dims, "
-          "Tensor(b!) kc, Tensor(c!) vc, bool emit_v, int v_off=-1, Tensor? v_cos_sin=None) -> Tensor");
-    m.def("hy_window_attention(Tensor qkv, Tensor kc, Tensor vc, Tensor block_table, Tensor q_start, Tensor pos, "
+          "Tensor(b!)? kc, Tensor(c!) vc, bool emit_v, int v_off=-1, Tensor? v_cos_sin=None, Tensor? q_temp=None, "
+          "Tensor(d!)? ks=None) -> Tensor");
+    m.def("hy_window_attention(Tensor qkv, Tensor? kc, Tensor vc, Tensor block_table, Tensor q_start, Tensor pos, "
           "Tensor? sink, Tensor? gate, float scale, int window, int keep, int chunk, int H, int max_q, int pool=0, "
-          "Tensor? kp=None, Tensor? vp=None, Tensor? v_cos_sin=None, int g_off=-1) -> Tensor");
+          "Tensor? kp=None, Tensor? vp=None, Tensor? v_cos_sin=None, int g_off=-1, Tensor? ks=None, "
+          "Tensor(a!)? out_cols=None) -> Tensor");
     m.def("hy_pool_blocks(Tensor kc, Tensor vc, Tensor(a!) kp, Tensor(b!) vp, Tensor block_table, Tensor q_start, "
           "Tensor pos0, int pool, int max_q) -> ()");
     m.def("hy_sandwich_join(Tensor? y, Tensor? y2, Tensor(a!) x, Tensor? w_y, Tensor? w_out, Tensor? w_a, Tensor? w_b, "
@@ -985,6 +1107,10 @@ TORCH_LIBRARY_IMPL(chronos, CUDA, m) {
     m.impl("hy_rms_norm", &hy_rms_norm);
     m.impl("hy_scale_add_rms_norm", &hy_scale_add_rms_norm);
     m.impl("hy_glu", &hy_glu);
+    m.impl("hy_glu_cols", &hy_glu_cols);
+    m.impl("hy_layer_norm_join", &hy_layer_norm_join);
+    m.impl("hy_norm_cols", &hy_norm_cols);
+    m.impl("hy_conv_prep", &hy_conv_prep);
     m.impl("hy_decay_pow", &hy_decay_pow);
     m.impl("hy_head_norm_gate", &hy_head_norm_gate);
     m.impl("hy_window_prep", &hy_window_prep);

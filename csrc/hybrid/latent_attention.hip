@@ -16,6 +16,7 @@
 //                     over 4 waves; 64-key tiles of the cache are staged in LDS; lanes are keys for the scores
 //                     (float accumulation, causal mask by each row's own position, online softmax in float) and
 //                     latent columns for the output.  Serves prefill chunks and decode rows (a tile of one token).
+//                     A sink per head may join the softmax denominator after the last key (no key, no value).
 //                     With window > 0 a row sees only the last `window` positions up to its own: the walk starts at
 //                     the tile of the first row's first visible key, and each row masks by its own position.
 #include <cstdlib>
@@ -37,19 +38,22 @@ __global__ void __launch_bounds__(256) latent_prep_kernel(
     const int blk = block_table[(int64_t)tok_seq[t] * max_blocks + p / BS];
     const int DK = rank + R;
     T* crow = cache + ((int64_t)blk * BS + p % BS) * DK;
-    const T* drow = dkv + t * ldkv;
-    float ss = 0.f;
-    for (int i = threadIdx.x; i < rank; i += 256) {
-        const float v = ld<T>(drow + i);
-        ss += v * v;
+    const bool own = dkv != nullptr;       // else the cache is another layer's: only the queries are rotated
+    const T* drow = own ? dkv + t * ldkv : nullptr;
+    if (own) {
+        float ss = 0.f;
+        for (int i = threadIdx.x; i < rank; i += 256) {
+            const float v = ld<T>(drow + i);
+            ss += v * v;
+        }
+        const float inv = 1.f / sqrtf(block_sum(ss, red) / (float)rank + eps);
+        for (int i = threadIdx.x; i < rank; i += 256) st<T>(crow + i, ld<T>(drow + i) * inv * w_norm[i]);
     }
-    const float inv = 1.f / sqrtf(block_sum(ss, red) / (float)rank + eps);
-    for (int i = threadIdx.x; i < rank; i += 256) st<T>(crow + i, ld<T>(drow + i) * inv * w_norm[i]);
     const int half = dims / 2;
     const float* cs = cos_sin + (int64_t)p * dims;
     // rows to rotate: the shared key part (row 0) and every head's rotated query columns.  Each thread owns whole pairs
     // (columns lo and hi), so rotating in place reads nothing another thread writes; columns past `dims` are copied.
-    for (int i = threadIdx.x; i < (H + 1) * half; i += 256) {
+    for (int i = threadIdx.x + (own ? 0 : half); i < (H + 1) * half; i += 256) {
         const int row = i / half, k = i % half;
         const int lo = inter ? 2 * k : k, hi = inter ? 2 * k + 1 : k + half;
         const T* src = row == 0 ? drow + rank : q + t * ldq + (int64_t)(row - 1) * (D + R) + D;
@@ -60,7 +64,7 @@ __global__ void __launch_bounds__(256) latent_prep_kernel(
         st<T>(dst + hi, v * c + u * s);
     }
     const int rest = R - dims;
-    for (int i = threadIdx.x; i < (qa != nullptr ? H + 1 : 1) * rest; i += 256) {
+    for (int i = threadIdx.x + (own ? 0 : rest); i < (qa != nullptr ? H + 1 : 1) * rest; i += 256) {
         const int row = i / rest, k = dims + i % rest;
         if (row == 0) crow[rank + k] = drow[rank + k];
         else qa[(t * H + row - 1) * DK + rank + k] = q[t * ldq + (int64_t)(row - 1) * (D + R) + D + k];
@@ -87,7 +91,8 @@ template <typename T, int DVL>
 __global__ void __launch_bounds__(256) latent_attention_kernel(
         const T* __restrict__ qa, const T* __restrict__ cache, const int32_t* __restrict__ block_table, int max_blocks,
         const int32_t* __restrict__ q_start, const int32_t* __restrict__ pos, const float* __restrict__ gate,
-        T* __restrict__ out, int H, int DK, int rank, int BS, int RBLK, int KT, int kstride, float scale, int window) {
+        T* __restrict__ out, int H, int DK, int rank, int BS, int RBLK, int KT, int kstride, float scale, int window,
+        const float* __restrict__ sink) {
     constexpr int E = Word<T>::E, RB = 4, RWMAX = 16;
     extern __shared__ __attribute__((aligned(16))) uint32_t smem[];
     const int b = blockIdx.x;
@@ -211,6 +216,10 @@ __global__ void __launch_bounds__(256) latent_attention_kernel(
         if (r < r1) {
             const int64_t grow = (int64_t)t0 * H + rb0 + r;  // row of qa / gate / out
             float f = 1.f / lrow[i];
+            if (sink != nullptr) {   // exp(sink) joins the denominator, without a value
+                const float sk = sink[grow % H], mn = fmaxf(mrow[i], sk), c = expf(mrow[i] - mn);
+                f = c / (lrow[i] * c + expf(sk - mn));
+            }
             if (gate != nullptr) f *= sigmoidf_(gate[grow]);
 #pragma unroll
             for (int v = 0; v < DVL; ++v) {
@@ -258,7 +267,8 @@ bool hy_latent_geometry(int H, int DK, int esize, int max_q, int lds_limit, int*
 template <typename T, int DVL>
 static void latent_attn_t(const T* qa, const T* cache, const int32_t* bt, int max_blocks, const int32_t* q_start,
                           const int32_t* pos, const float* gate, T* out, int B, int H, int DK, int rank, int BS,
-                          int max_q, int RBLK, int KT, int kstride, int bytes, float scale, int window, hipStream_t s) {
+                          int max_q, int RBLK, int KT, int kstride, int bytes, float scale, int window, const float* sink,
+                          hipStream_t s) {
     auto kern = hy::latent_attention_kernel<T, DVL>;
     static int set_bytes = 0;
     if (bytes > set_bytes) {  // raise the dynamic-LDS ceiling of this instantiation once per size
@@ -266,12 +276,12 @@ static void latent_attn_t(const T* qa, const T* cache, const int32_t* bt, int ma
         set_bytes = bytes;
     }
     const dim3 grid(B, (max_q * H + RBLK - 1) / RBLK);
-    kern<<<grid, 256, bytes, s>>>(qa, cache, bt, max_blocks, q_start, pos, gate, out, H, DK, rank, BS, RBLK, KT, kstride, scale, window);
+    kern<<<grid, 256, bytes, s>>>(qa, cache, bt, max_blocks, q_start, pos, gate, out, H, DK, rank, BS, RBLK, KT, kstride, scale, window, sink);
 }
 
 bool launch_hy_latent_attention_mfma(const uint16_t*, const uint16_t*, const int32_t*, int, const int32_t*, const int32_t*,
                                      const float*, uint16_t*, int, int, int, int, int, int, float, int, bool, int, float*,
-                                     float*, int64_t, hipStream_t);
+                                     float*, int64_t, const float*, hipStream_t);
 bool hy_latent_mfma_ok(int DK, int rank);
 
 // whether this call goes to the matrix-core kernel (bfloat16 at its sizes; CHRONOS_LATENT_MFMA=0 keeps the general
@@ -287,15 +297,16 @@ bool hy_latent_use_mfma(bool f32, int DK, int rank) {
 bool launch_hy_latent_attention(const void* qa, const void* cache, const int32_t* bt, int max_blocks,
                                 const int32_t* q_start, const int32_t* pos, const float* gate, void* out, int B, int H,
                                 int DK, int rank, int BS, int max_q, float scale, int window, bool two_term, bool f32,
-                                int nsplit, float* part_o, float* part_ml, int64_t total_rows, hipStream_t s) {
+                                int nsplit, float* part_o, float* part_ml, int64_t total_rows, const float* sink,
+                                hipStream_t s) {
     if (B == 0 || max_q == 0) return true;
     if (hy_latent_use_mfma(f32, DK, rank))
         return launch_hy_latent_attention_mfma((const uint16_t*)qa, (const uint16_t*)cache, bt, max_blocks, q_start, pos, gate,
                                                (uint16_t*)out, B, H, DK, rank, BS, max_q, scale, window, two_term, nsplit,
-                                               part_o, part_ml, total_rows, s);
+                                               part_o, part_ml, total_rows, sink, s);
     int RBLK, KT, kstride, bytes;
     if (rank > 512 || !hy_latent_geometry(H, DK, f32 ? 4 : 2, max_q, 160 * 1024, &RBLK, &KT, &kstride, &bytes)) return false;
-#define HY_LA(TT, DVL) latent_attn_t<TT, DVL>((const TT*)qa, (const TT*)cache, bt, max_blocks, q_start, pos, gate, (TT*)out, B, H, DK, rank, BS, max_q, RBLK, KT, kstride, bytes, scale, window, s)
+#define HY_LA(TT, DVL) latent_attn_t<TT, DVL>((const TT*)qa, (const TT*)cache, bt, max_blocks, q_start, pos, gate, (TT*)out, B, H, DK, rank, BS, max_q, RBLK, KT, kstride, bytes, scale, window, sink, s)
     const int dvl = (rank + 63) / 64;
     if (f32) {
         if (dvl <= 1) HY_LA(float, 1); else if (dvl <= 2) HY_LA(float, 2); else if (dvl <= 4) HY_LA(float, 4); else HY_LA(float, 8);

@@ -15,6 +15,7 @@
 //     fixed permutation of the 32 keys, the same one the transposed value image is read with), so the weights never
 //     leave registers.  Accumulators: rank / 16 tiles x 4 registers.  Optionally each weight enters as two
 //     bfloat16 terms (rounded value + remainder), which keeps the float softmax weights nearly exact.
+// After the last key a sink per head may join the denominator.
 // With a window a row sees only its last `window` positions: the walk starts at the tile of the first row's first
 // visible key and every row masks by its own position.
 // Sizes: DK % 8 == 0 (the last 32-column step of the scores is zero-filled), rank % 16 == 0, DK <= 576, rank <= 512.
@@ -39,7 +40,8 @@ __global__ void __launch_bounds__(64 * NW) latent_attention_mfma_kernel(
         const uint16_t* __restrict__ qa, const uint16_t* __restrict__ cache, const int32_t* __restrict__ block_table,
         int max_blocks, const int32_t* __restrict__ q_start, const int32_t* __restrict__ pos,
         const float* __restrict__ gate, uint16_t* __restrict__ out, int H, int DK, int rank, int BS, float scale,
-        int window, int nsplit, float* __restrict__ part_o, float* __restrict__ part_ml, int bs_shift) {
+        int window, int nsplit, float* __restrict__ part_o, float* __restrict__ part_ml, int bs_shift,
+        const float* __restrict__ sink) {
     extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
     const int b = blockIdx.x;
     const int t0 = q_start[b], t1 = q_start[b + 1];
@@ -208,6 +210,10 @@ __global__ void __launch_bounds__(64 * NW) latent_attention_mfma_kernel(
         return;
     }
     float f = 1.f / lrow;
+    if (sink != nullptr) {   // exp(sink) joins the denominator, without a value
+        const float sk = sink[rc % H], mn = fmaxf(mrow, sk), c = __expf(mrow - mn);
+        f = c / (lrow * c + __expf(sk - mn));
+    }
     if (gate != nullptr) f *= sigmoidf_(gate[grow]);
     // lane holds O^T[col = 16 c + 4 g + i][query row qi]
 #pragma unroll
@@ -218,20 +224,22 @@ __global__ void __launch_bounds__(64 * NW) latent_attention_mfma_kernel(
         }
 }
 
-// one wave per (token, head) row: out = sum_z exp(m_z - m) O_z / sum_z exp(m_z - m) l_z * sigmoid(gate).  Lane z holds
+// one wave per (token, head) row: out = sum_z exp(m_z - m) O_z / (sum_z exp(m_z - m) l_z + exp(sink - m)) * sigmoid(gate).  Lane z holds
 // split z's maximum and sum (nsplit <= 16); a lane then sums 4 neighbouring columns over the splits, whose loads do not
 // depend on each other.
 __global__ void __launch_bounds__(256) latent_combine_kernel(const float* __restrict__ part_o, const float* __restrict__ part_ml,
                                                              const float* __restrict__ gate, uint16_t* __restrict__ out,
-                                                             int64_t rows, int rank, int nsplit) {
+                                                             int64_t rows, int rank, int nsplit,
+                                                             const float* __restrict__ sink, int H) {
     const int lane = threadIdx.x & 63;
     const int64_t r = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
     if (r >= rows) return;
     const float mz = lane < nsplit ? part_ml[(r * nsplit + lane) * 2] : -INFINITY;
     const float lz = lane < nsplit ? part_ml[(r * nsplit + lane) * 2 + 1] : 0.f;
-    const float m = wave_max(mz);
+    const float sk = sink != nullptr ? sink[r % H] : -INFINITY;
+    const float m = fmaxf(wave_max(mz), sk);
     float e = mz == -INFINITY ? 0.f : expf(mz - m);   // (a split without a visible key adds nothing)
-    const float l = wave_sum(e * lz);
+    const float l = wave_sum(e * lz) + (sink != nullptr ? expf(sk - m) : 0.f);
     e *= (gate != nullptr ? sigmoidf_(gate[r]) : 1.f) / l;
     for (int c = lane * 4; c < rank; c += 256) {      // (rank is a multiple of 16)
         f32x4 acc = {0.f, 0.f, 0.f, 0.f};
@@ -250,7 +258,7 @@ template <int NS, int NCT, int KT, int NW, bool TT>
 static void la_mfma_launch(const uint16_t* qa, const uint16_t* cache, const int32_t* bt, int max_blocks,
                            const int32_t* q_start, const int32_t* pos, const float* gate, uint16_t* out, int B, int H,
                            int DK, int rank, int BS, int max_q, float scale, int window, int nsplit, float* part_o,
-                           float* part_ml, hipStream_t s) {
+                           float* part_ml, const float* sink, hipStream_t s) {
     auto kern = hy::latent_attention_mfma_kernel<NS, NCT, KT, NW, TT>;
     const int bytes = KT * ((DK + 31) / 32 * 64 + 16) + rank * (KT * 2 + 8);
     static int set_bytes = 0;
@@ -261,7 +269,7 @@ static void la_mfma_launch(const uint16_t* qa, const uint16_t* cache, const int3
     const dim3 grid(B, (max_q * H + 16 * NW - 1) / (16 * NW), nsplit);
     const int bs_shift = (BS & (BS - 1)) == 0 ? __builtin_ctz(BS) : -1;
     kern<<<grid, 64 * NW, bytes, s>>>(qa, cache, bt, max_blocks, q_start, pos, gate, out, H, DK, rank, BS, scale, window,
-                                  nsplit, part_o, part_ml, bs_shift);
+                                  nsplit, part_o, part_ml, bs_shift, sink);
 }
 
 bool hy_latent_mfma_ok(int DK, int rank) { return !(DK % 8 || rank % 16 || DK > 576 || rank > 512 || rank > DK); }
@@ -282,10 +290,11 @@ int hy_latent_nsplit(int wgs, int max_ctx, bool windowed) {
 bool launch_hy_latent_attention_mfma(const uint16_t* qa, const uint16_t* cache, const int32_t* bt, int max_blocks,
                                      const int32_t* q_start, const int32_t* pos, const float* gate, uint16_t* out, int B,
                                      int H, int DK, int rank, int BS, int max_q, float scale, int window, bool two_term,
-                                     int nsplit, float* part_o, float* part_ml, int64_t total_rows, hipStream_t s) {
+                                     int nsplit, float* part_o, float* part_ml, int64_t total_rows, const float* sink,
+                                     hipStream_t s) {
     if (!hy_latent_mfma_ok(DK, rank)) return false;
     if (B == 0 || max_q == 0) return true;
-#define HY_LAM(NS, NCT, KT, NW, TT) la_mfma_launch<NS, NCT, KT, NW, TT>(qa, cache, bt, max_blocks, q_start, pos, gate, out, B, H, DK, rank, BS, max_q, scale, window, nsplit, part_o, part_ml, s)
+#define HY_LAM(NS, NCT, KT, NW, TT) la_mfma_launch<NS, NCT, KT, NW, TT>(qa, cache, bt, max_blocks, q_start, pos, gate, out, B, H, DK, rank, BS, max_q, scale, window, nsplit, part_o, part_ml, sink, s)
     // 64-key tiles (32-key tiles measured slower at every size: the per-tile softmax and barriers weigh more than the
     // second workgroup per CU gains; CHRONOS_LATENT_KT=32 keeps them for A/B).  8 waves per workgroup when a sequence
     // brings more than 64 rows (CHRONOS_LATENT_NW=4 / 8 forces one).
@@ -305,7 +314,7 @@ bool launch_hy_latent_attention_mfma(const uint16_t* qa, const uint16_t* cache, 
 #undef HY_LAM_T
 #undef HY_LAM
     if (nsplit > 1)
-        hy::latent_combine_kernel<<<(unsigned)((total_rows + 3) / 4), 256, 0, s>>>(part_o, part_ml, gate, out, total_rows, rank, nsplit);
+        hy::latent_combine_kernel<<<(unsigned)((total_rows + 3) / 4), 256, 0, s>>>(part_o, part_ml, gate, out, total_rows, rank, nsplit, sink, H);
     return true;
 }
 

@@ -358,18 +358,24 @@ __global__ void __launch_bounds__(256) linear_scan_kernel(
 }  // namespace hy
 
 // x points at the first convolved column of the first row (rows ldx apart); bias may be nullptr
+void launch_hy_conv_hist(const void* x, int ldx, const int32_t* q_start, const int32_t* pos0, const int32_t* slots,
+                         void* hist, int B, int C, int K, bool f32, hipStream_t s) {
+    if (B == 0 || C == 0 || K <= 1) return;
+    const dim3 hg(B, (C + 255) / 256);
+    if (f32) hy::conv_hist_kernel<float><<<hg, 256, 0, s>>>((const float*)x, ldx, q_start, pos0, slots, (float*)hist, C, K);
+    else hy::conv_hist_kernel<uint16_t><<<hg, 256, 0, s>>>((const uint16_t*)x, ldx, q_start, pos0, slots, (uint16_t*)hist, C, K);
+}
+
 void launch_hy_short_conv(const void* x, int ldx, const float* w, const float* bias, const int32_t* tok_seq,
                           const int32_t* q_start, const int32_t* pos0, const int32_t* slots, void* hist, void* y, int T,
                           int B, int C, int K, bool silu, bool f32, hipStream_t s) {
     if (T == 0 || C == 0) return;
-    const dim3 hg(B, (C + 255) / 256);
     if (f32) {
         hy::short_conv_kernel<float><<<T, 256, 0, s>>>((const float*)x, ldx, w, tok_seq, q_start, pos0, slots, (const float*)hist, (float*)y, C, K, silu, bias);
-        if (K > 1) hy::conv_hist_kernel<float><<<hg, 256, 0, s>>>((const float*)x, ldx, q_start, pos0, slots, (float*)hist, C, K);
     } else {
         hy::short_conv_kernel<uint16_t><<<T, 256, 0, s>>>((const uint16_t*)x, ldx, w, tok_seq, q_start, pos0, slots, (const uint16_t*)hist, (uint16_t*)y, C, K, silu, bias);
-        if (K > 1) hy::conv_hist_kernel<uint16_t><<<hg, 256, 0, s>>>((const uint16_t*)x, ldx, q_start, pos0, slots, (uint16_t*)hist, C, K);
     }
+    launch_hy_conv_hist(x, ldx, q_start, pos0, slots, hist, B, C, K, f32, s);
 }
 
 void launch_hy_delta_prep(const void* y, int ldy, const float* ab, const float* a_log, float* qscale, float* kscale,

@@ -91,16 +91,15 @@ __global__ void __launch_bounds__(256) rms_norm_kernel(const TY* __restrict__ y,
     }
 }
 
+// grid (rows, column blocks); rows of gu (gate columns, then up columns) and of y may be parts of wider ones
 template <typename T, bool VEC>
-__global__ void __launch_bounds__(256) glu_kernel(const T* __restrict__ gu, T* __restrict__ y, int64_t rows, int F,
+__global__ void __launch_bounds__(256) glu_kernel(const T* __restrict__ gu, int64_t ldg, T* __restrict__ y, int64_t ldy, int F,
                                                   float limit, float slope, float shift) {
     constexpr int E = VEC ? 4 : 1;
-    const int64_t per = F / E;
-    const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
-    if (i >= rows * per) return;
-    const int64_t r = i / per;
-    const int c = (int)(i % per) * E;
-    const T* g = gu + r * 2 * F + c;
+    const int64_t r = blockIdx.x;
+    const int c = (int)(blockIdx.y * blockDim.x + threadIdx.x) * E;
+    if (c >= F) return;
+    const T* g = gu + r * ldg + c;
     if constexpr (VEC) {
         const f32x4 gv = ld4<T>(g), uv = ld4<T>(g + F);
         f32x4 o;
@@ -109,10 +108,10 @@ __global__ void __launch_bounds__(256) glu_kernel(const T* __restrict__ gu, T* _
             const float a = fminf(gv[k], limit), u = fminf(fmaxf(uv[k], -limit), limit);
             o[k] = a * sigmoidf_(slope * a) * (u + shift);
         }
-        st4<T>(y + r * F + c, o);
+        st4<T>(y + r * ldy + c, o);
     } else {
         const float a = fminf(ld<T>(g), limit), u = fminf(fmaxf(ld<T>(g + F), -limit), limit);
-        st<T>(y + r * F + c, a * sigmoidf_(slope * a) * (u + shift));
+        st<T>(y + r * ldy + c, a * sigmoidf_(slope * a) * (u + shift));
     }
 }
 
@@ -144,19 +143,18 @@ void launch_hy_rms_norm(const void* y, float* x, const float* w, void* h, bool o
 #undef HY_RN
 }
 
-void launch_hy_glu(const void* gu, void* y, int64_t rows, int F, float limit, float slope, float shift, bool f32,
-                   hipStream_t s) {
+// ldg, ldy: row strides of gu and y
+void launch_hy_glu(const void* gu, int64_t ldg, void* y, int64_t ldy, int64_t rows, int F, float limit, float slope,
+                   float shift, bool f32, hipStream_t s) {
     if (rows == 0 || F == 0) return;
-    const bool vec = F % 4 == 0;
-    const int64_t n = rows * (vec ? F / 4 : F);
-    const unsigned blocks = (unsigned)((n + 255) / 256);
-    if (f32) {
-        if (vec) hy::glu_kernel<float, true><<<blocks, 256, 0, s>>>((const float*)gu, (float*)y, rows, F, limit, slope, shift);
-        else hy::glu_kernel<float, false><<<blocks, 256, 0, s>>>((const float*)gu, (float*)y, rows, F, limit, slope, shift);
-    } else {
-        if (vec) hy::glu_kernel<uint16_t, true><<<blocks, 256, 0, s>>>((const uint16_t*)gu, (uint16_t*)y, rows, F, limit, slope, shift);
-        else hy::glu_kernel<uint16_t, false><<<blocks, 256, 0, s>>>((const uint16_t*)gu, (uint16_t*)y, rows, F, limit, slope, shift);
-    }
+    auto al = [&](const void* p) { return reinterpret_cast<uintptr_t>(p) % (f32 ? 16 : 8) == 0; };
+    const bool vec = F % 4 == 0 && ldg % 4 == 0 && ldy % 4 == 0 && al(gu) && al(y);
+    const int per = vec ? F / 4 : F, nt = per < 256 ? (per + 63) / 64 * 64 : 256;
+    const dim3 grid((unsigned)rows, (per + nt - 1) / nt);
+#define HY_GLU(T, VEC) hy::glu_kernel<T, VEC><<<grid, nt, 0, s>>>((const T*)gu, ldg, (T*)y, ldy, F, limit, slope, shift)
+    if (f32) { if (vec) HY_GLU(float, true); else HY_GLU(float, false); }
+    else { if (vec) HY_GLU(uint16_t, true); else HY_GLU(uint16_t, false); }
+#undef HY_GLU
 }
 
 void launch_hy_decay_pow(float* z, int64_t n, float p, hipStream_t s) {

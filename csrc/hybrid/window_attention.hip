@@ -7,7 +7,9 @@
 //                     (1 - lam) v + lam v_first, optionally rotated by the token's position over all Dv columns;
 //                     keys and values written to the token's page and slot of kc [NB, BS, G, D] / vc [NB, BS, G, Dv].
 //                     The values are read from column v_off of the projection's row (the column after the keys, or
-//                     for instance the keys' own columns: values = keys as projected).
+//                     for instance the keys' own columns: values = keys before norm and rotation).  Queries may be
+//                     multiplied by a factor from a table by position.  With unit keys (ks given, no kc) a key is the
+//                     cached value divided by its root mean square: only that factor is written, to ks [NB, BS, G].
 //   pool_blocks       per sequence and block of `pool` positions whose last position is among the step's tokens: the
 //                     float means of the block's cached keys and values, written to kp / vp [NB, EP, G, .] (block e
 //                     in row e % EP of the sequence's page e / EP, EP = ceil(BS / pool)).
@@ -26,6 +28,8 @@
 //                     With pool > 0 (and a window) the walk begins with tiles of POOLED pairs: the row at position i
 //                     sees block e when e pool + pool - 1 <= i - window, so a token that has left the window is seen
 //                     again only once its whole block has; tokens and blocks share the one softmax.
+//                     With unit keys the one cached row is staged once, a score is the query's product with the
+//                     value times the key's factor.
 //                     After the last key the sink joins the denominator: l += exp(sink_h - m) (no value), and the
 //                     row is multiplied by sigmoid(gate) when a gate is given.
 // Prompt portions, decode rows and mixed steps are one code path (a decode row is a tile of one token).
@@ -43,7 +47,8 @@ __global__ void __launch_bounds__(256) window_prep_kernel(
         const float* __restrict__ lam, const int32_t* __restrict__ pos, const int32_t* __restrict__ tok_seq,
         const int32_t* __restrict__ block_table, int max_blocks, const float* __restrict__ q_norm,
         const float* __restrict__ k_norm, float eps, const float* __restrict__ cos_sin, int dims, T* __restrict__ kc,
-        T* __restrict__ vc, int BS, T* __restrict__ v_out, int v_off, const float* __restrict__ v_cos_sin) {
+        T* __restrict__ vc, int BS, T* __restrict__ v_out, int v_off, const float* __restrict__ v_cos_sin,
+        const float* __restrict__ q_temp, float* __restrict__ ks) {
     extern __shared__ float wp_smem[];
     const int64_t t = blockIdx.x;
     const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6;
@@ -56,23 +61,29 @@ __global__ void __launch_bounds__(256) window_prep_kernel(
     for (int j = wv; j < H + G; j += 4) {  // heads 0..H-1: queries (in place); H..H+G-1: keys (to the cache)
         const T* src = base + (int64_t)j * D;
         const float* nw = j < H ? q_norm : k_norm;
-        if (nw == nullptr && dims == 0 && j < H) continue;  // plain queries stay as the projection wrote them
+        const bool unit = ks != nullptr;
+        if (nw == nullptr && dims == 0 && j < H && q_temp == nullptr && !unit) continue;  // plain queries stay as they are
         float ss = 0.f;
         for (int i = lane; i < D; i += 64) {
             const float v = ld<T>(src + i);
             row[i] = v;
             ss += v * v;
         }
-        const float inv = nw != nullptr ? 1.f / sqrtf(wave_sum(ss) / (float)D + eps) : 1.f;
+        const float inv = nw != nullptr || unit ? 1.f / sqrtf(wave_sum(ss) / (float)D + eps) : 1.f;
+        if (unit && j >= H) {
+            if (lane == 0) ks[slot * G + (j - H)] = inv;
+            continue;
+        }
+        const float temp = q_temp != nullptr && j < H ? q_temp[p] : 1.f;
         T* dst = j < H ? base + (int64_t)j * D : kc + (slot * G + (j - H)) * D;
         // (wave-private LDS row: the wave's own writes above are visible to its reads below without a barrier,
         // the compiler orders LDS accesses of one wave)
         for (int i = lane; i < D; i += 64) {
-            auto nrm = [&](int c) { return nw != nullptr ? row[c] * inv * nw[c] : row[c]; };
+            auto nrm = [&](int c) { return nw != nullptr ? row[c] * inv * nw[c] : row[c] * inv; };
             float v = nrm(i);
             if (i < half) v = v * cs[i] - nrm(i + half) * cs[half + i];
             else if (i < dims) v = v * cs[i - half] + nrm(i - half) * cs[i];
-            st<T>(dst + i, v);
+            st<T>(dst + i, v * temp);
         }
     }
     const float l = v_first != nullptr ? lam[0] : 0.f;
@@ -201,7 +212,8 @@ __global__ void __launch_bounds__(256) window_attention_kernel(
         const int32_t* __restrict__ block_table, int max_blocks, const int32_t* __restrict__ q_start,
         const int32_t* __restrict__ pos, const float* __restrict__ sink, const float* __restrict__ gate,
         T* __restrict__ out, int H, int G, int D, int Dv, int BS, float scale, int window, int keep, int chunk, int QT,
-        int rows_cap, int pool, int EP, const T* __restrict__ kp, const T* __restrict__ vp) {
+        int rows_cap, int pool, int EP, const T* __restrict__ kp, const T* __restrict__ vp, const float* __restrict__ ks,
+        int64_t ldo) {
     extern __shared__ __attribute__((aligned(16))) unsigned char wa_smem[];
     constexpr int PAD = WaPad<T>::V;
     const int R = H / G;
@@ -212,7 +224,7 @@ __global__ void __launch_bounds__(256) window_attention_kernel(
     const int nq = t1 - t0, rows = nq * R;
     const int ldk = D + PAD, ldv = Dv + PAD;
     T* Ks = reinterpret_cast<T*>(wa_smem);
-    T* Vs = Ks + kWaKT * ldk;
+    T* Vs = ks != nullptr ? Ks : Ks + kWaKT * ldk;   // unit keys: one row is key and value
     float* Qs = reinterpret_cast<float*>(wa_smem + (((size_t)kWaKT * (ldk + ldv) * sizeof(T) + 15) & ~(size_t)15));
     float* Ps = Qs + (size_t)rows_cap * D;
     const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6;
@@ -266,7 +278,7 @@ __global__ void __launch_bounds__(256) window_attention_kernel(
             if (j < j_end) v = ksrc[(((int64_t)block_table[(int64_t)b * max_blocks + j / per] * per + j % per) * G + g) * D + d];
             Ks[kk * ldk + d] = v;
         }
-        for (int i = threadIdx.x; i < kWaKT * Dv; i += 256) {
+        for (int i = threadIdx.x; i < (ks != nullptr ? 0 : kWaKT * Dv); i += 256) {
             const int kk = i / Dv, d = i % Dv, j = j0 + kk;
             T v;
             st<T>(&v, 0.f);
@@ -275,6 +287,9 @@ __global__ void __launch_bounds__(256) window_attention_kernel(
         }
         __syncthreads();
         const int j = j0 + lane;
+        // (pooled tiles never come with unit keys)
+        const float kf = ks == nullptr ? scale : j < j_end
+            ? scale * ks[((int64_t)block_table[(int64_t)b * max_blocks + j / BS] * BS + j % BS) * G + g] : 0.f;
 #pragma unroll
         for (int q = 0; q < MAXG; ++q) {
             if (q >= my_groups) break;
@@ -293,7 +308,7 @@ __global__ void __launch_bounds__(256) window_attention_kernel(
                 const bool vis = pooled ? (j < j_end && (j + 1) * pool - 1 + window <= pi)
                                         : (j < j_end && j <= pi && (window <= 0 || pi - j < window || j < keep) &&
                                            (chunk <= 0 || j >= pi / chunk * chunk));
-                const float sv = vis ? s[r] * scale : -INFINITY;
+                const float sv = vis ? s[r] * kf : -INFINITY;
                 const float mn = fmaxf(m_[q][r], wave_max(sv));
                 const float pw = mn == -INFINITY ? 0.f : expf(sv - mn);
                 const float corr = m_[q][r] == -INFINITY ? 0.f : expf(m_[q][r] - mn);
@@ -343,7 +358,7 @@ __global__ void __launch_bounds__(256) window_attention_kernel(
 #pragma unroll
             for (int c = 0; c < 4; ++c) {
                 const int col = c * 64 + lane;
-                if (c < NC && col < Dv) st<T>(out + (t * H + hd) * Dv + col, o_[q][r][c] * f);
+                if (c < NC && col < Dv) st<T>(out + t * ldo + hd * Dv + col, o_[q][r][c] * f);
             }
         }
     }
@@ -354,13 +369,13 @@ __global__ void __launch_bounds__(256) window_attention_kernel(
 void launch_hy_window_prep(void* qkv, int ld, int H, int G, int D, int Dv, const void* v_first, const float* lam,
                            const int32_t* pos, const int32_t* tok_seq, const int32_t* block_table, int max_blocks,
                            const float* q_norm, const float* k_norm, float eps, const float* cos_sin, int dims, void* kc,
-                           void* vc, int BS, void* v_out, int v_off, const float* v_cos_sin, int T, bool f32,
-                           hipStream_t s) {
+                           void* vc, int BS, void* v_out, int v_off, const float* v_cos_sin, const float* q_temp,
+                           float* ks, int T, bool f32, hipStream_t s) {
     if (T == 0) return;
     const int bytes = 4 * D * 4;
     if (v_off < 0) v_off = (H + G) * D;
-    if (f32) hy::window_prep_kernel<float><<<T, 256, bytes, s>>>((float*)qkv, ld, H, G, D, Dv, (const float*)v_first, lam, pos, tok_seq, block_table, max_blocks, q_norm, k_norm, eps, cos_sin, dims, (float*)kc, (float*)vc, BS, (float*)v_out, v_off, v_cos_sin);
-    else hy::window_prep_kernel<uint16_t><<<T, 256, bytes, s>>>((uint16_t*)qkv, ld, H, G, D, Dv, (const uint16_t*)v_first, lam, pos, tok_seq, block_table, max_blocks, q_norm, k_norm, eps, cos_sin, dims, (uint16_t*)kc, (uint16_t*)vc, BS, (uint16_t*)v_out, v_off, v_cos_sin);
+    if (f32) hy::window_prep_kernel<float><<<T, 256, bytes, s>>>((float*)qkv, ld, H, G, D, Dv, (const float*)v_first, lam, pos, tok_seq, block_table, max_blocks, q_norm, k_norm, eps, cos_sin, dims, (float*)kc, (float*)vc, BS, (float*)v_out, v_off, v_cos_sin, q_temp, ks);
+    else hy::window_prep_kernel<uint16_t><<<T, 256, bytes, s>>>((uint16_t*)qkv, ld, H, G, D, Dv, (const uint16_t*)v_first, lam, pos, tok_seq, block_table, max_blocks, q_norm, k_norm, eps, cos_sin, dims, (uint16_t*)kc, (uint16_t*)vc, BS, (uint16_t*)v_out, v_off, v_cos_sin, q_temp, ks);
 }
 
 // max_q: the most tokens a sequence brings in this step; a sequence completes at most max_q / pool + 1 blocks
@@ -398,7 +413,8 @@ int hy_window_rows_cap(int R, int D, int Dv, bool f32) {
 bool launch_hy_window_attention_mfma(const uint16_t*, int, const uint16_t*, const uint16_t*, const int32_t*, int,
                                      const int32_t*, const int32_t*, const float*, const float*, uint16_t*, int, int, int,
                                      int, int, int, int, float, int, int, int, int, float*, float*, int64_t, int, int,
-                                     const uint16_t*, const uint16_t*, const float*, int, hipStream_t);
+                                     const uint16_t*, const uint16_t*, const float*, int, const float*, int64_t,
+                                     hipStream_t);
 void launch_hy_unrotate_gate(const void*, const int32_t*, const float*, const void*, int, int, void*, int, int, int, bool,
                              hipStream_t);
 
@@ -406,12 +422,14 @@ void launch_hy_unrotate_gate(const void*, const int32_t*, const float*, const vo
 // vcs (may be nullptr): a rotation table [P, Dv] by which every head's output is turned back at the query's position;
 // g_off >= 0: the output is multiplied by sigmoid of the columns g_off .. g_off + H Dv of the query's row of qkv.
 // The matrix-core kernel does both in its epilogue (Dv % 32 == 0); otherwise a pass over the output follows.
+// ks (unit keys; kc is then not read): the keys' factors.  ldo: row stride of out (H Dv with vcs or g_off).
 void launch_hy_window_attention(const void* qkv, int ld, const void* kc, const void* vc, const int32_t* block_table,
                                 int max_blocks, const int32_t* q_start, const int32_t* pos, const float* sink,
                                 const float* gate, void* out, int B, int max_q, int H, int G, int D, int Dv, int BS,
                                 float scale, int window, int keep, int chunk, bool f32, int nsplit, float* part_o,
                                 float* part_ml, int64_t total_rows, int pool, int EP, const void* kp, const void* vp,
-                                const float* vcs, int g_off, hipStream_t s) {
+                                const float* vcs, int g_off, const float* ks, int64_t ldo, hipStream_t s) {
+    if (ks != nullptr) kc = vc;
     if (B == 0 || max_q == 0) return;
     const bool post = vcs != nullptr || g_off >= 0;
     const bool fused = post && (vcs == nullptr || Dv % 32 == 0);   // the matrix-core epilogue can do it
@@ -420,7 +438,7 @@ void launch_hy_window_attention(const void* qkv, int ld, const void* kc, const v
                                                 block_table, max_blocks, q_start, pos, sink, gate, (uint16_t*)out, B,
                                                 max_q, H, G, D, Dv, BS, scale, window, keep, chunk, nsplit, part_o,
                                                 part_ml, total_rows, pool, EP, (const uint16_t*)kp,
-                                                (const uint16_t*)vp, fused ? vcs : nullptr, fused ? g_off : -1, s)) {
+                                                (const uint16_t*)vp, fused ? vcs : nullptr, fused ? g_off : -1, ks, ldo, s)) {
         if (post && !fused) launch_hy_unrotate_gate(out, pos, vcs, g_off >= 0 ? qkv : nullptr, ld, g_off, out, T, H, Dv, false, s);
         return;
     }
@@ -432,11 +450,11 @@ void launch_hy_window_attention(const void* qkv, int ld, const void* kc, const v
     if (f32) {
         auto kern = hy::window_attention_kernel<float>;
         (void)hipFuncSetAttribute(reinterpret_cast<const void*>(kern), hipFuncAttributeMaxDynamicSharedMemorySize, bytes);
-        kern<<<grid, 256, bytes, s>>>((const float*)qkv, ld, (const float*)kc, (const float*)vc, block_table, max_blocks, q_start, pos, sink, gate, (float*)out, H, G, D, Dv, BS, scale, window, keep, chunk, QT, rows_cap, pool, EP, (const float*)kp, (const float*)vp);
+        kern<<<grid, 256, bytes, s>>>((const float*)qkv, ld, (const float*)kc, (const float*)vc, block_table, max_blocks, q_start, pos, sink, gate, (float*)out, H, G, D, Dv, BS, scale, window, keep, chunk, QT, rows_cap, pool, EP, (const float*)kp, (const float*)vp, ks, ldo);
     } else {
         auto kern = hy::window_attention_kernel<uint16_t>;
         (void)hipFuncSetAttribute(reinterpret_cast<const void*>(kern), hipFuncAttributeMaxDynamicSharedMemorySize, bytes);
-        kern<<<grid, 256, bytes, s>>>((const uint16_t*)qkv, ld, (const uint16_t*)kc, (const uint16_t*)vc, block_table, max_blocks, q_start, pos, sink, gate, (uint16_t*)out, H, G, D, Dv, BS, scale, window, keep, chunk, QT, rows_cap, pool, EP, (const uint16_t*)kp, (const uint16_t*)vp);
+        kern<<<grid, 256, bytes, s>>>((const uint16_t*)qkv, ld, (const uint16_t*)kc, (const uint16_t*)vc, block_table, max_blocks, q_start, pos, sink, gate, (uint16_t*)out, H, G, D, Dv, BS, scale, window, keep, chunk, QT, rows_cap, pool, EP, (const uint16_t*)kp, (const uint16_t*)vp, ks, ldo);
     }
     if (post) launch_hy_unrotate_gate(out, pos, vcs, g_off >= 0 ? qkv : nullptr, ld, g_off, out, T, H, Dv, f32, s);
 }

@@ -22,6 +22,8 @@
 // c + Dv / 32), and with a gate per output column the row is multiplied by sigmoid of the gate columns of the
 // query's own projection row.  Launches of few
 // rows (decode) deal a row block's key tiles to several workgroups and merge the float partials in a second kernel.
+// With unit keys (SH: a key is the cached value times a float factor) a row is loaded once and written to both images,
+// and a score is multiplied by its key's factor.
 // With chunk > 0 a row also hides the keys below its own chunk of positions (key >= floor(pos / chunk) * chunk).
 // Sizes: D % 32 == 0, Dv % 16 == 0, D <= 256, Dv <= 256.  Everything else takes the general kernel.
 #include <algorithm>
@@ -33,14 +35,15 @@ namespace hy {
 
 constexpr int WKT = 64;  // keys per tile
 
-template <int NS, int NCT, int NW>
+template <int NS, int NCT, int NW, bool SH>
 __global__ void __launch_bounds__(64 * NW) window_attention_mfma_kernel(
         const uint16_t* __restrict__ qkv, int ldq, const uint16_t* __restrict__ kc, const uint16_t* __restrict__ vc,
         const int32_t* __restrict__ block_table, int max_blocks, const int32_t* __restrict__ q_start,
         const int32_t* __restrict__ pos, const float* __restrict__ sink, const float* __restrict__ gate,
         uint16_t* __restrict__ out, int H, int G, int D, int Dv, int BS, float scale, int window, int keep, int chunk,
         int nsplit, float* __restrict__ part_o, float* __restrict__ part_ml, int pool, int EP,
-        const uint16_t* __restrict__ kp, const uint16_t* __restrict__ vp, const float* __restrict__ vcs, int g_off) {
+        const uint16_t* __restrict__ kp, const uint16_t* __restrict__ vp, const float* __restrict__ vcs, int g_off,
+        const float* __restrict__ ks, int64_t ldo) {
     extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
     constexpr int KT = WKT, NT = 64 * NW, RPB = 16 * NW, PP = KT / 2;
     const int R = H / G;
@@ -55,6 +58,7 @@ __global__ void __launch_bounds__(64 * NW) window_attention_mfma_kernel(
     const int krs = D * 2 + 16;          // row-major key image: bytes per key row
     constexpr int vts = KT * 2 + 8;      // transposed value image: bytes per value column
     __shared__ int krow[KT];             // cache row (page * page size + slot) of each key of the tile
+    __shared__ __attribute__((aligned(16))) float kfac[SH ? KT : 4];   // its factor
     unsigned char* kimg = smem;
     unsigned char* vimg = smem + KT * krs;
     const int r = rb0 + wv * 16 + qi;
@@ -102,9 +106,37 @@ __global__ void __launch_bounds__(64 * NW) window_attention_mfma_kernel(
             const int key = min(k0 + (int)threadIdx.x, k_last);  // past the end: a real row, masked below
             const int per = pooled ? EP : BS;
             krow[threadIdx.x] = (bt[key / per] * per + key % per) * G + kvh;
+            if constexpr (SH) kfac[threadIdx.x] = ks[krow[threadIdx.x]];
         }
         __syncthreads();
         // ---- stage: work item = (key pair jp, 8-element chunk dc); lanes of a wave take consecutive key pairs
+        if constexpr (SH) {
+            for (int it0 = threadIdx.x; it0 < PP * kchunks; it0 += NT * 2) {
+                u16x8 va[2], vb[2];
+#pragma unroll
+                for (int u = 0; u < 2; ++u) {
+                    const int it = it0 + NT * u;
+                    if (it < PP * kchunks) {
+                        const int jp = it & (PP - 1), dc = it / PP;
+                        va[u] = *reinterpret_cast<const u16x8*>(vc + (int64_t)krow[2 * jp] * D + dc * 8);
+                        vb[u] = *reinterpret_cast<const u16x8*>(vc + (int64_t)krow[2 * jp + 1] * D + dc * 8);
+                    }
+                }
+#pragma unroll
+                for (int u = 0; u < 2; ++u) {
+                    const int it = it0 + NT * u;
+                    if (it < PP * kchunks) {
+                        const int jp = it & (PP - 1), dc = it / PP;
+                        *reinterpret_cast<u16x8*>(kimg + (2 * jp) * krs + dc * 16) = va[u];
+                        *reinterpret_cast<u16x8*>(kimg + (2 * jp + 1) * krs + dc * 16) = vb[u];
+#pragma unroll
+                        for (int e = 0; e < 8; ++e)
+                            *reinterpret_cast<uint32_t*>(vimg + (dc * 8 + e) * vts + jp * 4) =
+                                (uint32_t)va[u][e] | ((uint32_t)vb[u][e] << 16);
+                    }
+                }
+            }
+        } else {
         for (int it = threadIdx.x; it < PP * kchunks; it += NT) {
             const int jp = it & (PP - 1), dc = it / PP;
             const u16x8 va = *reinterpret_cast<const u16x8*>(ksrc + (int64_t)krow[2 * jp] * D + dc * 8);
@@ -120,6 +152,7 @@ __global__ void __launch_bounds__(64 * NW) window_attention_mfma_kernel(
             for (int e = 0; e < 8; ++e)
                 *reinterpret_cast<uint32_t*>(vimg + (dc * 8 + e) * vts + jp * 4) = (uint32_t)va[e] | ((uint32_t)vb[e] << 16);
         }
+        }
         __syncthreads();
         // ---- scores: 4 key tiles of 16; lane gets keys 16 kt + 4 g4 + i of query row qi
         constexpr int NKT = KT / 16;
@@ -133,6 +166,7 @@ __global__ void __launch_bounds__(64 * NW) window_attention_mfma_kernel(
                 if (s < ns)
                     S[kt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8*>(arow + s * 64), qf[s],
                                                                     S[kt], 0, 0, 0);
+            if constexpr (SH) S[kt] *= *reinterpret_cast<const f32x4*>(kfac + 16 * kt + 4 * g4);
         }
         // scores, maxima and sums live in the base-2 domain (score * scale * log2 e): one multiply and one
         // subtraction in front of the hardware's exp2.  A tile that every row of the block sees whole (the common case
@@ -241,7 +275,7 @@ __global__ void __launch_bounds__(64 * NW) window_attention_mfma_kernel(
 #pragma unroll
             for (int i = 0; i < 4; ++i) v[i] *= sigmoidf_(bf2f(gv[i]));
         }
-        *reinterpret_cast<u16x4*>(out + (tok * H + head) * Dv + 16 * c + 4 * g4) =
+        *reinterpret_cast<u16x4*>(out + tok * ldo + head * Dv + 16 * c + 4 * g4) =
             u16x4{f2bf(v[0]), f2bf(v[1]), f2bf(v[2]), f2bf(v[3])};
     };
     if (vcs == nullptr) {
@@ -274,7 +308,7 @@ __global__ void __launch_bounds__(256) window_combine_kernel(const float* __rest
                                                              uint16_t* __restrict__ out, int64_t rows, int H, int Dv,
                                                              int nsplit, const float* __restrict__ vcs,
                                                              const int32_t* __restrict__ pos, const uint16_t* __restrict__ qkv,
-                                                             int ldq, int g_off) {
+                                                             int ldq, int g_off, int64_t ldo) {
     const int lane = threadIdx.x & 63;
     const int64_t r = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
     if (r >= rows) return;
@@ -298,30 +332,31 @@ __global__ void __launch_bounds__(256) window_combine_kernel(const float* __rest
         return acc * f;
     };
     const uint16_t* gsrc = g_off >= 0 ? qkv + (r / H) * ldq + g_off + (r % H) * Dv : nullptr;
+    uint16_t* orow = out + (r / H) * ldo + (r % H) * Dv;
     auto wide = [&](int c) { return gsrc != nullptr ? sigmoidf_(bf2f(gsrc[c])) : 1.f; };
     if (vcs == nullptr) {
-        for (int c = lane; c < Dv; c += 64) out[r * Dv + c] = f2bf(col(c) * wide(c));
+        for (int c = lane; c < Dv; c += 64) orow[c] = f2bf(col(c) * wide(c));
         return;
     }
     const int half = Dv / 2;
     const float* cs = vcs + (int64_t)pos[r / H] * Dv;
     for (int c = lane; c < half; c += 64) {
         const float a = col(c), b = col(c + half), co = cs[c], si = cs[half + c];
-        out[r * Dv + c] = f2bf((a * co + b * si) * wide(c));
-        out[r * Dv + c + half] = f2bf((b * co - a * si) * wide(c + half));
+        orow[c] = f2bf((a * co + b * si) * wide(c));
+        orow[c + half] = f2bf((b * co - a * si) * wide(c + half));
     }
 }
 
 }  // namespace hy
 
-template <int NS, int NCT, int NW>
+template <int NS, int NCT, int NW, bool SH>
 static void wa_mfma_launch(const uint16_t* qkv, int ldq, const uint16_t* kc, const uint16_t* vc, const int32_t* bt,
                            int max_blocks, const int32_t* q_start, const int32_t* pos, const float* sink,
                            const float* gate, uint16_t* out, int B, int max_q, int H, int G, int D, int Dv, int BS,
                            float scale, int window, int keep, int chunk, int nsplit, float* part_o, float* part_ml,
                            int pool, int EP, const uint16_t* kp, const uint16_t* vp, const float* vcs, int g_off,
-                           hipStream_t s) {
-    auto kern = hy::window_attention_mfma_kernel<NS, NCT, NW>;
+                           const float* ks, int64_t ldo, hipStream_t s) {
+    auto kern = hy::window_attention_mfma_kernel<NS, NCT, NW, SH>;
     const int bytes = hy::WKT * (D * 2 + 16) + Dv * (hy::WKT * 2 + 8);
     static int set_bytes = 0;
     if (bytes > set_bytes) {
@@ -330,7 +365,7 @@ static void wa_mfma_launch(const uint16_t* qkv, int ldq, const uint16_t* kc, con
     }
     const dim3 grid(B, (max_q * (H / G) + 16 * NW - 1) / (16 * NW) * nsplit, G);
     kern<<<grid, 64 * NW, bytes, s>>>(qkv, ldq, kc, vc, bt, max_blocks, q_start, pos, sink, gate, out, H, G, D, Dv, BS, scale,
-                                      window, keep, chunk, nsplit, part_o, part_ml, pool, EP, kp, vp, vcs, g_off);
+                                      window, keep, chunk, nsplit, part_o, part_ml, pool, EP, kp, vp, vcs, g_off, ks, ldo);
 }
 
 bool hy_window_mfma_ok(int ldq, int D, int Dv) { return !(D % 32 || Dv % 16 || D > 256 || Dv > 256 || ldq % 8); }
@@ -363,18 +398,21 @@ bool launch_hy_window_attention_mfma(const uint16_t* qkv, int ldq, const uint16_
                                      const float* sink, const float* gate, uint16_t* out, int B, int max_q, int H, int G,
                                      int D, int Dv, int BS, float scale, int window, int keep, int chunk, int nsplit,
                                      float* part_o, float* part_ml, int64_t total_rows, int pool, int EP,
-                                     const uint16_t* kp, const uint16_t* vp, const float* vcs, int g_off, hipStream_t s) {
-    if (!hy_window_mfma_ok(ldq, D, Dv)) return false;
+                                     const uint16_t* kp, const uint16_t* vp, const float* vcs, int g_off, const float* ks,
+                                     int64_t ldo, hipStream_t s) {
+    if (!hy_window_mfma_ok(ldq, D, Dv) || ldo % 4) return false;
     if (B == 0 || max_q == 0) return true;
-#define HY_WAM(NS, NCT, NW) wa_mfma_launch<NS, NCT, NW>(qkv, ldq, kc, vc, bt, max_blocks, q_start, pos, sink, gate, out, B, max_q, H, G, D, Dv, BS, scale, window, keep, chunk, nsplit, part_o, part_ml, pool, EP, kp, vp, vcs, g_off, s)
+#define HY_WAM_S(NS, NCT, NW, SH) wa_mfma_launch<NS, NCT, NW, SH>(qkv, ldq, kc, vc, bt, max_blocks, q_start, pos, sink, gate, out, B, max_q, H, G, D, Dv, BS, scale, window, keep, chunk, nsplit, part_o, part_ml, pool, EP, kp, vp, vcs, g_off, ks, ldo, s)
+#define HY_WAM(NS, NCT, NW) do { if (ks != nullptr) HY_WAM_S(NS, NCT, NW, true); else HY_WAM_S(NS, NCT, NW, false); } while (0)
     // 8 waves per workgroup when a sequence brings more than 64 rows per key/value head: a staged tile then serves
     // 128 rows and every SIMD holds two waves
     const bool nw8 = max_q * (H / G) > 64;
     if (D <= 128 && Dv <= 128) { if (nw8) HY_WAM(4, 8, 8); else HY_WAM(4, 8, 4); }
     else { if (nw8) HY_WAM(8, 16, 8); else HY_WAM(8, 16, 4); }
 #undef HY_WAM
+#undef HY_WAM_S
     if (nsplit > 1)
-        hy::window_combine_kernel<<<(unsigned)((total_rows + 3) / 4), 256, 0, s>>>(part_o, part_ml, sink, gate, out, total_rows, H, Dv, nsplit, vcs, pos, qkv, ldq, g_off);
+        hy::window_combine_kernel<<<(unsigned)((total_rows + 3) / 4), 256, 0, s>>>(part_o, part_ml, sink, gate, out, total_rows, H, Dv, nsplit, vcs, pos, qkv, ldq, g_off, ldo);
     return true;
 }
 

@@ -214,9 +214,10 @@ def window_attention(qkv, kc, vc, block_table, q_start, pos, sink, gate, scale: 
     ``ks`` f32 [NB, BS, G] (kc None): key j is value j times its factor, one cached row serves both.  ``out``: where the
     output goes, [T, H Dv] columns of wider rows (not with v_cos_sin or g_off)."""
     if _gpu(qkv):
-        return _k().hy_window_attention(qkv, kc, vc, block_table, q_start, pos, sink, gate, scale, window, keep_first,
-                                        chunk, H, max_q, pool, kp if pool else None, vp if pool else None, v_cos_sin,
-                                        g_off, ks, out)
+        o = _k().hy_window_attention(qkv, kc, vc, block_table, q_start, pos, sink, gate, scale, window, keep_first,
+                                     chunk, H, max_q, pool, kp if pool else None, vp if pool else None, v_cos_sin,
+                                     g_off, ks, out)
+        return o if out is None else out
     o = ref.window_attention(qkv, kc, vc, block_table, q_start, pos, sink, gate, scale, window, keep_first, H,
                              act_dtype, chunk, pool, kp, vp, ks)
     if v_cos_sin is not None or g_off >= 0:
