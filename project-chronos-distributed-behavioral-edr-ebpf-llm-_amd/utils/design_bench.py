@@ -1,14 +1,16 @@
-"""Throughput of a hybrid design (Zokunex, Kalesun, Tugovik, Vogerax, Lalasun) beside the framework's other models at equal width and depth:
+"""Throughput of a hybrid design (Zokunex, Kalesun, Tugovik, Vogerax, Lalasun, Nubodra) beside the framework's other models at equal width and depth:
 whole-model prefill and decode steps, and each of the design's kernels beside its closest existing kernel with the
 fraction of its roofline it reaches.
 
-``python bench.py --design-compare [--design zokunex|kalesun|tugovik|vogerax|lalasun] [--design-sizes 1k,2k,4k]`` prints one JSON line
+``python bench.py --design-compare [--design zokunex|kalesun|tugovik|vogerax|lalasun|nubodra] [--design-sizes 1k,2k,4k]`` prints one JSON line
 (the default benchmark and its output line are untouched).  Zokunex stands beside Llama; Kalesun beside Zokunex (the
 closest family: recurrent layers, attention and mixtures of experts on a float32 stream) and Llama; Tugovik beside
 Kalesun (masked grouped-query attention over paged keys and values, linear-state scans behind a short convolution,
 gated experts, RMS norms on the stream) and Llama; Vogerax beside Kalesun too (windowed and causal sink attention on
 the same kernels, a linear-state scan, RMS norms joined to a float32 stream) and Llama; Lalasun beside Kalesun (masked
-sink attention, gated linear attention, dense feed-forwards), Zokunex (latent attention) and Llama.  Weights are random; every number is measured on the GPU this
+sink attention, gated linear attention, dense feed-forwards), Zokunex (latent attention) and Llama; Nubodra beside
+Kalesun (grouped-query attention over pages, short convolution, gated feed-forwards), Zokunex (causal latent attention)
+and Llama.  Weights are random; every number is measured on the GPU this
 process runs on.
 
 Rooflines: HBM 8 TB/s for kernels bound by the bytes they must move, 2.5 PFLOP/s dense bf16 for the matrix-shaped
@@ -150,6 +152,29 @@ def lalasun_config(size: dict) -> dict:
     mlp = dict(kind="dense", ff=size["ff"])
     layers = [dict(m, mlp=mlp) for m in (mix_g, mix_l, mix_a, mix_l)][:LAYERS]
     return dict(architecture="Lalasun", vocab=VOCAB, width=size["width"], residual_mult=0.4, norm=dict(eps=1e-6), layers=layers)
+
+
+# Nubodra: width -> (attention heads, kv heads, dim, conv taps | latent heads, dim, rot, vdim, rank, query rank | dense ff)
+NUBODRA_SIZES = {
+    "1k": dict(width=1024, a=(8, 2, 128, 4), l=(8, 64, 32, 64, 256, 384), ff=2816),
+    "2k": dict(width=2048, a=(16, 4, 128, 4), l=(16, 128, 64, 128, 512, 768), ff=5632),
+    "4k": dict(width=4096, a=(32, 8, 128, 4), l=(32, 128, 64, 128, 512, 1536), ff=11008),
+}
+
+
+def nubodra_config(size: dict) -> dict:
+    ah, ag, ad, taps = size["a"]
+    lh, ld, lr, lv, rank, qr = size["l"]
+    mix_a = dict(type="attention", mixer=dict(heads=ah, kv_heads=ag, dim=ad, vdim=ad, conv=taps, scale=ad ** -0.5,
+                                              q_temp=dict(coef=0.1, every=1024)))
+    lat = dict(heads=lh, dim=ld, rot_dim=lr, vdim=lv, kv_rank=rank, q_rank=qr, scale=(ld + lr) ** -0.5,
+               rot=dict(base=5e5, dims=lr, scaling=dict(factor=4.0, original=4096, fast=32.0, slow=1.0)))
+    mix_l = dict(type="latent_attention", mixer=lat)
+    mix_s = dict(type="latent_attention", mixer=dict(lat, kv_from=1))
+    mlp = dict(kind="dense", ff=size["ff"])
+    layers = [dict(m, mlp=mlp) for m in (mix_a, mix_l, mix_a, mix_s)][:LAYERS]
+    return dict(architecture="Nubodra", vocab=VOCAB, width=size["width"], embedding=dict(scale=2.0), norm=dict(eps=1e-6),
+                layers=layers)
 
 
 def _say(msg: str) -> None:
@@ -1059,6 +1084,215 @@ def run_lalasun(sizes: list, seqs: int = 4, plen: int = 2048, rows: int = 64, ct
                 dtype="bf16", data="synthetic", sizes=res)
 
 
+def _kernels_nubodra(size: dict, ksize: dict, zsize: dict, dev, T: int, ctx: int, rows: int) -> dict:
+    """Nubodra's kernels and their closest existing kernels at this size: seconds, and the fraction of the roofline
+    reached.  ``ksize``, ``zsize``: the Kalesun and Zokunex sizes of the same width (for the kernels it stands beside)."""
+    from chronos import ops
+    from chronos.models.hybrid import query_temperature, rope_cos_sin
+    from chronos.ops import hybrid as hops
+
+    out = {}
+    bf = torch.bfloat16
+    d = size["width"]
+    g = torch.Generator(device=dev).manual_seed(1)
+    rnd = lambda *s, dt=bf, sc=1.0: (torch.randn(*s, device=dev, generator=g) * sc).to(dt)  # noqa: E731
+    f32 = lambda *s, sc=1.0: rnd(*s, dt=torch.float32, sc=sc)  # noqa: E731
+    i32 = dict(dtype=torch.int32, device=dev)
+
+    def rec(name, secs, nbytes=0.0, flops=0.0):
+        roof = max(nbytes / HBM_BPS, flops / BF16_FLOPS)
+        _say(f"  {name}: {secs * 1e6:.1f} us, roofline {roof * 1e6:.2f} us")
+        out[name] = dict(us=round(secs * 1e6, 1), roofline_us=round(roof * 1e6, 2), of_roofline=round(roof / secs, 4))
+
+    bs = 16
+    seqs = max(1, T // ctx)
+    n = seqs * ctx
+    per = ctx // bs + 1
+    nb = max(seqs, rows) * per + 1
+    bt = torch.arange(1, 1 + seqs * per, **i32).view(seqs, per)
+    qs = torch.arange(0, (seqs + 1) * ctx, ctx, **i32)
+    pos = torch.arange(ctx, **i32).repeat(seqs)
+    tseq = torch.arange(seqs, **i32).repeat_interleave(ctx)
+    btd = torch.arange(1, 1 + rows * per, **i32).view(rows, per)
+    qsd = torch.arange(rows + 1, **i32)
+    tseqd = torch.arange(rows, **i32)
+    posd = torch.full((rows,), ctx, **i32)
+    NS = max(seqs, rows) + 1
+    p0, sl, sld = torch.zeros(seqs, **i32), torch.arange(seqs, **i32), torch.arange(rows, **i32)
+    full_pairs = n * (ctx + 1) / 2
+    # ---- the stream's joins
+    for name, m in (("", T), (".decode", rows)):
+        y, y2, x32, w1 = rnd(m, d), rnd(m, d), f32(m, d), f32(d)
+        wb = torch.cat([w1, f32(d, sc=0.1)])
+        rec("layer_norm_join" + name, _time(lambda: hops.layer_norm_join(y, x32, wb, 1e-6, bf)), m * d * (2 + 4 + 4 + 2))
+        rec("layer_norm_join.two" + name, _time(lambda: hops.layer_norm_join(y, x32, wb, 1e-6, bf, y2)), m * d * (2 + 2 + 4 + 4 + 2))
+        rec("kalesun.scale_add_rms_norm" + name, _time(lambda: hops.scale_add_rms_norm(y, x32, w1, 1.0, 1e-6, bf)), m * d * (2 + 4 + 4 + 2))
+        rec("zokunex.add_layer_norm" + name, _time(lambda: hops.add_layer_norm(y, x32, w1, 1e-6, bf)), m * d * (2 + 4 + 4 + 2))
+        xb, wbf = rnd(m, d), rnd(d)
+        rec("llama.add_rmsnorm" + name, _time(lambda: ops.add_rmsnorm(y, xb, wbf, 1e-5)), m * d * (2 + 2 + 2 + 2))
+    # ---- attention on unit keys beside the same attention over stored keys, Kalesun's window and Llama's
+    H, G, D, K = size["a"]
+    F = size["ff"]
+    C = (H + G) * D
+    width = (C + 2 * F + H + 15) // 16 * 16
+    vc, ks = rnd(nb, bs, G, D, sc=0.3), torch.rand(nb, bs, G, device=dev) + 0.5
+    proj, projd = rnd(n, width, sc=0.3), rnd(rows, width, sc=0.3)
+    taps, temp = f32(C, K, sc=0.5), query_temperature(0.1, 1024, ctx + 2, dev)
+    hist = rnd(NS, K - 1, C)
+    q, gate = hops.conv_prep(proj, taps, tseq, qs, p0, sl, hist, pos, bt, H, G, D, 1e-6, temp, ks, vc, C + 2 * F, ctx)
+    qd, gated = hops.conv_prep(projd, taps, tseqd, qsd, posd, sld, hist, posd, btd, H, G, D, 1e-6, temp, ks, vc, C + 2 * F, 1)
+    kc = rnd(nb, bs, G, D, sc=0.3)
+    wide, wided = rnd(n, H * D + F), rnd(rows, H * D + F)
+    at, atd = (bt, qs, pos), (btd, qsd, posd)
+    fl = 4.0 * full_pairs * H * D
+    rec("unit_attention.prefill", _time(lambda: hops.window_attention(q, None, vc, *at, None, gate, D ** -0.5, 0, 0, H, bf, ctx, ks=ks, out=wide[:, :H * D]), iters=3, warm=1), flops=fl)
+    rec("stored_keys.attention.prefill", _time(lambda: hops.window_attention(q, kc, vc, *at, None, gate, D ** -0.5, 0, 0, H, bf, ctx), iters=3, warm=1), flops=fl)
+    rec("unit_attention.decode", _time(lambda: hops.window_attention(qd, None, vc, *atd, None, gated, D ** -0.5, 0, 0, H, bf, 1, ks=ks, out=wided[:, :H * D])),
+        nbytes=rows * (ctx + 1) * G * (D * 2.0 + 4.0))
+    rec("stored_keys.attention.decode", _time(lambda: hops.window_attention(qd, kc, vc, *atd, None, gated, D ** -0.5, 0, 0, H, bf, 1)),
+        nbytes=rows * (ctx + 1) * G * D * 4.0)
+    rec("conv_prep.prefill", _time(lambda: hops.conv_prep(proj, taps, tseq, qs, p0, sl, hist, pos, bt, H, G, D, 1e-6, temp, ks, vc, C + 2 * F, ctx)),
+        nbytes=n * (C * 4.0 + G * 4.0 + H * 6.0))
+    rec("conv_prep.decode", _time(lambda: hops.conv_prep(projd, taps, tseqd, qsd, posd, sld, hist, posd, btd, H, G, D, 1e-6, temp, ks, vc, C + 2 * F, 1)),
+        nbytes=rows * (C * 4.0 + 2 * (K - 1) * C * 2.0 + G * 4.0 + H * 6.0))
+    kH, kG, kD, kDv, kwin, keep = ksize["a"]
+    kkc, kvc = rnd(nb, bs, kG, kD, sc=0.3), rnd(nb, bs, kG, kDv, sc=0.3)
+    kqkv, kqkvd = rnd(n, (kH + kG) * kD + kG * kDv, sc=0.3), rnd(rows, (kH + kG) * kD + kG * kDv, sc=0.3)
+    kgate, kgated, ksink = f32(n, kH), f32(rows, kH), f32(kH)
+    qn, ktab = f32(kD), rope_cos_sin(5e5, kD // 2, ctx + 2, dev)
+    kvis = sum(min(i + 1, kwin) + max(0, min(keep, i + 1 - kwin)) for i in range(ctx))
+    rec("kalesun.window_attention.prefill", _time(lambda: hops.window_attention(kqkv, kkc, kvc, *at, ksink, kgate, kD ** -0.5, kwin, keep, kH, bf, ctx), iters=3, warm=1),
+        flops=2.0 * seqs * kvis * kH * (kD + kDv))
+    rec("kalesun.window_attention.decode", _time(lambda: hops.window_attention(kqkvd, kkc, kvc, *atd, ksink, kgated, kD ** -0.5, kwin, keep, kH, bf, 1)),
+        nbytes=rows * (min(ctx + 1, kwin) + keep) * kG * (kD + kDv) * 2.0)
+    for name, m, x, ps, ts, b_ in (("prefill", n, kqkv, pos, tseq, bt), ("decode", rows, kqkvd, posd, tseqd, btd)):
+        rec(f"kalesun.window_prep.{name}", _time(lambda: hops.window_prep(x, kH, kG, kD, kDv, None, None, ps, ts, b_, qn, qn, 1e-5, ktab, kD // 2, kkc, kvc, False)),
+            nbytes=m * (2 * (kH + kG) * kD + 2 * kG * kDv) * 2.0)
+    dh, dk, dd, dv = ksize["d"]
+    Cc = 2 * dk * dd + dh * dv
+    xc, xcd, ktaps = rnd(n, Cc + dh * dv), rnd(rows, Cc + dh * dv), f32(Cc, 4)
+    khist = torch.zeros(NS, 3, Cc, device=dev, dtype=bf)
+    rec("kalesun.short_conv.prefill", _time(lambda: hops.short_conv(xc, ktaps, tseq, qs, p0, sl, khist, True)), nbytes=n * Cc * 4.0)
+    rec("kalesun.short_conv.decode", _time(lambda: hops.short_conv(xcd, ktaps, tseqd, qsd, posd, sld, khist, True)), nbytes=rows * Cc * 16.0)
+    hq = d // 128
+    hkv = max(1, hq // 4)
+    akc, avc = rnd(nb, hkv, bs, 128, sc=0.3), rnd(nb, hkv, 128, bs, sc=0.3)
+    lq, lqd = rnd(n, hq, 128, sc=0.3), rnd(rows, hq, 128, sc=0.3)
+    ctxl, ctxd = torch.full((seqs,), ctx, **i32), torch.full((rows,), ctx + 1, **i32)
+    tiles = torch.tensor(ops.attention_tiles([ctx] * seqs, hq, hkv, 8), **i32).view(-1, 2)
+    rec("llama.attention.prefill", _time(lambda: ops.paged_attention(lq, akc, avc, bt, qs, ctxl, tiles, tiles.shape[0], 8, 1), iters=3, warm=1),
+        flops=4.0 * full_pairs * hq * 128)
+    nsp = ops.pick_nsplit(rows * hkv, ctx + 1)
+    rec("llama.attention.decode", _time(lambda: ops.paged_attention(lqd, akc, avc, btd, qsd, ctxd, None, rows, 1, nsp)),
+        nbytes=rows * (ctx + 1) * hkv * 128 * 2 * 2.0)
+    del kc, vc, kkc, kvc, akc, avc, kqkv, lq, xc
+    # ---- latent attention with sinks beside Zokunex's
+    lH, lD, R, Dv, rank, qr = size["l"]
+    DK, nq = rank + R, lH * (lD + R)
+    lat = rnd(nb, bs, DK, sc=0.3)
+    qa, qad, sink = rnd(n, lH, DK, sc=0.3), rnd(rows, lH, DK, sc=0.3), f32(lH)
+    rec("latent_sink.prefill", _time(lambda: hops.latent_attention(qa, lat, *at, None, 0.1, rank, bf, ctx, 0, True, sink), iters=3, warm=1),
+        flops=2.0 * full_pairs * lH * (DK + rank))
+    rec("latent_sink.decode", _time(lambda: hops.latent_attention(qad, lat, *atd, None, 0.1, rank, bf, 1, 0, True, sink)),
+        nbytes=rows * (ctx + 1) * DK * 2.0)
+    zH, zD, zR, zDv, zrank = zsize["a"]
+    zlat = rnd(nb, bs, zrank + zR, sc=0.3)
+    zqa, zqad = rnd(n, zH, zrank + zR, sc=0.3), rnd(rows, zH, zrank + zR, sc=0.3)
+    zg, zgd = f32(n, zH), f32(rows, zH)
+    rec("zokunex.latent_attention.prefill", _time(lambda: hops.latent_attention(zqa, zlat, *at, zg, 0.1, zrank, bf, ctx), iters=3, warm=1),
+        flops=2.0 * full_pairs * zH * (2 * zrank + zR))
+    rec("zokunex.latent_attention.decode", _time(lambda: hops.latent_attention(zqad, zlat, *atd, zgd, 0.1, zrank, bf, 1)),
+        nbytes=rows * (ctx + 1) * (zrank + zR) * 2.0)
+    ltab, wn, wq = rope_cos_sin(5e5, R, ctx + 2, dev, ("ramp", 4.0, 4096.0, 32.0, 1.0)), f32(rank), f32(qr)
+    wuk, wuv = rnd(lH, rank, lD, sc=lD ** -0.5), rnd(lH, Dv, rank, sc=rank ** -0.5)
+    for name, m, qx, ps, ts, b_ in (("prefill", n, qa, pos, tseq, bt), ("decode", rows, qad, posd, tseqd, btd)):
+        lw = (qr + DK + 7) // 8 * 8 + 2 * F
+        lproj, lqq, w_out = rnd(m, lw, sc=0.3), rnd(m, lH, lD + R, sc=0.3), rnd(m, lH * Dv + F)
+        xf = f32(m, qr)
+        rec(f"norm_cols.{name}", _time(lambda: hops.norm_cols(lproj, 0, qr, wq, 1e-6)), nbytes=m * qr * 4.0)
+        rec(f"rms_norm.{name}", _time(lambda: hops.rms_norm(xf, wq, 1e-6, bf)), nbytes=m * qr * 6.0)
+        rec(f"latent_prep.{name}", _time(lambda: hops.latent_prep(lqq, lproj[:, qr:qr + DK], ps, ts, b_, wn, 1e-6, ltab, R, rank, lat, qx, True)),
+            nbytes=m * (2 * DK + 2 * lH * R) * 2.0)
+        rec(f"latent_prep.shared.{name}", _time(lambda: hops.latent_prep(lqq, None, ps, ts, b_, None, 1e-6, ltab, R, rank, lat, qx, True)),
+            nbytes=m * 2 * lH * R * 2.0)
+        oa = rnd(m, lH, rank)
+        rec(f"head_matmul.to_latent.{name}", _time(lambda: hops.head_matmul(lqq[:, :, :lD], wuk, qx[:, :, :rank])),
+            nbytes=(m * lH * (lD + rank) + lH * lD * rank) * 2.0, flops=2.0 * m * lH * lD * rank)
+        rec(f"head_matmul.from_latent.{name}", _time(lambda: hops.head_matmul(oa, wuv, w_out[:, :lH * Dv].view(m, lH, Dv))),
+            nbytes=(m * lH * (Dv + rank) + lH * Dv * rank) * 2.0, flops=2.0 * m * lH * Dv * rank)
+        # ---- the gated unit on columns, and a layer's products: shared with the mixer's, or each its own
+        kz = rnd(m, 2 * ksize["ff"])
+        rec(f"glu_cols.{name}", _time(lambda: hops.glu_cols(lproj, lw - 2 * F, F, float("inf"), 1.0, 0.0, w_out[:, lH * Dv:])), nbytes=m * F * 6.0)
+        rec(f"kalesun.glu.{name}", _time(lambda: hops.glu(kz, 7.0, 1.702, 1.0, bf)), nbytes=m * ksize["ff"] * 6.0)
+    del lat, zlat, qa, zqa, oa, lproj, lqq
+    w_in, w_o = rnd(width, d, sc=d ** -0.5), rnd(d, H * D + F, sc=d ** -0.5)
+    wq_, wg_, wo_, wd_ = w_in[:C].contiguous(), w_in[C:C + 2 * F].contiguous(), w_o[:, :H * D].contiguous(), w_o[:, H * D:].contiguous()
+    wgate = w_in[C + 2 * F:C + 2 * F + H].contiguous()
+    lf = int(3.5 * d)
+    lgu, ldn = rnd(2 * lf, d, sc=d ** -0.5), rnd(d, lf, sc=lf ** -0.5)
+    for name, m in (("prefill", T), ("decode", rows)):
+        h, o = rnd(m, d), rnd(m, H * D)
+        w_out = rnd(m, H * D + F)
+
+        def fused():
+            p = hops.matmul(h, w_in)
+            hops.glu_cols(p, C, F, float("inf"), 1.0, 0.0, w_out[:, H * D:])
+            return hops.matmul(w_out, w_o)
+
+        def apart():
+            hops.matmul(h, wq_)
+            hops.rowdot(h, wgate)
+            return hops.matmul(o, wo_), hops.matmul(hops.glu(hops.matmul(h, wg_), float("inf"), 1.0, 0.0, bf), wd_)
+
+        fl = 2.0 * m * d * (C + 3 * F + H * D)
+        nby = (d * (C + 3 * F + H * D) + m * d * 2) * 2.0
+        rec(f"layer_products.shared.{name}", _time(fused, iters=3, warm=1), nbytes=nby, flops=fl)
+        rec(f"layer_products.apart.{name}", _time(apart, iters=3, warm=1), nbytes=nby, flops=fl)
+        rec(f"llama.mlp.{name}", _time(lambda: ops.linear(ops.gate_up_silu(h, lgu), ldn), iters=3, warm=1),
+            nbytes=3 * lf * d * 2.0 + m * d * 4.0, flops=m * 6.0 * lf * d)
+    return out
+
+
+def run_nubodra(sizes: list, seqs: int = 4, plen: int = 2048, rows: int = 64, ctx: int = 2048, device: str = "cuda") -> dict:
+    from chronos import ops
+    from chronos.models import kalesun, llama, nubodra, zokunex
+    from chronos.models.hybrid import HybridDecoder
+
+    dev = torch.device(device if ":" in device else device + ":0")
+    torch.cuda.set_device(dev)
+    ops.load()
+    ops.device_init()
+    res = {}
+    P = ctx + plen + 16
+    for name in sizes:
+        size, ksize, zsize = NUBODRA_SIZES[name], KALESUN_SIZES[name], SIZES[name]
+        t0 = time.time()
+        entry = {}
+        for mod, key, conf in ((nubodra, "nubodra", nubodra_config(size)), (kalesun, "kalesun", kalesun_config(ksize)),
+                               (zokunex, "zokunex", zokunex_config(zsize))):
+            cfg = mod.config_from_dict(conf, name=f"{key}-{name}", max_position=P)
+            m = HybridDecoder(cfg, mod.pack_weights(cfg, mod.random_tensors(cfg, 0), dev, torch.bfloat16), dev, P, torch.bfloat16)
+            entry[key] = dict(params=cfg.param_count(), **_model_steps(m, dev, seqs, plen, rows, ctx))
+            _say(f"size {name}: {key} {entry[key]}")
+            del m
+        d = size["width"]
+        lc = llama.LlamaConfig(name=f"llama-{name}", vocab_size=VOCAB, hidden_size=d, intermediate_size=int(3.5 * d),
+                               num_layers=LAYERS, num_heads=d // 128, num_kv_heads=max(1, d // 512), max_position=P)
+        lm = llama.LlamaModel(lc, llama.random_weights(lc, None, dev, 0), None, dev, P)
+        entry["llama"] = dict(params=lc.param_count(), **_model_steps(lm, dev, seqs, plen, rows, ctx))
+        _say(f"  llama {entry['llama']}")
+        del lm
+        torch.cuda.empty_cache()
+        entry["kernels"] = _kernels_nubodra(size, ksize, zsize, dev, seqs * plen, ctx, rows)
+        entry["seconds"] = round(time.time() - t0, 1)
+        res[name] = entry
+        torch.cuda.empty_cache()
+    return dict(metric="design_compare", design="nubodra", beside="kalesun, zokunex and llama (equal width and depth)",
+                layers=LAYERS, workload=dict(prefill=f"{seqs} x {plen} tokens in one step",
+                                             decode=f"{rows} rows at context {ctx}"),
+                dtype="bf16", data="synthetic", sizes=res)
+
+
 def run_kalesun(sizes: list, seqs: int = 4, plen: int = 2048, rows: int = 64, ctx: int = 2048, device: str = "cuda") -> dict:
     from chronos import ops
     from chronos.models import kalesun, llama, zokunex
@@ -1142,7 +1376,7 @@ def run(sizes: list, seqs: int = 4, plen: int = 2048, rows: int = 64, ctx: int =
 def main(a) -> int:
     sizes = [s for s in a.design_sizes.split(",") if s]
     fn = {"kalesun": run_kalesun, "tugovik": run_tugovik, "vogerax": run_vogerax,
-          "lalasun": run_lalasun}.get(getattr(a, "design", "zokunex"), run)
+          "lalasun": run_lalasun, "nubodra": run_nubodra}.get(getattr(a, "design", "zokunex"), run)
     out = fn(sizes, device=a.device)
     print(json.dumps(out), flush=True)
     return 0
