@@ -25,6 +25,34 @@ __device__ __forceinline__ float sigmoidf_(float z) { return 1.f / (1.f + expf(-
 // log(sigmoid(z)) without overflow on either side
 __device__ __forceinline__ float logsigmoidf_(float z) { return fminf(z, 0.f) - log1pf(expf(-fabsf(z))); }
 
+// Transposing LDS read (gfx950): the 16 lanes of a lane group name the 8-byte pieces of a 4 x 16 matrix of 16-bit
+// elements, row by row (lane l: row l / 4, columns 4 (l % 4) ..), and lane l receives column l, its 4 rows in order.
+// Rows may lie anywhere.  A row-major tile thus serves as either operand of a matrix product.
+__device__ __forceinline__ bf16x4 lds_read_tr4(const void* p) {
+    typedef __attribute__((address_space(3))) bf16x4 lds_bf16x4;
+    return __builtin_amdgcn_ds_read_tr16_b64_v4bf16((lds_bf16x4*)p);
+}
+
+// One 1 KiB piece from memory straight into LDS: lane l's 16 bytes from its own address to LDS offset lds + 16 l (lds the
+// same in all lanes).  Inline asm, so that the compiler does not wait for it before every LDS read; the kernel waits with
+// dma_wait() in front of the barrier that hands the piece over.
+__device__ __forceinline__ void dma_1k(const void* src, uint32_t lds) {
+    asm volatile("s_mov_b32 m0, %1\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %0, off" ::"v"(src), "s"(lds) : "memory");
+}
+__device__ __forceinline__ void dma_wait() { asm volatile("s_waitcnt vmcnt(0)" ::: "memory"); }
+__device__ __forceinline__ uint32_t lds_offset(const void* p) {
+    typedef __attribute__((address_space(3))) const void* lds_ptr;
+    return (uint32_t)(uintptr_t)(lds_ptr)p;
+}
+// Piece j of a tile of rows: an LDS image of row-major rows, each CPR chunks of 16 bytes of which the last is padding
+// (it spreads the rows over the banks; like the chunks past the row's n real ones it receives a copy of the last real
+// one).  rows: element offset factor of each row of the tile; width: elements per row in memory.
+template <int CPR> __device__ __forceinline__ void dma_rows(const uint16_t* src, const int* rows, int width, int n, int j,
+                                                            uint32_t lds, int lane) {
+    const int i = j * 64 + lane, row = i / CPR, ch = i - row * CPR;
+    dma_1k(src + (int64_t)rows[row] * width + min(ch, n - 1) * 8, __builtin_amdgcn_readfirstlane(lds + j * 1024));
+}
+
 constexpr int kActRelu2 = 0, kActGelu = 1;
 __device__ __forceinline__ float act_apply(float z, int kind) {
     if (kind == kActRelu2) {

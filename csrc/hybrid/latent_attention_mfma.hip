@@ -3,16 +3,16 @@
 //
 // One workgroup takes 64 (token, head) rows of one sequence — 16 per wave, rows are (token * H + head), so any head
 // count tiles the same way — and walks the sequence's keys 64 at a time:
-//   * the key tile is staged twice in LDS: row-major [64][DK] for the scores, and the value columns transposed
-//     [rank][64] for the weighted sum (both MFMA operands want 8 consecutive k-values per lane: dims for the scores,
-//     KEYS for the sum).  One pass of 16-byte global loads feeds both; the transposed image is written as 32-bit
-//     words holding two neighbouring keys.
+//   * the key tile goes from memory straight into LDS (no staging registers), row-major [64][DK], two tiles deep: the next
+//     tile is on its way while the current one is computed, one barrier per tile.  Both MFMA operands want 8 k-values per lane — dims for
+//     the scores, KEYS for the weighted sum: the scores read rows as they lie, the sum reads the same image through
+//     gfx950's transposing LDS reads (4 keys of 16 columns each).
 //   * scores  S^T = K Q^T : 16x16x32 MFMAs with the key rows as A operand and the wave's 16 query rows (held in
 //     registers for the whole kernel) as B operand, so a lane ends up with 4 keys x 1 query row per 16-key tile;
 //   * softmax in float per query row (lane & 15): causal mask by the row's own position, running maximum and sum,
 //     reductions over the 4 lane groups by two shuffles;
 //   * sum  O^T = V^T P^T : the lane's 8 weights of two neighbouring 16-key tiles ARE a B operand (the k index is a
-//     fixed permutation of the 32 keys, the same one the transposed value image is read with), so the weights never
+//     fixed permutation of the 32 keys, the same one the value columns are read with), so the weights never
 //     leave registers.  Accumulators: rank / 16 tiles x 4 registers.  Optionally each weight enters as two
 //     bfloat16 terms (rounded value + remainder), which keeps the float softmax weights nearly exact.
 // After the last key a sink per head may join the denominator.
@@ -27,15 +27,13 @@
 namespace chronos {
 namespace hy {
 
-constexpr int MKT = 64;  // keys per tile at most
+constexpr int MKT = 64;  // keys per tile
 
-// NS: k-steps of the scores (DK / 32) at most; NCT: 16-column tiles of the output (rank / 16) at most; KT: keys per
-// tile, 64 or 32 (32 halves the LDS images, so two workgroups share a CU at the widest rows and one stages while the
-// other multiplies).
+// NS: k-steps of the scores (DK / 32) at most; NCT: 16-column tiles of the output (rank / 16) at most.
 // NW: waves per workgroup, 4 or 8 (16 query rows each): with 8 a staged key tile serves 128 rows and every SIMD holds two
 // waves, so one wave's softmax and staging run beside the other's MFMAs.
 // TT: weights as two bfloat16 terms.
-template <int NS, int NCT, int KT, int NW, bool TT>
+template <int NS, int NCT, int NW, bool TT>
 __global__ void __launch_bounds__(64 * NW) latent_attention_mfma_kernel(
         const uint16_t* __restrict__ qa, const uint16_t* __restrict__ cache, const int32_t* __restrict__ block_table,
         int max_blocks, const int32_t* __restrict__ q_start, const int32_t* __restrict__ pos,
@@ -46,17 +44,13 @@ __global__ void __launch_bounds__(64 * NW) latent_attention_mfma_kernel(
     const int b = blockIdx.x;
     const int t0 = q_start[b], t1 = q_start[b + 1];
     const int rows_total = (t1 - t0) * H;
-    constexpr int NT = 64 * NW, RPB = 16 * NW;  // threads and query rows per workgroup
+    constexpr int KT = MKT, RPB = 16 * NW;  // query rows per workgroup
     const int rb0 = blockIdx.y * RPB;
     if (rb0 >= rows_total) return;
     const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6, g = lane >> 4, qi = lane & 15;
     const int ns = (DK + 31) / 32, nct = rank / 16;
-    const int krs = ns * 64 + 16;           // row-major image: bytes per key row
-    constexpr int vts = KT * 2 + 8;         // transposed image: bytes per value column
-    constexpr int PP = KT / 2;              // key pairs per tile
-    __shared__ int krow[MKT];  // cache row (page * page size + slot) of each key of the tile
-    unsigned char* kimg = smem;
-    unsigned char* vimg = smem + KT * krs;
+    constexpr int CPR = NS * 4 + 1, krs = CPR * 16;   // key row in LDS: 16-byte chunks, bytes
+    __shared__ int krow[2][KT];  // cache row (page * page size + slot) of each key of a tile
     // this lane's query row (for the B operand and for the softmax): row r of the sequence, token t0 + r / H
     const int r = rb0 + wv * 16 + qi;
     const bool rok = r < rows_total;
@@ -80,54 +74,32 @@ __global__ void __launch_bounds__(64 * NW) latent_attention_mfma_kernel(
     for (int c = 0; c < NCT; ++c) O[c] = f32x4{0.f, 0.f, 0.f, 0.f};
     float mrow = -INFINITY, lrow = 0.f;
     const int32_t* bt = block_table + (int64_t)b * max_blocks;
-    const int chunks = DK / 8, vchunks = rank / 8;
-    const int padc = ns * 4 - chunks;   // zero chunks behind a key row (staging never writes them)
-    for (int it = threadIdx.x; it < KT * padc; it += NT) {
-        const u16x8 z = {0, 0, 0, 0, 0, 0, 0, 0};
-        *reinterpret_cast<u16x8*>(kimg + it / padc * krs + (chunks + it % padc) * 16) = z;
-    }
+    const int chunks = DK / 8;
+    const uint32_t lds0 = lds_offset(smem);
     // key tiles are dealt round-robin to the nsplit workgroups of this row block (blockIdx.z): the context length is
     // only known on the device, and a split that gets no tile contributes an empty partial
-    for (int k0 = k_lo + blockIdx.z * KT; k0 <= pmax; k0 += KT * nsplit) {
-        __syncthreads();
-        // ---- cache rows of the tile's 64 keys (page lookup once per key, not once per staged vector: a lookup in
-        // front of every data load made each of them wait for two trips to memory)
-        if (threadIdx.x < KT) {
-            const int key = min(k0 + (int)threadIdx.x, pmax);  // past the end: a real row, masked below
-            krow[threadIdx.x] = bs_shift >= 0 ? ((bt[key >> bs_shift] << bs_shift) + (key & (BS - 1)))
-                                              : (bt[key / BS] * BS + key % BS);
-        }
-        __syncthreads();
-        // ---- stage: work item = (key pair jp, 8-dim chunk dc); lanes of a wave take consecutive key pairs; three
-        // items' loads (six 16-byte vectors) are issued before any of them is written to LDS
-        for (int it0 = threadIdx.x; it0 < PP * chunks; it0 += NT * 3) {
-            u16x8 va[3], vb[3];
+    const int kfirst = k_lo + blockIdx.z * KT, kstep = KT * nsplit;
+    auto row_of = [&](int k0) {
+        const int key = min(k0 + (int)threadIdx.x, pmax);  // past the end: a real row, masked below
+        return bs_shift >= 0 ? ((bt[key >> bs_shift] << bs_shift) + (key & (BS - 1))) : (bt[key / BS] * BS + key % BS);
+    };
+    auto stage = [&](int buf) {
 #pragma unroll
-            for (int u = 0; u < 3; ++u) {
-                const int it = it0 + NT * u;
-                if (it < PP * chunks) {
-                    const int jp = it & (PP - 1), dc = it / PP;
-                    va[u] = *reinterpret_cast<const u16x8*>(cache + (int64_t)krow[2 * jp] * DK + dc * 8);
-                    vb[u] = *reinterpret_cast<const u16x8*>(cache + (int64_t)krow[2 * jp + 1] * DK + dc * 8);
-                }
-            }
-#pragma unroll
-            for (int u = 0; u < 3; ++u) {
-                const int it = it0 + NT * u;
-                if (it < PP * chunks) {
-                    const int jp = it & (PP - 1), dc = it / PP;
-                    *reinterpret_cast<u16x8*>(kimg + (2 * jp) * krs + dc * 16) = va[u];
-                    *reinterpret_cast<u16x8*>(kimg + (2 * jp + 1) * krs + dc * 16) = vb[u];
-                    if (dc < vchunks) {
-#pragma unroll
-                        for (int e = 0; e < 8; ++e)
-                            *reinterpret_cast<uint32_t*>(vimg + (dc * 8 + e) * vts + jp * 4) =
-                                (uint32_t)va[u][e] | ((uint32_t)vb[u][e] << 16);
-                    }
-                }
-            }
-        }
-        __syncthreads();
+        for (int j = wv; j < CPR; j += NW) dma_rows<CPR>(cache, krow[buf], DK, chunks, j, lds0 + buf * KT * krs, lane);
+    };
+    if (threadIdx.x < KT) krow[0][threadIdx.x] = row_of(kfirst);
+    __syncthreads();
+    if (kfirst <= pmax) stage(0);
+    if (threadIdx.x < KT) krow[1][threadIdx.x] = row_of(kfirst + kstep);
+    const bool wave_on = rb0 + wv * 16 < rows_total;   // (a wave without rows only helps to stage)
+    int buf = 0;
+    for (int k0 = kfirst; k0 <= pmax; k0 += kstep, buf ^= 1) {
+        dma_wait();        // this wave's pieces of the tile have landed
+        __syncthreads();   // ... everyone's; the other buffer's tile has been read by all; its next rows are known
+        if (k0 + kstep <= pmax) stage(buf ^ 1);
+        const int nrow = threadIdx.x < KT ? row_of(k0 + 2 * kstep) : 0;
+        const unsigned char* kimg = smem + buf * KT * krs;
+        if (wave_on) {
         // ---- scores: KT / 16 key tiles of 16; lane gets keys 16 kt + 4 g + i of query row qi
         constexpr int NKT = KT / 16;
         f32x4 S[NKT];
@@ -171,31 +143,29 @@ __global__ void __launch_bounds__(64 * NW) latent_attention_mfma_kernel(
         mrow = mn;
         // ---- weighted sum of the value columns: k index of step u = [tile 2u keys 4g..4g+3 | tile 2u+1 keys 4g..4g+3]
         constexpr int NU = KT / 32;
-        bf16x8 pf[NU], pl[TT ? NU : 1];
+        const unsigned char* vt = kimg + (4 * g + (qi >> 2)) * krs + (qi & 3) * 8;
 #pragma unroll
         for (int u = 0; u < NU; ++u) {
-            pf[u] = bf16x8{(__bf16)S[2 * u][0], (__bf16)S[2 * u][1], (__bf16)S[2 * u][2], (__bf16)S[2 * u][3],
-                           (__bf16)S[2 * u + 1][0], (__bf16)S[2 * u + 1][1], (__bf16)S[2 * u + 1][2], (__bf16)S[2 * u + 1][3]};
-            if constexpr (TT) {
+            bf16x8 pf, pl;
 #pragma unroll
-                for (int e = 0; e < 8; ++e) pl[u][e] = (__bf16)(S[2 * u + (e >> 2)][e & 3] - (float)pf[u][e]);
+            for (int e = 0; e < 8; ++e) {
+                const float w = S[2 * u + (e >> 2)][e & 3];
+                pf[e] = (__bf16)w;
+                if constexpr (TT) pl[e] = (__bf16)(w - (float)pf[e]);
             }
-        }
 #pragma unroll
-        for (int c = 0; c < NCT; ++c) {
-            if (c < nct) {
-                O[c] *= corr;
-                const unsigned char* vrow = vimg + (16 * c + qi) * vts + g * 8;
-#pragma unroll
-                for (int u = 0; u < NU; ++u) {
-                    const bf16x4 lo = *reinterpret_cast<const bf16x4*>(vrow + u * 64);
-                    const bf16x4 hi = *reinterpret_cast<const bf16x4*>(vrow + u * 64 + 32);
+            for (int c = 0; c < NCT; ++c)
+                if (c < nct) {
+                    const bf16x4 lo = lds_read_tr4(vt + 32 * u * krs + c * 32);
+                    const bf16x4 hi = lds_read_tr4(vt + (32 * u + 16) * krs + c * 32);
                     const bf16x8 vf = __builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7);
-                    O[c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pf[u], O[c], 0, 0, 0);
-                    if constexpr (TT) O[c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pl[u], O[c], 0, 0, 0);
+                    if (u == 0) O[c] *= corr;
+                    O[c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pf, O[c], 0, 0, 0);
+                    if constexpr (TT) O[c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pl, O[c], 0, 0, 0);
                 }
-            }
         }
+        }
+        if (threadIdx.x < KT) krow[buf][threadIdx.x] = nrow;
     }
     if (!rok) return;
     if (nsplit > 1) {  // unnormalised partial: the combine kernel merges the splits
@@ -254,13 +224,13 @@ __global__ void __launch_bounds__(256) latent_combine_kernel(const float* __rest
 
 }  // namespace hy
 
-template <int NS, int NCT, int KT, int NW, bool TT>
+template <int NS, int NCT, int NW, bool TT>
 static void la_mfma_launch(const uint16_t* qa, const uint16_t* cache, const int32_t* bt, int max_blocks,
                            const int32_t* q_start, const int32_t* pos, const float* gate, uint16_t* out, int B, int H,
                            int DK, int rank, int BS, int max_q, float scale, int window, int nsplit, float* part_o,
                            float* part_ml, const float* sink, hipStream_t s) {
-    auto kern = hy::latent_attention_mfma_kernel<NS, NCT, KT, NW, TT>;
-    const int bytes = KT * ((DK + 31) / 32 * 64 + 16) + rank * (KT * 2 + 8);
+    auto kern = hy::latent_attention_mfma_kernel<NS, NCT, NW, TT>;
+    constexpr int bytes = 2 * hy::MKT * (NS * 64 + 16);
     static int set_bytes = 0;
     if (bytes > set_bytes) {
         (void)hipFuncSetAttribute(reinterpret_cast<const void*>(kern), hipFuncAttributeMaxDynamicSharedMemorySize, bytes);
@@ -294,19 +264,14 @@ bool launch_hy_latent_attention_mfma(const uint16_t* qa, const uint16_t* cache, 
                                      hipStream_t s) {
     if (!hy_latent_mfma_ok(DK, rank)) return false;
     if (B == 0 || max_q == 0) return true;
-#define HY_LAM(NS, NCT, KT, NW, TT) la_mfma_launch<NS, NCT, KT, NW, TT>(qa, cache, bt, max_blocks, q_start, pos, gate, out, B, H, DK, rank, BS, max_q, scale, window, nsplit, part_o, part_ml, sink, s)
-    // 64-key tiles (32-key tiles measured slower at every size: the per-tile softmax and barriers weigh more than the
-    // second workgroup per CU gains; CHRONOS_LATENT_KT=32 keeps them for A/B).  8 waves per workgroup when a sequence
-    // brings more than 64 rows (CHRONOS_LATENT_NW=4 / 8 forces one).
-    static const int force_kt = [] { const char* v = getenv("CHRONOS_LATENT_KT"); return v ? atoi(v) : 0; }();
+#define HY_LAM(NS, NCT, NW, TT) la_mfma_launch<NS, NCT, NW, TT>(qa, cache, bt, max_blocks, q_start, pos, gate, out, B, H, DK, rank, BS, max_q, scale, window, nsplit, part_o, part_ml, sink, s)
+    // 8 waves per workgroup when a sequence brings more than 64 rows (CHRONOS_LATENT_NW=4 / 8 forces one)
     static const int force_nw = [] { const char* v = getenv("CHRONOS_LATENT_NW"); return v ? atoi(v) : 0; }();
-    const bool kt32 = force_kt == 32;
     const bool nw8 = force_nw == 8 || (force_nw != 4 && max_q * H > 64);
 #define HY_LAM_T(NS, NCT)                                                            \
     do {                                                                             \
-        if (two_term) { if (nw8) HY_LAM(NS, NCT, 64, 8, true); else HY_LAM(NS, NCT, 64, 4, true); }         \
-        else if (kt32) { if (nw8) HY_LAM(NS, NCT, 32, 8, false); else HY_LAM(NS, NCT, 32, 4, false); }      \
-        else { if (nw8) HY_LAM(NS, NCT, 64, 8, false); else HY_LAM(NS, NCT, 64, 4, false); }                \
+        if (two_term) { if (nw8) HY_LAM(NS, NCT, 8, true); else HY_LAM(NS, NCT, 4, true); }   \
+        else { if (nw8) HY_LAM(NS, NCT, 8, false); else HY_LAM(NS, NCT, 4, false); }          \
     } while (0)
     if (DK <= 128 && rank <= 64) HY_LAM_T(4, 4);
     else if (DK <= 320 && rank <= 256) HY_LAM_T(10, 16);

@@ -6,15 +6,16 @@
 // at a time: first (with pooled blocks) the pooled pairs of the blocks that lie wholly before a row's window, then the
 // kept first tokens that lie below the window's first tile, then the tiles from the window's first key to the last
 // query.  Per tile:
-//   * the keys are staged row-major [64][D] and the values transposed [Dv][64] in LDS (both MFMA operands want 8
-//     consecutive k-values per lane: dims for the scores, KEYS for the sum); the transposed image is written as
-//     32-bit words holding two neighbouring keys;
+//   * keys and values go from memory straight into LDS (no staging registers), row-major [64][D] and [64][Dv], two tiles
+//     deep: the next tile is on its way while the current one is computed, one barrier per tile.  Both MFMA operands want 8 k-values per lane —
+//     dims for the scores, KEYS for the sum: the sum reads the values through gfx950's transposing LDS reads (4 keys of
+//     16 columns each);
 //   * scores  S^T = K Q^T : 16x16x32 MFMAs, key rows as A operand, the wave's 16 query rows (in registers for the
 //     whole kernel) as B operand: a lane ends up with 4 keys x 1 query row per 16-key tile;
 //   * softmax in float per query row (lane & 15): each row masks by its own position (causal, window, kept tokens),
 //     running maximum and sum, reductions over the 4 lane groups by two shuffles;
 //   * sum  O^T = V^T P^T : the lane's 8 weights of two neighbouring 16-key tiles ARE a B operand (the k index is a
-//     fixed permutation of the 32 keys, the same one the transposed value image is read with); each weight enters
+//     fixed permutation of the 32 keys, the same one the value columns are read with); each weight enters
 //     as two bfloat16 terms (rounded value + remainder), which keeps the float softmax weights nearly exact.
 // After the last tile the head's sink joins the denominator and the row is scaled by sigmoid(gate).  Two more steps
 // may follow in the same epilogue: with a rotation table for the values, the head's output row is turned BACK by the
@@ -22,8 +23,8 @@
 // c + Dv / 32), and with a gate per output column the row is multiplied by sigmoid of the gate columns of the
 // query's own projection row.  Launches of few
 // rows (decode) deal a row block's key tiles to several workgroups and merge the float partials in a second kernel.
-// With unit keys (SH: a key is the cached value times a float factor) a row is loaded once and written to both images,
-// and a score is multiplied by its key's factor.
+// With unit keys (SH: a key is the cached value times a float factor) the one image serves both products, and a score is
+// multiplied by its key's factor.
 // With chunk > 0 a row also hides the keys below its own chunk of positions (key >= floor(pos / chunk) * chunk).
 // Sizes: D % 32 == 0, Dv % 16 == 0, D <= 256, Dv <= 256.  Everything else takes the general kernel.
 #include <algorithm>
@@ -45,7 +46,7 @@ __global__ void __launch_bounds__(64 * NW) window_attention_mfma_kernel(
         const uint16_t* __restrict__ kp, const uint16_t* __restrict__ vp, const float* __restrict__ vcs, int g_off,
         const float* __restrict__ ks, int64_t ldo) {
     extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
-    constexpr int KT = WKT, NT = 64 * NW, RPB = 16 * NW, PP = KT / 2;
+    constexpr int KT = WKT, RPB = 16 * NW;
     const int R = H / G;
     const int b = blockIdx.x, kvh = blockIdx.z;
     const int t0 = q_start[b], t1 = q_start[b + 1];
@@ -55,12 +56,11 @@ __global__ void __launch_bounds__(64 * NW) window_attention_mfma_kernel(
     if (rb0 >= rows_total) return;
     const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6, g4 = lane >> 4, qi = lane & 15;
     const int ns = D / 32, nct = Dv / 16;
-    const int krs = D * 2 + 16;          // row-major key image: bytes per key row
-    constexpr int vts = KT * 2 + 8;      // transposed value image: bytes per value column
-    __shared__ int krow[KT];             // cache row (page * page size + slot) of each key of the tile
-    __shared__ __attribute__((aligned(16))) float kfac[SH ? KT : 4];   // its factor
-    unsigned char* kimg = smem;
-    unsigned char* vimg = smem + KT * krs;
+    constexpr int KCH = NS * 4 + 1, krs = KCH * 16;                     // key row in LDS: 16-byte chunks, bytes
+    constexpr int VCH = SH ? KCH : NCT * 2 + 1, vrs = VCH * 16;         // value row
+    constexpr int BUF = KT * (krs + (SH ? 0 : vrs));                    // one tile
+    __shared__ int krow[2][KT];                                         // cache row of each key of a tile
+    __shared__ __attribute__((aligned(16))) float kfac[2][SH ? KT : 4]; // its factor
     const int r = rb0 + wv * 16 + qi;
     const bool rok = r < rows_total;
     const int rc = rok ? r : rows_total - 1;
@@ -80,6 +80,7 @@ __global__ void __launch_bounds__(64 * NW) window_attention_mfma_kernel(
     const float scale2 = scale * 1.4426950408889634f;
     const int32_t* bt = block_table + (int64_t)b * max_blocks;
     const int kchunks = D / 8, vchunks = Dv / 8;
+    const uint32_t lds0 = lds_offset(smem);
     // the first key any row of the block may see: the window's or the chunk's lower bound of the first row
     const int w_lo = max(window > 0 ? max(0, pmin - window + 1) : 0, chunk > 0 ? pmin / chunk * chunk : 0);
     const int w_start = w_lo / KT * KT;
@@ -93,67 +94,53 @@ __global__ void __launch_bounds__(64 * NW) window_attention_mfma_kernel(
     const int n_pool = (pool > 0 && window > 0) ? max(0, pmax - window + 1) / pool : 0;
     const int n_pool_tiles = (n_pool + KT - 1) / KT;
     const int n_tiles = n_pool_tiles + n_keep_tiles + (pmax - w_start) / KT + 1;
-    for (int tz = split; tz < n_tiles; tz += nsplit) {
-        const bool pooled = tz < n_pool_tiles;   // a tile of pooled pairs: "key" e is block e
+    // where tile tz starts and its last real key (of a tile of pooled pairs: "key" e is block e)
+    auto tile_at = [&](int tz, bool& pooled, bool& kept, int& k0, int& k_last) {
+        pooled = tz < n_pool_tiles;
         const int ti = tz - n_pool_tiles;
-        const bool kept = !pooled && ti < n_keep_tiles;
-        const int k0 = pooled ? tz * KT : kept ? ti * KT : w_start + (ti - n_keep_tiles) * KT;
-        const int k_last = pooled ? n_pool - 1 : kept ? k_end - 1 : pmax;  // last real key this tile may hold
-        const uint16_t* ksrc = pooled ? kp : kc;
-        const uint16_t* vsrc = pooled ? vp : vc;
-        __syncthreads();
-        if (threadIdx.x < KT) {
-            const int key = min(k0 + (int)threadIdx.x, k_last);  // past the end: a real row, masked below
-            const int per = pooled ? EP : BS;
-            krow[threadIdx.x] = (bt[key / per] * per + key % per) * G + kvh;
-            if constexpr (SH) kfac[threadIdx.x] = ks[krow[threadIdx.x]];
-        }
-        __syncthreads();
-        // ---- stage: work item = (key pair jp, 8-element chunk dc); lanes of a wave take consecutive key pairs
-        if constexpr (SH) {
-            for (int it0 = threadIdx.x; it0 < PP * kchunks; it0 += NT * 2) {
-                u16x8 va[2], vb[2];
-#pragma unroll
-                for (int u = 0; u < 2; ++u) {
-                    const int it = it0 + NT * u;
-                    if (it < PP * kchunks) {
-                        const int jp = it & (PP - 1), dc = it / PP;
-                        va[u] = *reinterpret_cast<const u16x8*>(vc + (int64_t)krow[2 * jp] * D + dc * 8);
-                        vb[u] = *reinterpret_cast<const u16x8*>(vc + (int64_t)krow[2 * jp + 1] * D + dc * 8);
-                    }
-                }
-#pragma unroll
-                for (int u = 0; u < 2; ++u) {
-                    const int it = it0 + NT * u;
-                    if (it < PP * kchunks) {
-                        const int jp = it & (PP - 1), dc = it / PP;
-                        *reinterpret_cast<u16x8*>(kimg + (2 * jp) * krs + dc * 16) = va[u];
-                        *reinterpret_cast<u16x8*>(kimg + (2 * jp + 1) * krs + dc * 16) = vb[u];
-#pragma unroll
-                        for (int e = 0; e < 8; ++e)
-                            *reinterpret_cast<uint32_t*>(vimg + (dc * 8 + e) * vts + jp * 4) =
-                                (uint32_t)va[u][e] | ((uint32_t)vb[u][e] << 16);
-                    }
-                }
-            }
-        } else {
-        for (int it = threadIdx.x; it < PP * kchunks; it += NT) {
-            const int jp = it & (PP - 1), dc = it / PP;
-            const u16x8 va = *reinterpret_cast<const u16x8*>(ksrc + (int64_t)krow[2 * jp] * D + dc * 8);
-            const u16x8 vb = *reinterpret_cast<const u16x8*>(ksrc + (int64_t)krow[2 * jp + 1] * D + dc * 8);
-            *reinterpret_cast<u16x8*>(kimg + (2 * jp) * krs + dc * 16) = va;
-            *reinterpret_cast<u16x8*>(kimg + (2 * jp + 1) * krs + dc * 16) = vb;
-        }
-        for (int it = threadIdx.x; it < PP * vchunks; it += NT) {
-            const int jp = it & (PP - 1), dc = it / PP;
-            const u16x8 va = *reinterpret_cast<const u16x8*>(vsrc + (int64_t)krow[2 * jp] * Dv + dc * 8);
-            const u16x8 vb = *reinterpret_cast<const u16x8*>(vsrc + (int64_t)krow[2 * jp + 1] * Dv + dc * 8);
-#pragma unroll
-            for (int e = 0; e < 8; ++e)
-                *reinterpret_cast<uint32_t*>(vimg + (dc * 8 + e) * vts + jp * 4) = (uint32_t)va[e] | ((uint32_t)vb[e] << 16);
-        }
-        }
-        __syncthreads();
+        kept = !pooled && ti < n_keep_tiles;
+        k0 = pooled ? tz * KT : kept ? ti * KT : w_start + (ti - n_keep_tiles) * KT;
+        k_last = pooled ? n_pool - 1 : kept ? k_end - 1 : pmax;
+    };
+    auto row_of = [&](int tz) {   // the cache row of key threadIdx.x of tile tz (past the end: a real row, masked below)
+        bool pooled, kept;
+        int k0, k_last;
+        tile_at(min(tz, n_tiles - 1), pooled, kept, k0, k_last);
+        const int key = min(k0 + (int)threadIdx.x, k_last), per = pooled ? EP : BS;
+        return (bt[key / per] * per + key % per) * G + kvh;
+    };
+    auto stage = [&](int tz, int buf) {
+        const bool pooled = tz < n_pool_tiles;
+        const uint32_t at = lds0 + buf * BUF;
+        for (int j = wv; j < KCH; j += NW) dma_rows<KCH>(pooled ? kp : SH ? vc : kc, krow[buf], D, kchunks, j, at, lane);
+        if constexpr (!SH)
+            for (int j = wv; j < VCH; j += NW) dma_rows<VCH>(pooled ? vp : vc, krow[buf], Dv, vchunks, j, at + KT * krs, lane);
+    };
+    const bool looks = threadIdx.x < KT;    // these threads look the rows up: two tiles ahead, the factors one
+    int row1 = 0;
+    if (looks && split < n_tiles) {
+        const int row0 = row_of(split);
+        krow[0][threadIdx.x] = row0;
+        if constexpr (SH) kfac[0][threadIdx.x] = ks[row0];
+    }
+    __syncthreads();
+    if (split < n_tiles) stage(split, 0);
+    if (looks && split < n_tiles) krow[1][threadIdx.x] = row1 = row_of(split + nsplit);
+    const bool wave_on = rb0 + wv * 16 < rows_total;   // (a wave without rows only helps to stage)
+    int buf = 0;
+    for (int tz = split; tz < n_tiles; tz += nsplit, buf ^= 1) {
+        bool pooled, kept;
+        int k0, k_last;
+        tile_at(tz, pooled, kept, k0, k_last);
+        dma_wait();        // this wave's pieces of the tile have landed
+        __syncthreads();   // ... everyone's; the other buffer's tile has been read by all; its next rows are known
+        if (tz + nsplit < n_tiles) stage(tz + nsplit, buf ^ 1);
+        const int nrow = looks ? row_of(tz + 2 * nsplit) : 0;
+        float nfac = 0.f;
+        if constexpr (SH) nfac = looks ? ks[row1] : 0.f;
+        const unsigned char* kimg = smem + buf * BUF;
+        const unsigned char* vimg = SH ? kimg : kimg + KT * krs;
+        if (wave_on) {
         // ---- scores: 4 key tiles of 16; lane gets keys 16 kt + 4 g4 + i of query row qi
         constexpr int NKT = KT / 16;
         f32x4 S[NKT];
@@ -166,7 +153,7 @@ __global__ void __launch_bounds__(64 * NW) window_attention_mfma_kernel(
                 if (s < ns)
                     S[kt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8*>(arow + s * 64), qf[s],
                                                                     S[kt], 0, 0, 0);
-            if constexpr (SH) S[kt] *= *reinterpret_cast<const f32x4*>(kfac + 16 * kt + 4 * g4);
+            if constexpr (SH) S[kt] *= *reinterpret_cast<const f32x4*>(kfac[buf] + 16 * kt + 4 * g4);
         }
         // scores, maxima and sums live in the base-2 domain (score * scale * log2 e): one multiply and one
         // subtraction in front of the hardware's exp2.  A tile that every row of the block sees whole (the common case
@@ -234,16 +221,21 @@ __global__ void __launch_bounds__(64 * NW) window_attention_mfma_kernel(
         for (int c = 0; c < NCT; ++c) {
             if (c < nct) {
                 O[c] *= corr;
-                const unsigned char* vrow = vimg + (16 * c + qi) * vts + g4 * 8;
+                const unsigned char* vt = vimg + (4 * g4 + (qi >> 2)) * vrs + (qi & 3) * 8 + c * 32;
 #pragma unroll
                 for (int u = 0; u < NU; ++u) {
-                    const bf16x4 lo = *reinterpret_cast<const bf16x4*>(vrow + u * 64);
-                    const bf16x4 hi = *reinterpret_cast<const bf16x4*>(vrow + u * 64 + 32);
+                    const bf16x4 lo = lds_read_tr4(vt + 32 * u * vrs);
+                    const bf16x4 hi = lds_read_tr4(vt + (32 * u + 16) * vrs);
                     const bf16x8 vf = __builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7);
                     O[c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pf[u], O[c], 0, 0, 0);
                     O[c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pl[u], O[c], 0, 0, 0);
                 }
             }
+        }
+        }
+        if (looks) {   // (this tile's rows were last read when it was staged, the next tile's factors' place by the last one)
+            krow[buf][threadIdx.x] = row1 = nrow;
+            if constexpr (SH) kfac[buf ^ 1][threadIdx.x] = nfac;
         }
     }
     if (!rok) return;
@@ -357,7 +349,7 @@ static void wa_mfma_launch(const uint16_t* qkv, int ldq, const uint16_t* kc, con
                            int pool, int EP, const uint16_t* kp, const uint16_t* vp, const float* vcs, int g_off,
                            const float* ks, int64_t ldo, hipStream_t s) {
     auto kern = hy::window_attention_mfma_kernel<NS, NCT, NW, SH>;
-    const int bytes = hy::WKT * (D * 2 + 16) + Dv * (hy::WKT * 2 + 8);
+    constexpr int bytes = 2 * hy::WKT * (NS * 64 + 16 + (SH ? 0 : NCT * 32 + 16));
     static int set_bytes = 0;
     if (bytes > set_bytes) {
         (void)hipFuncSetAttribute(reinterpret_cast<const void*>(kern), hipFuncAttributeMaxDynamicSharedMemorySize, bytes);
