@@ -70,7 +70,7 @@ void launch_hy_window_attention(const void*, int, const void*, const void*, cons
                                 const int32_t*, const float*, const float*, void*, int, int, int, int, int, int, int, float,
                                 int, int, int, bool, int, float*, float*, int64_t, int, int, const void*, const void*, const float*, int,
                                 const float*, int64_t, hipStream_t);
-int hy_window_nsplit(bool, int, int, int, int, int, int, int, int, int, int, int, int);
+int hy_window_nsplit(bool, int, int, int, int, int, int, int, int, int, int, int, int, bool);
 void launch_hy_short_conv(const void*, int, const float*, const float*, const int32_t*, const int32_t*, const int32_t*,
                           const int32_t*, void*, void*, int, int, int, int, bool, bool, hipStream_t);
 void launch_hy_delta_prep(const void*, int, const float*, const float*, float*, float*, float*, float*, int, int, int, int,
@@ -654,7 +654,7 @@ Tensor hy_window_attention(const Tensor& qkv, const c10::optional<Tensor>& kc_in
     const int mq = (int)std::max<int64_t>(1, max_q);
     const int nsplit = chronos::hy_window_nsplit(f32(qkv), (int)qkv.size(1), (int)B, mq, (int)H, (int)G, (int)D, (int)Dv,
                                                  (int)window, (int)keep, (int)chunk, (int)(block_table.size(1) * kc.size(1)),
-                                                 (int)pool);
+                                                 (int)pool, ks.has_value());
     Tensor part_o, part_ml;
     if (nsplit > 1) {
         part_o = at::empty({T * H * nsplit, Dv}, qkv.options().dtype(at::kFloat));

@@ -33,6 +33,11 @@ __device__ __forceinline__ bf16x4 lds_read_tr4(const void* p) {
     return __builtin_amdgcn_ds_read_tr16_b64_v4bf16((lds_bf16x4*)p);
 }
 
+__device__ __forceinline__ f32x4 mfma_16x16x16(bf16x4 a, bf16x4 b, f32x4 c) {
+    typedef short s16x4 __attribute__((ext_vector_type(4)));
+    return __builtin_amdgcn_mfma_f32_16x16x16bf16_1k(__builtin_bit_cast(s16x4, a), __builtin_bit_cast(s16x4, b), c, 0, 0, 0);
+}
+
 // One 1 KiB piece from memory straight into LDS: lane l's 16 bytes from its own address to LDS offset lds + 16 l (lds the
 // same in all lanes).  Inline asm, so that the compiler does not wait for it before every LDS read; the kernel waits with
 // dma_wait() in front of the barrier that hands the piece over.

@@ -1,12 +1,12 @@
 // latent_attention_mfma.hip — the bfloat16 latent attention on the matrix cores (see latent_attention.hip for the
 // math: one cached row per token, key = the whole row, value = its first `rank` columns, shared by all heads).
 //
-// One workgroup takes 64 (token, head) rows of one sequence — 16 per wave, rows are (token * H + head), so any head
-// count tiles the same way — and walks the sequence's keys 64 at a time:
-//   * the key tile goes from memory straight into LDS (no staging registers), row-major [64][DK], two tiles deep: the next
-//     tile is on its way while the current one is computed, one barrier per tile.  Both MFMA operands want 8 k-values per lane — dims for
-//     the scores, KEYS for the weighted sum: the scores read rows as they lie, the sum reads the same image through
-//     gfx950's transposing LDS reads (4 keys of 16 columns each).
+// One workgroup takes up to 128 (token, head) rows of one sequence — 16 per wave, rows are (token * H + head), so any
+// head count tiles the same way — and walks the sequence's keys 64 at a time:
+//   * the key tile goes from memory straight into LDS (no staging registers), row-major [64][DK], two tiles deep: the
+//     next tile is on its way while the current one is computed, one barrier per tile.  Both MFMA operands want 8
+//     k-values per lane — dims for the scores, KEYS for the weighted sum: the scores read rows as they lie, the sum
+//     reads the same image through gfx950's transposing LDS reads (4 keys of 16 columns each).
 //   * scores  S^T = K Q^T : 16x16x32 MFMAs with the key rows as A operand and the wave's 16 query rows (held in
 //     registers for the whole kernel) as B operand, so a lane ends up with 4 keys x 1 query row per 16-key tile;
 //   * softmax in float per query row (lane & 15): causal mask by the row's own position, running maximum and sum,
@@ -18,22 +18,25 @@
 // After the last key a sink per head may join the denominator.
 // With a window a row sees only its last `window` positions: the walk starts at the tile of the first row's first
 // visible key and every row masks by its own position.
-// Sizes: DK % 8 == 0 (the last 32-column step of the scores is zero-filled), rank % 16 == 0, DK <= 576, rank <= 512.
+// Sizes: DK % 8 == 0 (the scores' steps past it are zero), rank % 16 == 0, DK <= 576, rank <= 512.
 // Everything else takes latent_attention.hip.
-#include <cstdlib>
-
 #include "hybrid_common.h"
 
 namespace chronos {
 namespace hy {
 
 constexpr int MKT = 64;  // keys per tile
+constexpr float kLog2e = 1.4426950408889634f;
 
-// NS: k-steps of the scores (DK / 32) at most; NCT: 16-column tiles of the output (rank / 16) at most.
+// NS: k-steps of the scores (DK / 32) at most; NCT: 16-column tiles of the output (rank / 16) at most.  All of them are
+// computed whatever the sizes (a run-time test in front of every product would serialise the loop); the surplus is zero
+// times a real number or never stored.
 // NW: waves per workgroup, 4 or 8 (16 query rows each): with 8 a staged key tile serves 128 rows and every SIMD holds two
 // waves, so one wave's softmax and staging run beside the other's MFMAs.
 // TT: weights as two bfloat16 terms.
-template <int NS, int NCT, int NW, bool TT>
+// KS: waves that share 16 query rows.  With few rows (decode) a tile's keys are dealt to 2 or 4 waves, each with a softmax
+// of its own over its keys (16 keys per wave: 16x16x16 products in the sum), and merged through LDS at the end.
+template <int NS, int NCT, int NW, int KS, bool TT>
 __global__ void __launch_bounds__(64 * NW) latent_attention_mfma_kernel(
         const uint16_t* __restrict__ qa, const uint16_t* __restrict__ cache, const int32_t* __restrict__ block_table,
         int max_blocks, const int32_t* __restrict__ q_start, const int32_t* __restrict__ pos,
@@ -44,15 +47,16 @@ __global__ void __launch_bounds__(64 * NW) latent_attention_mfma_kernel(
     const int b = blockIdx.x;
     const int t0 = q_start[b], t1 = q_start[b + 1];
     const int rows_total = (t1 - t0) * H;
-    constexpr int KT = MKT, RPB = 16 * NW;  // query rows per workgroup
+    constexpr int KT = MKT, RPB = 16 * NW / KS;  // query rows per workgroup
     const int rb0 = blockIdx.y * RPB;
     if (rb0 >= rows_total) return;
     const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6, g = lane >> 4, qi = lane & 15;
-    const int ns = (DK + 31) / 32, nct = rank / 16;
+    const int nct = rank / 16;
     constexpr int CPR = NS * 4 + 1, krs = CPR * 16;   // key row in LDS: 16-byte chunks, bytes
     __shared__ int krow[2][KT];  // cache row (page * page size + slot) of each key of a tile
     // this lane's query row (for the B operand and for the softmax): row r of the sequence, token t0 + r / H
-    const int r = rb0 + wv * 16 + qi;
+    const int kpart = wv % KS;   // which part of a tile's keys this wave takes
+    const int r = rb0 + wv / KS * 16 + qi;
     const bool rok = r < rows_total;
     const int rc = rok ? r : rows_total - 1;
     const int64_t grow = (int64_t)t0 * H + rc;              // row of qa / out / gate
@@ -63,16 +67,16 @@ __global__ void __launch_bounds__(64 * NW) latent_attention_mfma_kernel(
     const int row_lo = window > 0 ? prow - window + 1 : 0;  // the first key this lane's row sees
     bf16x8 qf[NS];
 #pragma unroll
-    for (int s = 0; s < NS; ++s)
-        if (s < ns) {
-            const u16x8 z = {0, 0, 0, 0, 0, 0, 0, 0};
-            qf[s] = 32 * s + 8 * g < DK ? *reinterpret_cast<const bf16x8*>(qa + grow * DK + 32 * s + 8 * g)
-                                        : __builtin_bit_cast(bf16x8, z);
-        }
+    for (int s = 0; s < NS; ++s) {   // columns past the row's end are zero here (and real numbers in the key image)
+        const u16x8 z = {0, 0, 0, 0, 0, 0, 0, 0};
+        qf[s] = 32 * s + 8 * g < DK ? *reinterpret_cast<const bf16x8*>(qa + grow * DK + 32 * s + 8 * g)
+                                    : __builtin_bit_cast(bf16x8, z);
+    }
     f32x4 O[NCT];
 #pragma unroll
     for (int c = 0; c < NCT; ++c) O[c] = f32x4{0.f, 0.f, 0.f, 0.f};
     float mrow = -INFINITY, lrow = 0.f;
+    const float scale2 = scale * kLog2e;   // scores, maxima and sums live in the base-2 domain
     const int32_t* bt = block_table + (int64_t)b * max_blocks;
     const int chunks = DK / 8;
     const uint32_t lds0 = lds_offset(smem);
@@ -91,7 +95,7 @@ __global__ void __launch_bounds__(64 * NW) latent_attention_mfma_kernel(
     __syncthreads();
     if (kfirst <= pmax) stage(0);
     if (threadIdx.x < KT) krow[1][threadIdx.x] = row_of(kfirst + kstep);
-    const bool wave_on = rb0 + wv * 16 < rows_total;   // (a wave without rows only helps to stage)
+    const bool wave_on = rb0 + wv / KS * 16 < rows_total;   // (a wave without rows only helps to stage)
     int buf = 0;
     for (int k0 = kfirst; k0 <= pmax; k0 += kstep, buf ^= 1) {
         dma_wait();        // this wave's pieces of the tile have landed
@@ -101,17 +105,17 @@ __global__ void __launch_bounds__(64 * NW) latent_attention_mfma_kernel(
         const unsigned char* kimg = smem + buf * KT * krs;
         if (wave_on) {
         // ---- scores: KT / 16 key tiles of 16; lane gets keys 16 kt + 4 g + i of query row qi
-        constexpr int NKT = KT / 16;
+        constexpr int NKT = KT / 16 / KS;
+        const int key0 = kpart * (KT / KS);
         f32x4 S[NKT];
 #pragma unroll
         for (int kt = 0; kt < NKT; ++kt) {
             S[kt] = f32x4{0.f, 0.f, 0.f, 0.f};
-            const unsigned char* arow = kimg + (16 * kt + qi) * krs + g * 16;
+            const unsigned char* arow = kimg + (key0 + 16 * kt + qi) * krs + g * 16;
 #pragma unroll
             for (int s = 0; s < NS; ++s)
-                if (s < ns)
-                    S[kt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8*>(arow + s * 64), qf[s],
-                                                                    S[kt], 0, 0, 0);
+                S[kt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8*>(arow + s * 64), qf[s],
+                                                                S[kt], 0, 0, 0);
         }
         // ---- softmax over the tile for query row qi (this lane and the 3 other lane groups hold its keys)
         float mx = -INFINITY;
@@ -119,21 +123,22 @@ __global__ void __launch_bounds__(64 * NW) latent_attention_mfma_kernel(
         for (int kt = 0; kt < NKT; ++kt)
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
-                const int key = k0 + 16 * kt + 4 * g + i;
-                const float sv = key <= prow && key >= row_lo ? S[kt][i] * scale : -INFINITY;
+                const int key = k0 + key0 + 16 * kt + 4 * g + i;
+                const float sv = key <= prow && key >= row_lo ? S[kt][i] * scale2 : -INFINITY;
                 S[kt][i] = sv;
                 mx = fmaxf(mx, sv);
             }
         mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
         mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
         const float mn = fmaxf(mrow, mx);
-        const float corr = (mn == -INFINITY) ? 1.f : __expf(mrow - mn);
+        const float corr = (mn == -INFINITY) ? 1.f : __builtin_amdgcn_exp2f(mrow - mn);
+        const float mref = (mn == -INFINITY) ? 0.f : mn;   // (all masked: every exponent is -inf, every weight 0)
         float sum = 0.f;
 #pragma unroll
         for (int kt = 0; kt < NKT; ++kt)
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
-                const float p = (mn == -INFINITY) ? 0.f : __expf(S[kt][i] - mn);
+                const float p = __builtin_amdgcn_exp2f(S[kt][i] - mref);
                 S[kt][i] = p;
                 sum += p;
             }
@@ -142,8 +147,26 @@ __global__ void __launch_bounds__(64 * NW) latent_attention_mfma_kernel(
         lrow = lrow * corr + sum;
         mrow = mn;
         // ---- weighted sum of the value columns: k index of step u = [tile 2u keys 4g..4g+3 | tile 2u+1 keys 4g..4g+3]
-        constexpr int NU = KT / 32;
-        const unsigned char* vt = kimg + (4 * g + (qi >> 2)) * krs + (qi & 3) * 8;
+        constexpr int NU = NKT / 2;
+        if (__builtin_amdgcn_ballot_w64(corr != 1.f) != 0) {   // (rarely, once the maxima have settled)
+#pragma unroll
+            for (int c = 0; c < NCT; ++c) O[c] *= corr;
+        }
+        const unsigned char* vt = kimg + (key0 + 4 * g + (qi >> 2)) * krs + (qi & 3) * 8;
+        if constexpr (NKT == 1) {
+            bf16x4 pf, pl;
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                pf[e] = (__bf16)S[0][e];
+                if constexpr (TT) pl[e] = (__bf16)(S[0][e] - (float)pf[e]);
+            }
+#pragma unroll
+            for (int c = 0; c < NCT; ++c) {
+                const bf16x4 vf = lds_read_tr4(vt + c * 32);
+                O[c] = mfma_16x16x16(vf, pf, O[c]);
+                if constexpr (TT) O[c] = mfma_16x16x16(vf, pl, O[c]);
+            }
+        }
 #pragma unroll
         for (int u = 0; u < NU; ++u) {
             bf16x8 pf, pl;
@@ -154,18 +177,50 @@ __global__ void __launch_bounds__(64 * NW) latent_attention_mfma_kernel(
                 if constexpr (TT) pl[e] = (__bf16)(w - (float)pf[e]);
             }
 #pragma unroll
-            for (int c = 0; c < NCT; ++c)
-                if (c < nct) {
-                    const bf16x4 lo = lds_read_tr4(vt + 32 * u * krs + c * 32);
-                    const bf16x4 hi = lds_read_tr4(vt + (32 * u + 16) * krs + c * 32);
-                    const bf16x8 vf = __builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7);
-                    if (u == 0) O[c] *= corr;
-                    O[c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pf, O[c], 0, 0, 0);
-                    if constexpr (TT) O[c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pl, O[c], 0, 0, 0);
-                }
+            for (int c = 0; c < NCT; ++c) {
+                const bf16x4 lo = lds_read_tr4(vt + 32 * u * krs + c * 32);
+                const bf16x4 hi = lds_read_tr4(vt + (32 * u + 16) * krs + c * 32);
+                const bf16x8 vf = __builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7);
+                O[c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pf, O[c], 0, 0, 0);
+                if constexpr (TT) O[c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pl, O[c], 0, 0, 0);
+            }
         }
         }
         if (threadIdx.x < KT) krow[buf][threadIdx.x] = nrow;
+    }
+    if constexpr (KS > 1) {   // the waves that share these rows merge their partial results; the first one goes on
+        constexpr int MS = NCT * 16 + 4;    // floats per row (padded)
+        float* mb = reinterpret_cast<float*>(smem);
+        static_assert(NW * 16 * MS * 4 <= 2 * KT * krs, "the partial rows fit the key tiles' LDS");
+        __shared__ float ml[NW][16][2];
+        __syncthreads();                    // everyone is done with the key tiles
+#pragma unroll
+        for (int c = 0; c < NCT; ++c) *reinterpret_cast<f32x4*>(mb + (wv * 16 + qi) * MS + 16 * c + 4 * g) = O[c];
+        if (g == 0) {
+            ml[wv][qi][0] = mrow;
+            ml[wv][qi][1] = lrow;
+        }
+        __syncthreads();
+        if (kpart != 0) return;
+        float mn = mrow, e[KS];
+#pragma unroll
+        for (int k = 1; k < KS; ++k) mn = fmaxf(mn, ml[wv + k][qi][0]);
+        const float mref = mn == -INFINITY ? 0.f : mn;
+        e[0] = exp2f(mrow - mref);
+        lrow *= e[0];
+#pragma unroll
+        for (int k = 1; k < KS; ++k) {
+            e[k] = exp2f(ml[wv + k][qi][0] - mref);
+            lrow += e[k] * ml[wv + k][qi][1];
+        }
+        mrow = mn;
+#pragma unroll
+        for (int c = 0; c < NCT; ++c) {
+            O[c] *= e[0];
+#pragma unroll
+            for (int k = 1; k < KS; ++k)
+                O[c] += e[k] * *reinterpret_cast<const f32x4*>(mb + ((wv + k) * 16 + qi) * MS + 16 * c + 4 * g);
+        }
     }
     if (!rok) return;
     if (nsplit > 1) {  // unnormalised partial: the combine kernel merges the splits
@@ -181,8 +236,8 @@ __global__ void __launch_bounds__(64 * NW) latent_attention_mfma_kernel(
     }
     float f = 1.f / lrow;
     if (sink != nullptr) {   // exp(sink) joins the denominator, without a value
-        const float sk = sink[rc % H], mn = fmaxf(mrow, sk), c = __expf(mrow - mn);
-        f = c / (lrow * c + __expf(sk - mn));
+        const float sk = sink[rc % H] * kLog2e, mn = fmaxf(mrow, sk), c = exp2f(mrow - mn);
+        f = c / (lrow * c + exp2f(sk - mn));
     }
     if (gate != nullptr) f *= sigmoidf_(gate[grow]);
     // lane holds O^T[col = 16 c + 4 g + i][query row qi]
@@ -194,7 +249,8 @@ __global__ void __launch_bounds__(64 * NW) latent_attention_mfma_kernel(
         }
 }
 
-// one wave per (token, head) row: out = sum_z exp(m_z - m) O_z / (sum_z exp(m_z - m) l_z + exp(sink - m)) * sigmoid(gate).  Lane z holds
+// one wave per (token, head) row: out = sum_z 2^(m_z - m) O_z / (sum_z 2^(m_z - m) l_z + 2^(sink log2 e - m)) * sigmoid(gate)
+// (the partial maxima are in the base-2 domain: score * scale * log2 e).  Lane z holds
 // split z's maximum and sum (nsplit <= 16); a lane then sums 4 neighbouring columns over the splits, whose loads do not
 // depend on each other.
 __global__ void __launch_bounds__(256) latent_combine_kernel(const float* __restrict__ part_o, const float* __restrict__ part_ml,
@@ -206,10 +262,10 @@ __global__ void __launch_bounds__(256) latent_combine_kernel(const float* __rest
     if (r >= rows) return;
     const float mz = lane < nsplit ? part_ml[(r * nsplit + lane) * 2] : -INFINITY;
     const float lz = lane < nsplit ? part_ml[(r * nsplit + lane) * 2 + 1] : 0.f;
-    const float sk = sink != nullptr ? sink[r % H] : -INFINITY;
+    const float sk = sink != nullptr ? sink[r % H] * kLog2e : -INFINITY;
     const float m = fmaxf(wave_max(mz), sk);
-    float e = mz == -INFINITY ? 0.f : expf(mz - m);   // (a split without a visible key adds nothing)
-    const float l = wave_sum(e * lz) + (sink != nullptr ? expf(sk - m) : 0.f);
+    float e = mz == -INFINITY ? 0.f : exp2f(mz - m);   // (a split without a visible key adds nothing)
+    const float l = wave_sum(e * lz) + (sink != nullptr ? exp2f(sk - m) : 0.f);
     e *= (gate != nullptr ? sigmoidf_(gate[r]) : 1.f) / l;
     for (int c = lane * 4; c < rank; c += 256) {      // (rank is a multiple of 16)
         f32x4 acc = {0.f, 0.f, 0.f, 0.f};
@@ -224,19 +280,19 @@ __global__ void __launch_bounds__(256) latent_combine_kernel(const float* __rest
 
 }  // namespace hy
 
-template <int NS, int NCT, int NW, bool TT>
+template <int NS, int NCT, int NW, int KS, bool TT>
 static void la_mfma_launch(const uint16_t* qa, const uint16_t* cache, const int32_t* bt, int max_blocks,
                            const int32_t* q_start, const int32_t* pos, const float* gate, uint16_t* out, int B, int H,
                            int DK, int rank, int BS, int max_q, float scale, int window, int nsplit, float* part_o,
                            float* part_ml, const float* sink, hipStream_t s) {
-    auto kern = hy::latent_attention_mfma_kernel<NS, NCT, NW, TT>;
+    auto kern = hy::latent_attention_mfma_kernel<NS, NCT, NW, KS, TT>;
     constexpr int bytes = 2 * hy::MKT * (NS * 64 + 16);
     static int set_bytes = 0;
     if (bytes > set_bytes) {
         (void)hipFuncSetAttribute(reinterpret_cast<const void*>(kern), hipFuncAttributeMaxDynamicSharedMemorySize, bytes);
         set_bytes = bytes;
     }
-    const dim3 grid(B, (max_q * H + 16 * NW - 1) / (16 * NW), nsplit);
+    const dim3 grid(B, (max_q * H + 16 * NW / KS - 1) / (16 * NW / KS), nsplit);
     const int bs_shift = (BS & (BS - 1)) == 0 ? __builtin_ctz(BS) : -1;
     kern<<<grid, 64 * NW, bytes, s>>>(qa, cache, bt, max_blocks, q_start, pos, gate, out, H, DK, rank, BS, scale, window,
                                   nsplit, part_o, part_ml, bs_shift, sink);
@@ -264,19 +320,26 @@ bool launch_hy_latent_attention_mfma(const uint16_t* qa, const uint16_t* cache, 
                                      hipStream_t s) {
     if (!hy_latent_mfma_ok(DK, rank)) return false;
     if (B == 0 || max_q == 0) return true;
-#define HY_LAM(NS, NCT, NW, TT) la_mfma_launch<NS, NCT, NW, TT>(qa, cache, bt, max_blocks, q_start, pos, gate, out, B, H, DK, rank, BS, max_q, scale, window, nsplit, part_o, part_ml, sink, s)
-    // 8 waves per workgroup when a sequence brings more than 64 rows (CHRONOS_LATENT_NW=4 / 8 forces one)
-    static const int force_nw = [] { const char* v = getenv("CHRONOS_LATENT_NW"); return v ? atoi(v) : 0; }();
-    const bool nw8 = force_nw == 8 || (force_nw != 4 && max_q * H > 64);
-#define HY_LAM_T(NS, NCT)                                                            \
-    do {                                                                             \
-        if (two_term) { if (nw8) HY_LAM(NS, NCT, 8, true); else HY_LAM(NS, NCT, 4, true); }   \
-        else { if (nw8) HY_LAM(NS, NCT, 8, false); else HY_LAM(NS, NCT, 4, false); }          \
+#define HY_LAM(NS, NCT, NW, KS, TT) la_mfma_launch<NS, NCT, NW, KS, TT>(qa, cache, bt, max_blocks, q_start, pos, gate, out, B, H, DK, rank, BS, max_q, scale, window, nsplit, part_o, part_ml, sink, s)
+    // 8 waves per workgroup when a sequence brings more than 64 rows; up to 32 or 16 rows 2 or 4 waves share them
+    const int rows = max_q * H;
+#define HY_LAM_R(NS, NCT, TT)                             \
+    do {                                                  \
+        if (rows > 64) HY_LAM(NS, NCT, 8, 1, TT);         \
+        else if (rows > 32) HY_LAM(NS, NCT, 4, 1, TT);    \
+        else if (rows > 16) HY_LAM(NS, NCT, 4, 2, TT);    \
+        else HY_LAM(NS, NCT, 4, 4, TT);                   \
+    } while (0)
+#define HY_LAM_T(NS, NCT)                                                                       \
+    do {                                                                                        \
+        if (two_term) HY_LAM_R(NS, NCT, true); else HY_LAM_R(NS, NCT, false);                   \
     } while (0)
     if (DK <= 128 && rank <= 64) HY_LAM_T(4, 4);
+    else if (DK <= 192 && rank <= 128) HY_LAM_T(6, 8);
     else if (DK <= 320 && rank <= 256) HY_LAM_T(10, 16);
     else HY_LAM_T(18, 32);
 #undef HY_LAM_T
+#undef HY_LAM_R
 #undef HY_LAM
     if (nsplit > 1)
         hy::latent_combine_kernel<<<(unsigned)((total_rows + 3) / 4), 256, 0, s>>>(part_o, part_ml, gate, out, total_rows, rank, nsplit, sink, H);

@@ -7,9 +7,9 @@
 // kept first tokens that lie below the window's first tile, then the tiles from the window's first key to the last
 // query.  Per tile:
 //   * keys and values go from memory straight into LDS (no staging registers), row-major [64][D] and [64][Dv], two tiles
-//     deep: the next tile is on its way while the current one is computed, one barrier per tile.  Both MFMA operands want 8 k-values per lane —
-//     dims for the scores, KEYS for the sum: the sum reads the values through gfx950's transposing LDS reads (4 keys of
-//     16 columns each);
+//     deep: the next tile is on its way while the current one is computed, one barrier per tile.  Both MFMA operands want
+//     8 k-values per lane — dims for the scores, KEYS for the sum: the sum reads the values through gfx950's transposing
+//     LDS reads (4 keys of 16 columns each);
 //   * scores  S^T = K Q^T : 16x16x32 MFMAs, key rows as A operand, the wave's 16 query rows (in registers for the
 //     whole kernel) as B operand: a lane ends up with 4 keys x 1 query row per 16-key tile;
 //   * softmax in float per query row (lane & 15): each row masks by its own position (causal, window, kept tokens),
@@ -21,12 +21,12 @@
 // may follow in the same epilogue: with a rotation table for the values, the head's output row is turned BACK by the
 // query's position (column m pairs with m + Dv / 2; a lane holds both when Dv % 32 == 0: accumulator tile c and tile
 // c + Dv / 32), and with a gate per output column the row is multiplied by sigmoid of the gate columns of the
-// query's own projection row.  Launches of few
-// rows (decode) deal a row block's key tiles to several workgroups and merge the float partials in a second kernel.
+// query's own projection row.  Launches of few rows (decode) deal a row block's key tiles to several workgroups and
+// merge the float partials in a second kernel.
 // With unit keys (SH: a key is the cached value times a float factor) the one image serves both products, and a score is
 // multiplied by its key's factor.
 // With chunk > 0 a row also hides the keys below its own chunk of positions (key >= floor(pos / chunk) * chunk).
-// Sizes: D % 32 == 0, Dv % 16 == 0, D <= 256, Dv <= 256.  Everything else takes the general kernel.
+// Sizes: D % 8 == 0, Dv % 16 == 0, D <= 256, Dv <= 256.  Everything else takes the general kernel.
 #include <algorithm>
 
 #include "hybrid_common.h"
@@ -36,7 +36,12 @@ namespace hy {
 
 constexpr int WKT = 64;  // keys per tile
 
-template <int NS, int NCT, int NW, bool SH>
+// NS: k-steps of the scores (D / 32) at most; NCT: 16-column tiles of the output (Dv / 16) at most.  All of them are
+// computed whatever the sizes (a run-time test in front of every product would serialise the loop); the surplus is zero
+// times a real number or never stored.  NW: waves per workgroup.
+// KS: waves that share 16 query rows.  With few rows (decode) a tile's keys are dealt to 2 or 4 waves, each with a softmax
+// of its own over its keys (16 keys per wave: 16x16x16 products in the sum), and merged through LDS at the end.
+template <int NS, int NCT, int NW, int KS, bool SH>
 __global__ void __launch_bounds__(64 * NW) window_attention_mfma_kernel(
         const uint16_t* __restrict__ qkv, int ldq, const uint16_t* __restrict__ kc, const uint16_t* __restrict__ vc,
         const int32_t* __restrict__ block_table, int max_blocks, const int32_t* __restrict__ q_start,
@@ -46,7 +51,7 @@ __global__ void __launch_bounds__(64 * NW) window_attention_mfma_kernel(
         const uint16_t* __restrict__ kp, const uint16_t* __restrict__ vp, const float* __restrict__ vcs, int g_off,
         const float* __restrict__ ks, int64_t ldo) {
     extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
-    constexpr int KT = WKT, RPB = 16 * NW;
+    constexpr int KT = WKT, RPB = 16 * NW / KS;
     const int R = H / G;
     const int b = blockIdx.x, kvh = blockIdx.z;
     const int t0 = q_start[b], t1 = q_start[b + 1];
@@ -55,13 +60,14 @@ __global__ void __launch_bounds__(64 * NW) window_attention_mfma_kernel(
     const int rb0 = blockIdx.y / nsplit * RPB;
     if (rb0 >= rows_total) return;
     const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6, g4 = lane >> 4, qi = lane & 15;
-    const int ns = D / 32, nct = Dv / 16;
+    const int nct = Dv / 16;
     constexpr int KCH = NS * 4 + 1, krs = KCH * 16;                     // key row in LDS: 16-byte chunks, bytes
     constexpr int VCH = SH ? KCH : NCT * 2 + 1, vrs = VCH * 16;         // value row
     constexpr int BUF = KT * (krs + (SH ? 0 : vrs));                    // one tile
     __shared__ int krow[2][KT];                                         // cache row of each key of a tile
-    __shared__ __attribute__((aligned(16))) float kfac[2][SH ? KT : 4]; // its factor
-    const int r = rb0 + wv * 16 + qi;
+    __shared__ __attribute__((aligned(16))) float kfac[2][SH ? KT : 4]; // its factor, times the score scale
+    const int kpart = wv % KS;   // which part of a tile's keys this wave takes
+    const int r = rb0 + wv / KS * 16 + qi;
     const bool rok = r < rows_total;
     const int rc = rok ? r : rows_total - 1;
     const int64_t tok = t0 + rc / R;
@@ -71,8 +77,11 @@ __global__ void __launch_bounds__(64 * NW) window_attention_mfma_kernel(
     const int pmin = pos[t0 + rb0 / R], pmax = pos[t0 + last_row / R];  // positions grow along the sequence
     bf16x8 qf[NS];
 #pragma unroll
-    for (int s = 0; s < NS; ++s)
-        if (s < ns) qf[s] = *reinterpret_cast<const bf16x8*>(qkv + tok * ldq + head * D + 32 * s + 8 * g4);
+    for (int s = 0; s < NS; ++s) {   // columns past the head's end are zero here (and real numbers in the key image)
+        const u16x8 z = {0, 0, 0, 0, 0, 0, 0, 0};
+        qf[s] = 32 * s + 8 * g4 < D ? *reinterpret_cast<const bf16x8*>(qkv + tok * ldq + head * D + 32 * s + 8 * g4)
+                                    : __builtin_bit_cast(bf16x8, z);
+    }
     f32x4 O[NCT];
 #pragma unroll
     for (int c = 0; c < NCT; ++c) O[c] = f32x4{0.f, 0.f, 0.f, 0.f};
@@ -121,12 +130,12 @@ __global__ void __launch_bounds__(64 * NW) window_attention_mfma_kernel(
     if (looks && split < n_tiles) {
         const int row0 = row_of(split);
         krow[0][threadIdx.x] = row0;
-        if constexpr (SH) kfac[0][threadIdx.x] = ks[row0];
+        if constexpr (SH) kfac[0][threadIdx.x] = ks[row0] * scale2;
     }
     __syncthreads();
     if (split < n_tiles) stage(split, 0);
     if (looks && split < n_tiles) krow[1][threadIdx.x] = row1 = row_of(split + nsplit);
-    const bool wave_on = rb0 + wv * 16 < rows_total;   // (a wave without rows only helps to stage)
+    const bool wave_on = rb0 + wv / KS * 16 < rows_total;   // (a wave without rows only helps to stage)
     int buf = 0;
     for (int tz = split; tz < n_tiles; tz += nsplit, buf ^= 1) {
         bool pooled, kept;
@@ -137,27 +146,28 @@ __global__ void __launch_bounds__(64 * NW) window_attention_mfma_kernel(
         if (tz + nsplit < n_tiles) stage(tz + nsplit, buf ^ 1);
         const int nrow = looks ? row_of(tz + 2 * nsplit) : 0;
         float nfac = 0.f;
-        if constexpr (SH) nfac = looks ? ks[row1] : 0.f;
+        if constexpr (SH) nfac = looks ? ks[row1] * scale2 : 0.f;
         const unsigned char* kimg = smem + buf * BUF;
         const unsigned char* vimg = SH ? kimg : kimg + KT * krs;
         if (wave_on) {
         // ---- scores: 4 key tiles of 16; lane gets keys 16 kt + 4 g4 + i of query row qi
-        constexpr int NKT = KT / 16;
+        constexpr int NKT = KT / 16 / KS;
+        const int key0 = kpart * (KT / KS);
         f32x4 S[NKT];
 #pragma unroll
         for (int kt = 0; kt < NKT; ++kt) {
             S[kt] = f32x4{0.f, 0.f, 0.f, 0.f};
-            const unsigned char* arow = kimg + (16 * kt + qi) * krs + g4 * 16;
+            const unsigned char* arow = kimg + (key0 + 16 * kt + qi) * krs + g4 * 16;
 #pragma unroll
             for (int s = 0; s < NS; ++s)
-                if (s < ns)
-                    S[kt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8*>(arow + s * 64), qf[s],
-                                                                    S[kt], 0, 0, 0);
-            if constexpr (SH) S[kt] *= *reinterpret_cast<const f32x4*>(kfac[buf] + 16 * kt + 4 * g4);
+                S[kt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8*>(arow + s * 64), qf[s],
+                                                                S[kt], 0, 0, 0);
+            if constexpr (SH) S[kt] *= *reinterpret_cast<const f32x4*>(kfac[buf] + key0 + 16 * kt + 4 * g4);
+            else S[kt] *= scale2;
         }
-        // scores, maxima and sums live in the base-2 domain (score * scale * log2 e): one multiply and one
-        // subtraction in front of the hardware's exp2.  A tile that every row of the block sees whole (the common case
-        // inside a window) skips the per-key visibility tests.
+        // scores, maxima and sums live in the base-2 domain (score * scale * log2 e): one multiply (with unit keys the
+        // factor carries it) and one subtraction in front of the hardware's exp2.  A tile that every row of the block
+        // sees whole (the common case) skips the per-key visibility tests.
         const bool whole = pooled ? (k0 + KT - 1 <= k_last && (k0 + KT) * pool - 1 + window <= pmin)
                                   : (k0 + KT - 1 <= min(k_last, pmin) && (window <= 0 || kept || pmax - k0 < window) &&
                                      k0 >= c_lo_max);
@@ -166,20 +176,17 @@ __global__ void __launch_bounds__(64 * NW) window_attention_mfma_kernel(
 #pragma unroll
             for (int kt = 0; kt < NKT; ++kt)
 #pragma unroll
-                for (int i = 0; i < 4; ++i) {
-                    S[kt][i] *= scale2;
-                    mx = fmaxf(mx, S[kt][i]);
-                }
+                for (int i = 0; i < 4; ++i) mx = fmaxf(mx, S[kt][i]);
         } else {
 #pragma unroll
             for (int kt = 0; kt < NKT; ++kt)
 #pragma unroll
                 for (int i = 0; i < 4; ++i) {
-                    const int key = k0 + 16 * kt + 4 * g4 + i;
+                    const int key = k0 + key0 + 16 * kt + 4 * g4 + i;
                     const bool vis = pooled ? (key <= k_last && (key + 1) * pool - 1 + window <= prow)
                                             : (key <= k_last && key <= prow &&
                                                (window <= 0 || prow - key < window || key < keep) && key >= c_lo);
-                    const float sv = vis ? S[kt][i] * scale2 : -INFINITY;
+                    const float sv = vis ? S[kt][i] : -INFINITY;
                     S[kt][i] = sv;
                     mx = fmaxf(mx, sv);
                 }
@@ -203,39 +210,84 @@ __global__ void __launch_bounds__(64 * NW) window_attention_mfma_kernel(
         lrow = lrow * corr + sum;
         mrow = mn;
         // ---- weighted sum of the values: k index of step u = [tile 2u keys 4g4..4g4+3 | tile 2u+1 keys 4g4..4g4+3]
-        constexpr int NU = KT / 32;
+        constexpr int NU = NKT / 2;
         // the float weights enter the MFMA as a sum of two bfloat16 terms (the rounded weight and the rounding's
         // remainder), so the weighted sum sees them to about 2^-17 instead of 2^-9
-        bf16x8 pf[NU], pl[NU];
+        if (__builtin_amdgcn_ballot_w64(corr != 1.f) != 0) {   // (rarely, once the maxima have settled)
 #pragma unroll
-        for (int u = 0; u < NU; ++u) {
+            for (int c = 0; c < NCT; ++c) O[c] *= corr;
+        }
+        const unsigned char* vt = vimg + (key0 + 4 * g4 + (qi >> 2)) * vrs + (qi & 3) * 8;
+        if constexpr (NKT == 1) {
+            bf16x4 pf, pl;
 #pragma unroll
-            for (int e = 0; e < 8; ++e) {
-                const float w = S[2 * u + (e >> 2)][e & 3];
-                const __bf16 hi = (__bf16)w;
-                pf[u][e] = hi;
-                pl[u][e] = (__bf16)(w - (float)hi);
+            for (int e = 0; e < 4; ++e) {
+                pf[e] = (__bf16)S[0][e];
+                pl[e] = (__bf16)(S[0][e] - (float)pf[e]);
+            }
+#pragma unroll
+            for (int c = 0; c < NCT; ++c) {
+                const bf16x4 vf = lds_read_tr4(vt + c * 32);
+                O[c] = mfma_16x16x16(vf, pf, O[c]);
+                O[c] = mfma_16x16x16(vf, pl, O[c]);
             }
         }
 #pragma unroll
-        for (int c = 0; c < NCT; ++c) {
-            if (c < nct) {
-                O[c] *= corr;
-                const unsigned char* vt = vimg + (4 * g4 + (qi >> 2)) * vrs + (qi & 3) * 8 + c * 32;
+        for (int u = 0; u < NU; ++u) {
+            bf16x8 pf, pl;
 #pragma unroll
-                for (int u = 0; u < NU; ++u) {
-                    const bf16x4 lo = lds_read_tr4(vt + 32 * u * vrs);
-                    const bf16x4 hi = lds_read_tr4(vt + (32 * u + 16) * vrs);
-                    const bf16x8 vf = __builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7);
-                    O[c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pf[u], O[c], 0, 0, 0);
-                    O[c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pl[u], O[c], 0, 0, 0);
-                }
+            for (int e = 0; e < 8; ++e) {
+                const float w = S[2 * u + (e >> 2)][e & 3];
+                pf[e] = (__bf16)w;
+                pl[e] = (__bf16)(w - (float)pf[e]);
+            }
+#pragma unroll
+            for (int c = 0; c < NCT; ++c) {
+                const bf16x4 lo = lds_read_tr4(vt + 32 * u * vrs + c * 32);
+                const bf16x4 hi = lds_read_tr4(vt + (32 * u + 16) * vrs + c * 32);
+                const bf16x8 vf = __builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7);
+                O[c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pf, O[c], 0, 0, 0);
+                O[c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pl, O[c], 0, 0, 0);
             }
         }
         }
         if (looks) {   // (this tile's rows were last read when it was staged, the next tile's factors' place by the last one)
             krow[buf][threadIdx.x] = row1 = nrow;
             if constexpr (SH) kfac[buf ^ 1][threadIdx.x] = nfac;
+        }
+    }
+    if constexpr (KS > 1) {   // the waves that share these rows merge their partial results; the first one goes on
+        constexpr int MS = NCT * 16 + 4;    // floats per row (padded)
+        float* mb = reinterpret_cast<float*>(smem);
+        static_assert(NW * 16 * MS * 4 <= 2 * BUF, "the partial rows fit the key tiles' LDS");
+        __shared__ float ml[NW][16][2];
+        __syncthreads();                    // everyone is done with the key tiles
+#pragma unroll
+        for (int c = 0; c < NCT; ++c) *reinterpret_cast<f32x4*>(mb + (wv * 16 + qi) * MS + 16 * c + 4 * g4) = O[c];
+        if (g4 == 0) {
+            ml[wv][qi][0] = mrow;
+            ml[wv][qi][1] = lrow;
+        }
+        __syncthreads();
+        if (kpart != 0) return;
+        float mn = mrow, e[KS];
+#pragma unroll
+        for (int k = 1; k < KS; ++k) mn = fmaxf(mn, ml[wv + k][qi][0]);
+        const float mref = mn == -INFINITY ? 0.f : mn;
+        e[0] = exp2f(mrow - mref);
+        lrow *= e[0];
+#pragma unroll
+        for (int k = 1; k < KS; ++k) {
+            e[k] = exp2f(ml[wv + k][qi][0] - mref);
+            lrow += e[k] * ml[wv + k][qi][1];
+        }
+        mrow = mn;
+#pragma unroll
+        for (int c = 0; c < NCT; ++c) {
+            O[c] *= e[0];
+#pragma unroll
+            for (int k = 1; k < KS; ++k)
+                O[c] += e[k] * *reinterpret_cast<const f32x4*>(mb + ((wv + k) * 16 + qi) * MS + 16 * c + 4 * g4);
         }
     }
     if (!rok) return;
@@ -294,89 +346,104 @@ __global__ void __launch_bounds__(64 * NW) window_attention_mfma_kernel(
 }
 
 // one wave per (token, head) row: out = sum_z 2^(m_z - m) O_z / (sum_z 2^(m_z - m) l_z + 2^(sink log2 e - m)) * sigmoid(gate),
-// then (with a table) turned back by the row's position and (with gate columns) times sigmoid of them
+// then (with a table) turned back by the row's position and (with gate columns) times sigmoid of them.  Lane z holds split
+// z's maximum and sum (nsplit <= 64); a lane then sums 4 neighbouring columns over the splits, whose loads do not depend
+// on each other (rows up to 128 wide: half the lanes the even splits, half the odd ones).
 __global__ void __launch_bounds__(256) window_combine_kernel(const float* __restrict__ part_o, const float* __restrict__ part_ml,
                                                              const float* __restrict__ sink, const float* __restrict__ gate,
                                                              uint16_t* __restrict__ out, int64_t rows, int H, int Dv,
                                                              int nsplit, const float* __restrict__ vcs,
                                                              const int32_t* __restrict__ pos, const uint16_t* __restrict__ qkv,
                                                              int ldq, int g_off, int64_t ldo) {
-    const int lane = threadIdx.x & 63;
-    const int64_t r = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
-    if (r >= rows) return;
+    __shared__ float rowbuf[4][256];
+    const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6;
+    const int64_t r = (int64_t)blockIdx.x * 4 + wv;
+    if (r >= rows) return;   // (whole waves; a wave's row of rowbuf is its own)
     // (the partial maxima are in the base-2 domain: score * scale * log2 e)
+    const float mz = lane < nsplit ? part_ml[(r * nsplit + lane) * 2] : -INFINITY;
+    const float lz = lane < nsplit ? part_ml[(r * nsplit + lane) * 2 + 1] : 0.f;
     const float sk = sink != nullptr ? sink[r % H] * 1.4426950408889634f : -INFINITY;
-    float m = sk;
-    for (int z = 0; z < nsplit; ++z) m = fmaxf(m, part_ml[(r * nsplit + z) * 2]);
-    float l = sink != nullptr ? exp2f(sk - m) : 0.f;
-    for (int z = 0; z < nsplit; ++z) {
-        const float mz = part_ml[(r * nsplit + z) * 2];
-        if (mz != -INFINITY) l += exp2f(mz - m) * part_ml[(r * nsplit + z) * 2 + 1];
+    const float m = fmaxf(wave_max(mz), sk);
+    float e = mz == -INFINITY ? 0.f : exp2f(mz - m);   // (a split without a visible key adds nothing)
+    const float l = wave_sum(e * lz) + (sink != nullptr ? exp2f(sk - m) : 0.f);
+    e *= l > 0.f ? (gate != nullptr ? sigmoidf_(gate[r]) : 1.f) / l : 0.f;
+    const bool two = Dv <= 128;
+    const int step = two ? 2 : 1, half = two ? lane >> 5 : 0, c = (two ? lane & 31 : lane) * 4;
+    f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+    const float* po = part_o + r * nsplit * Dv + min(c, Dv - 4);
+#pragma unroll 4
+    for (int z = half; z < nsplit + (step - 1 - half); z += step) {   // both halves take the same number of steps
+        const float w = z < nsplit ? __shfl(e, z, 64) : 0.f;
+        if (w != 0.f) acc += w * *reinterpret_cast<const f32x4*>(po + (int64_t)z * Dv);
     }
-    float f = l > 0.f ? 1.f / l : 0.f;
-    if (gate != nullptr) f *= sigmoidf_(gate[r]);
-    auto col = [&](int c) {
-        float acc = 0.f;
-        for (int z = 0; z < nsplit; ++z) {
-            const float mz = part_ml[(r * nsplit + z) * 2];
-            if (mz != -INFINITY) acc += exp2f(mz - m) * part_o[(r * nsplit + z) * Dv + c];
-        }
-        return acc * f;
-    };
+    if (two) {
+#pragma unroll
+        for (int i = 0; i < 4; ++i) acc[i] += __shfl_xor(acc[i], 32, 64);
+    }
     const uint16_t* gsrc = g_off >= 0 ? qkv + (r / H) * ldq + g_off + (r % H) * Dv : nullptr;
     uint16_t* orow = out + (r / H) * ldo + (r % H) * Dv;
-    auto wide = [&](int c) { return gsrc != nullptr ? sigmoidf_(bf2f(gsrc[c])) : 1.f; };
-    if (vcs == nullptr) {
-        for (int c = lane; c < Dv; c += 64) orow[c] = f2bf(col(c) * wide(c));
+    if (vcs == nullptr && gsrc == nullptr) {
+        if (half == 0 && c < Dv)
+            *reinterpret_cast<u16x4*>(orow + c) = u16x4{f2bf(acc[0]), f2bf(acc[1]), f2bf(acc[2]), f2bf(acc[3])};
         return;
     }
-    const int half = Dv / 2;
+    float* row = rowbuf[wv];
+    if (half == 0 && c < Dv) *reinterpret_cast<f32x4*>(row + c) = acc;
+    __builtin_amdgcn_wave_barrier();   // the wave's row is in LDS before any lane reads it
+    auto wide = [&](int k) { return gsrc != nullptr ? sigmoidf_(bf2f(gsrc[k])) : 1.f; };
+    if (vcs == nullptr) {
+        for (int k = lane; k < Dv; k += 64) orow[k] = f2bf(row[k] * wide(k));
+        return;
+    }
+    const int hv = Dv / 2;
     const float* cs = vcs + (int64_t)pos[r / H] * Dv;
-    for (int c = lane; c < half; c += 64) {
-        const float a = col(c), b = col(c + half), co = cs[c], si = cs[half + c];
-        orow[c] = f2bf((a * co + b * si) * wide(c));
-        orow[c + half] = f2bf((b * co - a * si) * wide(c + half));
+    for (int k = lane; k < hv; k += 64) {
+        const float a = row[k], b = row[k + hv], co = cs[k], si = cs[hv + k];
+        orow[k] = f2bf((a * co + b * si) * wide(k));
+        orow[k + hv] = f2bf((b * co - a * si) * wide(k + hv));
     }
 }
 
 }  // namespace hy
 
-template <int NS, int NCT, int NW, bool SH>
+template <int NS, int NCT, int NW, int KS, bool SH>
 static void wa_mfma_launch(const uint16_t* qkv, int ldq, const uint16_t* kc, const uint16_t* vc, const int32_t* bt,
                            int max_blocks, const int32_t* q_start, const int32_t* pos, const float* sink,
                            const float* gate, uint16_t* out, int B, int max_q, int H, int G, int D, int Dv, int BS,
                            float scale, int window, int keep, int chunk, int nsplit, float* part_o, float* part_ml,
                            int pool, int EP, const uint16_t* kp, const uint16_t* vp, const float* vcs, int g_off,
                            const float* ks, int64_t ldo, hipStream_t s) {
-    auto kern = hy::window_attention_mfma_kernel<NS, NCT, NW, SH>;
+    auto kern = hy::window_attention_mfma_kernel<NS, NCT, NW, KS, SH>;
     constexpr int bytes = 2 * hy::WKT * (NS * 64 + 16 + (SH ? 0 : NCT * 32 + 16));
     static int set_bytes = 0;
     if (bytes > set_bytes) {
         (void)hipFuncSetAttribute(reinterpret_cast<const void*>(kern), hipFuncAttributeMaxDynamicSharedMemorySize, bytes);
         set_bytes = bytes;
     }
-    const dim3 grid(B, (max_q * (H / G) + 16 * NW - 1) / (16 * NW) * nsplit, G);
+    const dim3 grid(B, (max_q * (H / G) + 16 * NW / KS - 1) / (16 * NW / KS) * nsplit, G);
     kern<<<grid, 64 * NW, bytes, s>>>(qkv, ldq, kc, vc, bt, max_blocks, q_start, pos, sink, gate, out, H, G, D, Dv, BS, scale,
                                       window, keep, chunk, nsplit, part_o, part_ml, pool, EP, kp, vp, vcs, g_off, ks, ldo);
 }
 
-bool hy_window_mfma_ok(int ldq, int D, int Dv) { return !(D % 32 || Dv % 16 || D > 256 || Dv > 256 || ldq % 8); }
+bool hy_window_mfma_ok(int ldq, int D, int Dv) { return !(D % 8 || Dv % 16 || D > 256 || Dv > 256 || ldq % 8); }
 
 // Splits of a row block's key tiles over workgroups (merged by a combine kernel) for launches that would leave most
-// of the chip idle — decode rows, a lone short portion: enough workgroups to cover the CUs four times, at least 2 key
-// tiles per split, at most 16.  The tile count follows from sizes the host knows (the window, or the block table's
-// width when there is none).  1 for float32 and sizes the matrix-core kernel does not serve.
+// of the chip idle — decode rows, a lone short portion: enough workgroups to cover the CUs twice (four times for few
+// rows with unit keys, whose workgroups need half the LDS), at least 2 key tiles per split, at most 16.  The tile count
+// follows from sizes the host knows (the window, or the block table's width when there is none).  1 for float32 and
+// sizes the matrix-core kernel does not serve.
 int hy_window_nsplit(bool f32, int ldq, int B, int max_q, int H, int G, int D, int Dv, int window, int keep, int chunk,
-                     int max_ctx, int pool) {
+                     int max_ctx, int pool, bool unit) {
     if (f32 || !hy_window_mfma_ok(ldq, D, Dv) || B <= 0) return 1;
     const int rows = max_q * (H / G);
     const int wgs = B * ((rows + (rows > 64 ? 127 : 63)) / (rows > 64 ? 128 : 64)) * G;
-    if (wgs >= 512) return 1;
+    const int enough = unit && rows <= 64 ? 1024 : 512;
+    if (wgs >= enough) return 1;
     int span = window > 0 ? std::min(max_ctx, window + max_q) : max_ctx;
     if (chunk > 0) span = std::min(span, chunk + max_q);   // a row block's keys start in its first row's chunk
     const int tiles = span / hy::WKT + 1 + (window > 0 ? (std::min(keep, max_ctx) + hy::WKT - 1) / hy::WKT : 0) +
                       (window > 0 && pool > 0 ? (max_ctx / pool + hy::WKT - 1) / hy::WKT : 0);
-    int want = (1024 + wgs - 1) / wgs;
+    int want = (enough + wgs - 1) / wgs;
     want = std::min(want, std::min(16, tiles / 2));
     return want < 1 ? 1 : want;
 }
@@ -394,14 +461,23 @@ bool launch_hy_window_attention_mfma(const uint16_t* qkv, int ldq, const uint16_
                                      int64_t ldo, hipStream_t s) {
     if (!hy_window_mfma_ok(ldq, D, Dv) || ldo % 4) return false;
     if (B == 0 || max_q == 0) return true;
-#define HY_WAM_S(NS, NCT, NW, SH) wa_mfma_launch<NS, NCT, NW, SH>(qkv, ldq, kc, vc, bt, max_blocks, q_start, pos, sink, gate, out, B, max_q, H, G, D, Dv, BS, scale, window, keep, chunk, nsplit, part_o, part_ml, pool, EP, kp, vp, vcs, g_off, ks, ldo, s)
-#define HY_WAM(NS, NCT, NW) do { if (ks != nullptr) HY_WAM_S(NS, NCT, NW, true); else HY_WAM_S(NS, NCT, NW, false); } while (0)
+#define HY_WAM_S(NS, NCT, NW, KS, SH) wa_mfma_launch<NS, NCT, NW, KS, SH>(qkv, ldq, kc, vc, bt, max_blocks, q_start, pos, sink, gate, out, B, max_q, H, G, D, Dv, BS, scale, window, keep, chunk, nsplit, part_o, part_ml, pool, EP, kp, vp, vcs, g_off, ks, ldo, s)
+#define HY_WAM_K(NS, NCT, NW, KS) do { if (ks != nullptr) HY_WAM_S(NS, NCT, NW, KS, true); else HY_WAM_S(NS, NCT, NW, KS, false); } while (0)
     // 8 waves per workgroup when a sequence brings more than 64 rows per key/value head: a staged tile then serves
-    // 128 rows and every SIMD holds two waves
-    const bool nw8 = max_q * (H / G) > 64;
-    if (D <= 128 && Dv <= 128) { if (nw8) HY_WAM(4, 8, 8); else HY_WAM(4, 8, 4); }
-    else { if (nw8) HY_WAM(8, 16, 8); else HY_WAM(8, 16, 4); }
+    // 128 rows and every SIMD holds two waves; up to 32 or 16 rows 2 or 4 waves share them
+    const int rows = max_q * (H / G);
+#define HY_WAM(NS, NCT)                               \
+    do {                                              \
+        if (rows > 64) HY_WAM_K(NS, NCT, 8, 1);       \
+        else if (rows > 32) HY_WAM_K(NS, NCT, 4, 1);  \
+        else if (rows > 16) HY_WAM_K(NS, NCT, 4, 2);  \
+        else HY_WAM_K(NS, NCT, 4, 4);                 \
+    } while (0)
+    if (D <= 64 && Dv <= 64) HY_WAM(2, 4);
+    else if (D <= 128 && Dv <= 128) HY_WAM(4, 8);
+    else HY_WAM(8, 16);
 #undef HY_WAM
+#undef HY_WAM_K
 #undef HY_WAM_S
     if (nsplit > 1)
         hy::window_combine_kernel<<<(unsigned)((total_rows + 3) / 4), 256, 0, s>>>(part_o, part_ml, sink, gate, out, total_rows, H, Dv, nsplit, vcs, pos, qkv, ldq, g_off, ldo);
