@@ -8,8 +8,9 @@
 //   gate columns: their float copy                                        -> gate [T, H]
 //
 //   conv_prep_vec   up to 4 taps, D = 32, 64, 128 or 256: a thread owns 8 neighbouring columns of one head (16-byte
-//                   loads), D / 8 lanes share a head (the mean of squares is a few shuffles), and walks several consecutive tokens
-//                   with its taps and the last K-1 inputs in registers, so that a projected value is loaded once.
+//                   loads), D / 8 lanes share a head (the mean of squares is a few shuffles), and walks several
+//                   consecutive tokens with its taps and the last K-1 inputs in registers, so that a projected value is
+//                   loaded once.
 //   conv_prep       any other sizes (D <= 256): one wave per head and token.
 //
 // With one token per sequence (decode) the history is rewritten in the same pass: a thread is the only reader and writer of
